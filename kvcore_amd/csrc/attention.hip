@@ -417,8 +417,9 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
                                          int interleaved, const int32_t* kv_slot, int T, int nh,
                                          int nkv, int d, int dv, int page_size, int write_kv,
                                          int dtype, kvc_stream stream) {
-  if (T < 0 || nh <= 0 || nkv <= 0 || d <= 0 || dv <= 0 || page_size <= 0)
+  if (T < 0 || nh <= 0 || nkv < 0 || d <= 0 || dv <= 0 || page_size <= 0)
     return kvc_fail("kvc_qk_norm_rope_kv_write: bad sizes");
+  if (nkv == 0 && write_kv) return kvc_fail("kvc_qk_norm_rope_kv_write: rows without keys have nothing to write");
   if (d > kMaxHeadDim) return kvc_fail("kvc_qk_norm_rope_kv_write: head size above 512");
   if (rot_dim < 0 || rot_dim > d || (rot_dim & 1))
     return kvc_fail("kvc_qk_norm_rope_kv_write: rot_dim must be even and at most the head size");
@@ -437,9 +438,10 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
   // steps of many tokens store the values eight tokens at a time, 16 bytes a store (the planes
   // must be 16-byte aligned for that, which whole pages of 8 tokens and more are)
   bool tiled_values = write_kv && T >= 16 && page_size % 8 == 0;
+  const bool queries_only = !write_kv && nkv == 0 && T >= 16;
   for (int c = 0; c < num_v_planes; ++c)
     tiled_values = tiled_values && (reinterpret_cast<uintptr_t>(host_v_planes[c]) & 15) == 0;
-  if (tiled_values && d <= kWave) {
+  if ((tiled_values || queries_only) && d <= kWave) {
     // many tokens and heads of up to 64 elements: a wave a head, then the values
     const int64_t waves = static_cast<int64_t>(T) * (nh + nkv);
     KVC_DISPATCH_DTYPE(
@@ -449,9 +451,10 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
                            dim3(256), 0, reinterpret_cast<hipStream_t>(stream), static_cast<Tp*>(qkv),
                            row_stride, static_cast<Tp*>(k_cache), q_gain, k_gain, eps, cos_tab, sin_tab,
                            rot_dim, interleaved, kv_slot, T, nh, nkv, d, page_size, write_kv);
-        hipLaunchKernelGGL(value_planes_write_tile_kernel<Tp>, dim3((T + 7) / 8), dim3(256), 0,
-                           reinterpret_cast<hipStream_t>(stream), static_cast<const Tp*>(qkv), row_stride,
-                           planes, v_chunk, kv_slot, T, (nh + nkv) * d, nkv, dv, page_size));
+        if (tiled_values) hipLaunchKernelGGL(
+            value_planes_write_tile_kernel<Tp>, dim3((T + 7) / 8), dim3(256), 0,
+            reinterpret_cast<hipStream_t>(stream), static_cast<const Tp*>(qkv), row_stride,
+            planes, v_chunk, kv_slot, T, (nh + nkv) * d, nkv, dv, page_size));
     return kvc_check_launch("kvc_qk_norm_rope_kv_write");
   }
   if (d > kUsualHeadDim) {

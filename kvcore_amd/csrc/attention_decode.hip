@@ -1,6 +1,7 @@
 // Paged attention for single tokens (decode), bfloat16, on the matrix cores, with the
 // rotation of the token's query and key and the write of its key and value into the cache
-// done by the same kernel.
+// done by the same kernel, where the layer has one behind a norm of every query and key head.
+// Value heads are as wide as the keys or half as wide.
 //
 // One block of W waves per (token, kv head, split of the key range); the waves take the
 // 16-key blocks of the range in turn.  The query heads that share the kv head are the
@@ -8,9 +9,9 @@
 // group, straight from global memory:
 //
 //   S^T[16 keys, 16 heads]  = K[16 keys, d]       * Q^T[d, 16 heads]     (16x16x32)
-//   O^T[d, 16 heads]       += V^T[d, 16 keys]     * P^T[16 keys, 16 heads] (16x16x16)
+//   O^T[dv, 16 heads]      += V^T[dv, 16 keys]    * P^T[16 keys, 16 heads] (16x16x16)
 //
-// K pages are [page_size, d] (d contiguous) and V pages are [d, page_size] (keys
+// K pages are [page_size, d] (d contiguous) and V pages are [dv, page_size] (keys
 // contiguous), which are exactly the A-operand layouts of the two products; the
 // accumulator layout of S^T is the B-operand layout of the second product, so the
 // probabilities never leave registers.  Softmax state (max, sum) is float32, one per
@@ -52,7 +53,7 @@ struct DecodeArgs {
   int out_f32;  // out receives float32 values (the sums as they are) instead of bfloat16
   float* part_o;
   float* part_ml;
-  const bf16_t* qkv;  // rows [nh q heads | nkv k heads | nkv v heads] of d
+  const bf16_t* qkv;  // rows [nh q heads of d | nkv k heads of d | nkv v heads of dv]
   int64_t qkv_stride;
   bf16_t* k_cache;
   bf16_t* v_cache;
@@ -66,6 +67,9 @@ struct DecodeArgs {
   const float* sin_tab;
   int rot_dim;
   int interleaved;
+  const float* q_gain;  // [d] or null: every q head (and the k head, with k_gain) is first divided by
+  const float* k_gain;  // its root mean square, norm_eps inside the root, and multiplied by the gain
+  float norm_eps;
   int write_kv;  // store the token's key and value (and attend to them from LDS)
   int nh, nkv, page_size, num_pages;
   float scale_log2e;
@@ -95,7 +99,8 @@ inline size_t lds_total(int waves, int g, int d, int lds_pages) {
 template <int D>
 constexpr int max_waves() { return D > 128 ? 4 : kMaxWaves; }
 
-template <int D>
+// D: the size of a query and key head; DV: the size of a value head.
+template <int D, int DV>
 __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(const DecodeArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
   const int t = blockIdx.x;
@@ -112,16 +117,16 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
   const int g = nh / nkv;
   const float slope_l2e = (a.slopes != nullptr && col < g) ? a.slopes[hk * g + col] * kLog2e : 0.f;
   const bool head_live = col < g;
-  constexpr int NJ = D / 16;  // output row blocks
+  constexpr int NJ = DV / 16;  // output row blocks
   constexpr int NC = D / 32;  // 32-wide chunks of the head for Q.K
   constexpr int NBUF = 3;     // 16-key blocks a wave holds: one in work, two on their way
 
   bf16_t* sq = reinterpret_cast<bf16_t*>(lds);                       // [g][D + kQPad]
-  bf16_t* sk = reinterpret_cast<bf16_t*>(lds + lds_q_bytes(g, D));   // [D] key, then [D] value
+  bf16_t* sk = reinterpret_cast<bf16_t*>(lds + lds_q_bytes(g, D));   // [D] key, then [DV] value
   bf16_t* sv = sk + D;
   float* sml = reinterpret_cast<float*>(lds + lds_q_bytes(g, D) + lds_kv_bytes(D));  // [waves][16][2]
-  float* so = sml + waves * 32;                                      // [waves][g][D + kOPad]
-  int32_t* spage = reinterpret_cast<int32_t*>(so + static_cast<int64_t>(waves) * g * (D + kOPad));  // [lds_pages]
+  float* so = sml + waves * 32;                                      // [waves][g][DV + kOPad]
+  int32_t* spage = reinterpret_cast<int32_t*>(so + static_cast<int64_t>(waves) * g * (DV + kOPad));  // [lds_pages]
 
   // which row of the block table: one load if the caller resolved it, else two in a chain
   const int pos = __builtin_amdgcn_readfirstlane(a.positions[t]);
@@ -135,8 +140,8 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
   trow_idx = __builtin_amdgcn_readfirstlane(trow_idx);
   if (trow_idx < 0) {  // padding token
     if (nsplit == 1) {
-      for (int idx = tid; idx < g * D; idx += nthreads)
-        store_result(a.out, (static_cast<int64_t>(t) * nh + hk * g) * D + idx, 0.f, a.out_f32);
+      for (int idx = tid; idx < g * DV; idx += nthreads)
+        store_result(a.out, (static_cast<int64_t>(t) * nh + hk * g) * DV + idx, 0.f, a.out_f32);
     } else if (tid < g) {
       float* ml = a.part_ml + ((static_cast<int64_t>(t) * nh + hk * g + tid) * nsplit + split) * 2;
       ml[0] = -INFINITY;
@@ -182,7 +187,7 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
     const bf16_t* krow = real ? a.k_cache + ((static_cast<int64_t>(page) * nkv + hk) * page_size +
                                              sub * 16 + col) * D + 8 * quad
                               : a.k_cache;
-    const bf16_t* vrow = real ? a.v_cache + ((static_cast<int64_t>(page) * nkv + hk) * D + col) * page_size +
+    const bf16_t* vrow = real ? a.v_cache + ((static_cast<int64_t>(page) * nkv + hk) * DV + col) * page_size +
                                     sub * 16 + 4 * quad
                               : a.v_cache;
     const int64_t v_step = real ? static_cast<int64_t>(16) * page_size : 0;
@@ -211,7 +216,7 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
     for (int s = 0; s < NBUF - 1; ++s) okb[s] = issue_block(b_wave + s * waves, first_pages[s], kb[s], vb[s]);
   }
 
-  // ---- rotation of the group's queries (and the key) into LDS; key and value into the cache
+  // ---- norm and rotation of the group's queries (and the key) into LDS; key and value into the cache
   {
     const bf16_t* trow = a.qkv + static_cast<int64_t>(t) * a.qkv_stride;
     const int rot_dim = a.rot_dim, half = rot_dim / 2;
@@ -223,16 +228,33 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
       if (page > 0 && page < a.num_pages) {
         const int off = pos % page_size;
         k_off = ((static_cast<int64_t>(page) * nkv + hk) * page_size + off) * D;
-        v_off = (static_cast<int64_t>(page) * nkv + hk) * D * page_size + off;
+        v_off = (static_cast<int64_t>(page) * nkv + hk) * DV * page_size + off;
       }
     }
     const int n_heads = owner ? g + 1 : g;  // the key is one more head to rotate
+    if (a.q_gain != nullptr) {  // a wave a head: its scale factor, into what will hold the waves' sums
+      for (int hh = wave; hh < n_heads; hh += waves) {
+        const bf16_t* src = (hh < g) ? trow + static_cast<int64_t>(hk * g + hh) * D
+                                     : trow + static_cast<int64_t>(nh + hk) * D;
+        float ss = 0.f;
+        for (int e = lane; e < D; e += 64) {
+          const float x = to_float(src[e]);
+          ss = fmaf(x, x, ss);
+        }
+        ss = wave_sum(ss);
+        if (lane == 0) sml[hh] = 1.f / sqrtf(ss / static_cast<float>(D) + a.norm_eps);
+      }
+      __syncthreads();
+    }
     for (int idx = tid; idx < n_heads * D; idx += nthreads) {
       const int hh = idx / D;
       const int e = idx - hh * D;
       const bf16_t* src = (hh < g) ? trow + static_cast<int64_t>(hk * g + hh) * D
                                    : trow + static_cast<int64_t>(nh + hk) * D;
       bf16_t y = src[e];
+      const float* gain = (hh < g) ? a.q_gain : a.k_gain;
+      const float norm = (gain != nullptr) ? sml[hh] : 1.f;
+      if (gain != nullptr && e >= rot_dim) y = from_float<bf16_t>(to_float(y) * norm * gain[e]);
       if (e < rot_dim) {
         int j, partner;
         bool is_first;
@@ -246,7 +268,11 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
           partner = is_first ? e + half : e - half;
         }
         const float c = cs[j], s_ = sn[j];
-        const float xe = to_float(y), xp = to_float(src[partner]);
+        float xe = to_float(y), xp = to_float(src[partner]);
+        if (gain != nullptr) {
+          xe = xe * norm * gain[e];
+          xp = xp * norm * gain[partner];
+        }
         y = from_float<bf16_t>(is_first ? rotate_first(xe, xp, c, s_) : rotate_second(xp, xe, c, s_));
       }
       if (hh < g) {
@@ -257,8 +283,8 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
       }
     }
     if (owner) {
-      const bf16_t* vsrc = trow + static_cast<int64_t>(nh + nkv + hk) * D;
-      for (int e = tid; e < D; e += nthreads) {
+      const bf16_t* vsrc = trow + static_cast<int64_t>(nh + nkv) * D + static_cast<int64_t>(hk) * DV;
+      for (int e = tid; e < DV; e += nthreads) {
         const bf16_t v = vsrc[e];
         sv[e] = v;
         if (v_off >= 0) a.v_cache[v_off + static_cast<int64_t>(e) * page_size] = v;
@@ -375,7 +401,7 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
   // ---- merge the waves' partials in wave order
   // o[j][i] = O^T[element 16j + 4*quad + i, head col]
   if (head_live) {
-    float* wo = so + (static_cast<int64_t>(wave) * g + col) * (D + kOPad) + 4 * quad;
+    float* wo = so + (static_cast<int64_t>(wave) * g + col) * (DV + kOPad) + 4 * quad;
 #pragma unroll
     for (int j = 0; j < NJ; ++j) *reinterpret_cast<f32x4_t*>(wo + 16 * j) = o[j];
     if (quad == 0) {
@@ -384,9 +410,9 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
     }
   }
   __syncthreads();
-  for (int idx = tid; idx < g * D; idx += nthreads) {
-    const int h = idx / D;
-    const int e = idx - h * D;
+  for (int idx = tid; idx < g * DV; idx += nthreads) {
+    const int h = idx / DV;
+    const int e = idx - h * DV;
     // the sink counts once for a row: the first split takes it, as one more partial sum without values
     const float sink_l2e = (a.sinks != nullptr && split == 0) ? a.sinks[hk * g + h] * kLog2e : -INFINITY;
     float mmax = sink_l2e;
@@ -397,14 +423,14 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
       const float wgt = __builtin_amdgcn_exp2f(sml[(w * 16 + h) * 2] - m_safe);
       if (wgt > 0.f) {
         denom += wgt * sml[(w * 16 + h) * 2 + 1];
-        acc += wgt * so[(static_cast<int64_t>(w) * g + h) * (D + kOPad) + e];
+        acc += wgt * so[(static_cast<int64_t>(w) * g + h) * (DV + kOPad) + e];
       }
     }
     const int64_t th = static_cast<int64_t>(t) * nh + hk * g + h;
     if (nsplit == 1) {
-      store_result(a.out, th * D + e, denom > 0.f ? acc / denom : 0.f, a.out_f32);
+      store_result(a.out, th * DV + e, denom > 0.f ? acc / denom : 0.f, a.out_f32);
     } else {
-      a.part_o[(th * nsplit + split) * D + e] = acc;
+      a.part_o[(th * nsplit + split) * DV + e] = acc;
       if (e == 0) {
         a.part_ml[(th * nsplit + split) * 2] = mmax;
         a.part_ml[(th * nsplit + split) * 2 + 1] = denom;
@@ -457,7 +483,7 @@ int decode_waves(int g, int d) {
   return waves;
 }
 
-template <int D>
+template <int D, int DV>
 int launch_decode(DecodeArgs& args, int T, hipStream_t stream) {
   const int g = args.nh / args.nkv;
   // a split's range of pages always fits: the table's width cut into nsplit parts, and slack
@@ -470,11 +496,11 @@ int launch_decode(DecodeArgs& args, int T, hipStream_t stream) {
   if (lds_total(waves, g, D, args.lds_pages) > kLdsLimit)
     return kvc_fail("kvc_decode_attention: the block table is wider than kvc_decode_attention_max_table "
                     "allows for one split");
-  hipLaunchKernelGGL(decode_attention_kernel<D>, dim3(T, args.nkv, args.nsplit), dim3(waves * 64),
+  hipLaunchKernelGGL((decode_attention_kernel<D, DV>), dim3(T, args.nkv, args.nsplit), dim3(waves * 64),
                      lds_total(waves, g, D, args.lds_pages), stream, args);
   if (args.nsplit > 1)
-    hipLaunchKernelGGL(decode_combine_kernel, dim3(T * args.nh), dim3((D + 63) / 64 * 64), 0, stream,
-                       args.out, args.part_o, args.part_ml, D, args.nsplit, args.out_f32);
+    hipLaunchKernelGGL(decode_combine_kernel, dim3(T * args.nh), dim3((DV + 63) / 64 * 64), 0, stream,
+                       args.out, args.part_o, args.part_ml, DV, args.nsplit, args.out_f32);
   return kvc_check_launch("kvc_decode_attention");
 }
 
@@ -490,8 +516,9 @@ int kvc::launch_attention_combine(bf16_t* out, const float* part_o, const float*
   return kvc_check_launch("attention combine");
 }
 
-extern "C" int kvc_decode_attention_supported(int nh, int nkv, int d, int page_size, int dtype) {
+extern "C" int kvc_decode_attention_supported(int nh, int nkv, int d, int dv, int page_size, int dtype) {
   if (dtype != 1) return 0;
+  if (dv != d && 2 * dv != d) return 0;
   if (nkv <= 0 || nh % nkv || nh / nkv > 16) return 0;
   if (page_size % 16) return 0;
   return d == 32 || d == 64 || d == 96 || d == 128 || d == 160 || d == 192 || d == 224 || d == 256;
@@ -515,16 +542,17 @@ extern "C" int kvc_decode_attention(void* out, void* part_o, void* part_ml, cons
                                     const int32_t* table, int table_stride,
                                     const int32_t* positions, const int32_t* token_req,
                                     const int32_t* slots, const int32_t* token_rows,
-                                    const float* cos_tab, const float* sin_tab, int rot_dim, int interleaved, int write_kv, int T, int nh,
-                                    int nkv, int d, int page_size, int num_pages, float scale,
+                                    const float* cos_tab, const float* sin_tab, int rot_dim, int interleaved,
+                                    const float* q_gain, const float* k_gain, float norm_eps, int write_kv, int T, int nh,
+                                    int nkv, int d, int dv, int page_size, int num_pages, float scale,
                                     int window, const float* slopes, int chunk, const float* sinks,
                                     int nsplit, int out_f32, kvc_stream stream) {
-  if (!kvc_decode_attention_supported(nh, nkv, d, page_size, 1))
+  if (!kvc_decode_attention_supported(nh, nkv, d, dv, page_size, 1))
     return kvc_fail("kvc_decode_attention: unsupported shape (bfloat16, head size a multiple of 32 "
-                    "up to 256, at most 16 query heads per kv head, page size a multiple of 16)");
+                    "up to 256, values as wide or half as wide, at most 16 query heads per kv head, page size a multiple of 16)");
   if (T < 0 || nsplit < 1 || nsplit > kMaxSplits || nkv > 65535 || table_stride <= 0 || num_pages <= 0)
     return kvc_fail("kvc_decode_attention: bad sizes (at most 64 splits)");
-  if (qkv_stride % 8 || qkv_stride < static_cast<int64_t>(nh + (write_kv ? 2 * nkv : 0)) * d)
+  if (qkv_stride % 8 || qkv_stride < static_cast<int64_t>(nh) * d + (write_kv ? static_cast<int64_t>(nkv) * (d + dv) : 0))
     return kvc_fail("kvc_decode_attention: token rows must be 16-byte aligned and hold q (and k, v)");
   if (rot_dim < 0 || rot_dim > d || rot_dim % 2)
     return kvc_fail("kvc_decode_attention: the rotated width must be even and at most the head size");
@@ -532,6 +560,8 @@ extern "C" int kvc_decode_attention(void* out, void* part_o, void* part_ml, cons
     return kvc_fail("kvc_decode_attention: rotation needs its cos and sin tables");
   if (nsplit > 1 && (part_o == nullptr || part_ml == nullptr))
     return kvc_fail("kvc_decode_attention: splits need a workspace");
+  if ((k_gain != nullptr && q_gain == nullptr) || (q_gain != nullptr && k_gain == nullptr && write_kv))
+    return kvc_fail("kvc_decode_attention: a norm of the heads has gains for the queries and for the keys it writes");
   if (T == 0) return 0;
   DecodeArgs args;
   args.out = static_cast<bf16_t*>(out);
@@ -552,6 +582,9 @@ extern "C" int kvc_decode_attention(void* out, void* part_o, void* part_ml, cons
   args.sin_tab = sin_tab;
   args.rot_dim = rot_dim;
   args.interleaved = interleaved;
+  args.q_gain = q_gain;
+  args.k_gain = k_gain;
+  args.norm_eps = norm_eps;
   args.write_kv = write_kv;
   args.nh = nh;
   args.nkv = nkv;
@@ -565,15 +598,18 @@ extern "C" int kvc_decode_attention(void* out, void* part_o, void* part_ml, cons
   args.nsplit = nsplit;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   kvc_note_variant(kVariantDecodeAttention, nsplit > 1 ? "decode_attention_kernel with splits" : "decode_attention_kernel");
+#define KVC_DECODE(D_) \
+  case D_: return dv == d ? launch_decode<D_, D_>(args, T, s) : launch_decode<D_, D_ / 2>(args, T, s)
   switch (d) {
-    case 32: return launch_decode<32>(args, T, s);
-    case 64: return launch_decode<64>(args, T, s);
-    case 96: return launch_decode<96>(args, T, s);
-    case 128: return launch_decode<128>(args, T, s);
-    case 160: return launch_decode<160>(args, T, s);
-    case 192: return launch_decode<192>(args, T, s);
-    case 224: return launch_decode<224>(args, T, s);
-    case 256: return launch_decode<256>(args, T, s);
+    KVC_DECODE(32);
+    KVC_DECODE(64);
+    KVC_DECODE(96);
+    KVC_DECODE(128);
+    KVC_DECODE(160);
+    KVC_DECODE(192);
+    KVC_DECODE(224);
+    KVC_DECODE(256);
   }
+#undef KVC_DECODE
   return kvc_fail("kvc_decode_attention: unsupported head size");
 }

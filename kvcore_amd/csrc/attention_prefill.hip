@@ -9,7 +9,9 @@
 // pages ([d, key]) regrouped so that operand reads are contiguous.  Per wave:
 //
 //   S^T[16 keys, 16 rows]  = K[16 keys, d]   * Q^T[d, 16 rows]        (16x16x32, per key block)
-//   O^T[d, 16 rows]       += V^T[d, 32 keys] * P^T[32 keys, 16 rows]  (16x16x32, per two key blocks)
+//   O^T[dv, 16 rows]      += V^T[dv, 32 keys] * P^T[32 keys, 16 rows] (16x16x32, per two key blocks)
+//
+// with value heads as wide as the keys or half as wide.
 //
 // A lane's four accumulator values of S^T for key blocks a and b are the eight values of
 // the B operand of the second product, if the product's k index 8*quad + e stands for key
@@ -70,14 +72,15 @@ __device__ __forceinline__ float quad_sum(float v) {
 }
 
 // KB: 16-key blocks per LDS tile
-template <int D, int KB>
+template <int D, int DV, int KB>
 constexpr int tile_bytes() {
-  return KB * 16 * (D + 16) * 2 + KB * D * 16 * 2;  // K rows padded, then V
+  return KB * 16 * (D + 16) * 2 + KB * DV * 16 * 2;  // K rows padded, then V
 }
 
 // W: waves of a block (4 or 8).  Eight waves stage each key tile for twice the rows, which
 // halves the block's loads and LDS writes per row; a compute unit then holds one block.
-template <int D, int CT, int KB, int W>
+// D: the size of a query and key head; DV: the size of a value head.
+template <int D, int DV, int CT, int KB, int W>
 __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ q, int64_t q_stride,
     const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
@@ -89,13 +92,13 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
     const float* __restrict__ cos_tab, const float* __restrict__ sin_tab, int rot_dim, int interleaved,
     int out_f32) {
   constexpr int kKeyBlocks = KB;
-  constexpr int NJ = D / 16;
+  constexpr int NJ = DV / 16;
   constexpr int NC = D / 32;
   // padded K row in LDS (elements): with 32 bytes of padding the operand reads (16 rows x 4
   // pieces of 16 bytes a wave) meet no bank conflict; with 16 they took 1.45 times as long
   constexpr int KROW = D + 16;
   constexpr int K_ELEMS = kKeyBlocks * 16 * KROW;
-  constexpr int TILE_ELEMS = tile_bytes<D, KB>() / 2;
+  constexpr int TILE_ELEMS = tile_bytes<D, DV, KB>() / 2;
   extern __shared__ __attribute__((aligned(16))) bf16_t tiles[];  // two tiles: [K | V] each
 
   const int g = nh / nkv;
@@ -272,7 +275,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
   const int kb_first = first_lo / 16;
   const int kb_end = pos_hi / 16 + 1;
   constexpr int K_CHUNKS = kKeyBlocks * 16 * (D / 8);  // 16-byte pieces of a K tile
-  constexpr int V_CHUNKS = kKeyBlocks * D * 2;         // 16-byte pieces of a V tile
+  constexpr int V_CHUNKS = kKeyBlocks * DV * 2;        // 16-byte pieces of a V tile
   constexpr int THREADS = W * 64;
   constexpr int K_PER_THREAD = K_CHUNKS / THREADS;
   constexpr int V_PER_THREAD = V_CHUNKS / THREADS;
@@ -281,13 +284,13 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
   // Fetch the tile that starts at key block kb0 into registers.  Keys beyond the request's
   // last position, key blocks beyond the range and pages that are gone arrive as zeros.
   // The key blocks that a thread fetches from are the same for its whole wave (K: 16 rows of
-  // 16-byte pieces are 128 or 256 threads; V: a key block takes 2 * D threads), so a wave looks
+  // 16-byte pieces are 128 or 256 threads; V: a key block takes 2 * DV threads), so a wave looks
   // up the pages of its own key blocks only, as scalars.
   constexpr int PIECES = D / 8;                    // 16-byte pieces of a K row
   constexpr int ROWS_PER_STEP = THREADS / PIECES;  // K rows that the block fetches per step
   // V: a key block's rows of the head times its two halves of 8 keys take V_THREADS threads;
   // the block's threads form V_GROUPS such groups, each with an even number of key blocks
-  constexpr int V_THREADS = 2 * D;
+  constexpr int V_THREADS = 2 * DV;
   constexpr int V_GROUPS = THREADS / V_THREADS;
   static_assert(THREADS % V_THREADS == 0 && kKeyBlocks % (2 * V_GROUPS) == 0 &&
                     V_PER_THREAD == kKeyBlocks / V_GROUPS && (kKeyBlocks * 16) % ROWS_PER_STEP == 0 &&
@@ -317,8 +320,10 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
   // kernel.)
   const int sub_mask = blocks_per_page - 1;
   const int sub_shift = (blocks_per_page & sub_mask) == 0 ? __builtin_ctz(blocks_per_page) : -1;
-  const int64_t page_elems = static_cast<int64_t>(nkv) * page_size * D;  // of one plane
+  const int64_t page_elems = static_cast<int64_t>(nkv) * page_size * D;  // of the keys' plane
   const int64_t head_elems = static_cast<int64_t>(hk) * page_size * D;
+  const int64_t v_page_elems = static_cast<int64_t>(nkv) * page_size * DV;
+  const int64_t v_head_elems = static_cast<int64_t>(hk) * page_size * DV;
   const int lk_lane = lane & 15;
   int lk_page = 0, lk_sub = 0;
   auto lookup_issue = [&](int kb0) {
@@ -341,7 +346,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
     const bool ok = lk_sub >= 0 && lk_page > 0 && lk_page < num_pages;
     const int64_t at = lk_page * page_elems + head_elems;
     const int64_t k_at = ok ? at + lk_sub * (16 * D) : -1;
-    const int64_t v_at = ok ? at + lk_sub * 16 : -1;
+    const int64_t v_at = ok ? lk_page * v_page_elems + v_head_elems + lk_sub * 16 : -1;
     auto pick = [&](int64_t v, int from) -> int64_t {
       const uint32_t lo = __builtin_amdgcn_readlane(static_cast<int>(static_cast<uint64_t>(v) & 0xffffffffu), from);
       const uint32_t hi = __builtin_amdgcn_readlane(static_cast<int>(static_cast<uint64_t>(v) >> 32), from);
@@ -468,7 +473,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
     // with registers to spare the first value operands are asked for now: they do not depend
     // on the softmax
     constexpr bool kEarlyValues = CT == 1;
-    constexpr int GJ = NJ / (2 * CT);  // operand reads a group
+    constexpr int GJ = NJ / (2 * CT) > 0 ? NJ / (2 * CT) : 1;  // operand reads a group
     constexpr int NG = NJ / GJ;        // groups a pair of key blocks
     static_assert(GJ > 0 && NJ % GJ == 0,
                   "a head size whose column groups do not divide into whole read groups would "
@@ -624,7 +629,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
       // sums relative to m, and m in the exponent's units, as the combining kernel expects
       const int64_t slot =
           (static_cast<int64_t>(my_tok[ct]) * nh + my_head[ct]) * gridDim.z + blockIdx.z;
-      float* po = part_o + slot * D + 4 * quad;
+      float* po = part_o + slot * DV + 4 * quad;
 #pragma unroll
       for (int j = 0; j < NJ; ++j) *reinterpret_cast<f32x4_t*>(po + 16 * j) = o_acc[ct][j];
       if (quad == 0) {
@@ -634,7 +639,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
       continue;
     }
     const float inv = (l_row > 0.f) ? 1.f / l_row : 0.f;
-    const int64_t at = (static_cast<int64_t>(my_tok[ct]) * nh + my_head[ct]) * D + 4 * quad;
+    const int64_t at = (static_cast<int64_t>(my_tok[ct]) * nh + my_head[ct]) * DV + 4 * quad;
     if (out_f32) {  // the sums as they are, for a consumer that joins them before anything is rounded
       float* op = reinterpret_cast<float*>(out) + at;
 #pragma unroll
@@ -652,7 +657,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
   }  // turn
 }
 
-template <int D, int CT, int W>
+template <int D, int DV, int CT, int W>
 int launch_prefill_ct(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t* k_cache,
                       const bf16_t* v_cache, const int32_t* table, int table_stride,
                       const int32_t* positions, const int32_t* q_start, const int32_t* slots, int T,
@@ -669,10 +674,12 @@ int launch_prefill_ct(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16
   // unit's LDS to itself and takes tiles of 128 keys: half the barriers and page lookups per key
   // (16,384 tokens 2.52 against 2.39 ms), and on heads of 64 a thread then still stages whole
   // pairs of key blocks
-  constexpr int KB = (W == 8) ? 8 : 4;
-  constexpr int lds_bytes = 2 * tile_bytes<D, KB>();
+  // Values of 32: the threads of a block stage four key blocks' values at once, so a tile holds
+  // eight key blocks for every thread to stage a pair.
+  constexpr int KB = (W == 8 || DV < 64) ? 8 : 4;
+  constexpr int lds_bytes = 2 * tile_bytes<D, DV, KB>();
   static const hipError_t attr = hipFuncSetAttribute(
-      reinterpret_cast<const void*>(&prefill_attention_kernel<D, CT, KB, W>),
+      reinterpret_cast<const void*>(&prefill_attention_kernel<D, DV, CT, KB, W>),
       hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);
   if (attr != hipSuccess) return kvc_fail("kvc_prefill_attention: the kernel's LDS size was refused");
   // see the kernel on how block ids map to (kv head, pair)
@@ -683,16 +690,16 @@ int launch_prefill_ct(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16
   snprintf(variant, sizeof(variant), "prefill_attention_kernel<%d,%d,%d,%d>%s x%d", D, CT, KB, W,
            single ? " one tile a block" : "", nsplit);
   kvc_note_variant(kVariantPrefillAttention, variant);
-  hipLaunchKernelGGL((prefill_attention_kernel<D, CT, KB, W>), dim3(static_cast<unsigned>(wide), 1, nsplit), dim3(W * 64),
+  hipLaunchKernelGGL((prefill_attention_kernel<D, DV, CT, KB, W>), dim3(static_cast<unsigned>(wide), 1, nsplit), dim3(W * 64),
                      lds_bytes, stream, out, q, q_stride, k_cache, v_cache, table, table_stride, positions,
                      q_start, slots, R, nh, nkv, page_size, num_pages, scale * kLog2e, window, slopes, chunk,
                      sinks, part_o, part_ml, single, cos_tab, sin_tab, rot_dim, interleaved, out_f32);
   if (nsplit > 1)
-    return launch_attention_combine(out, part_o, part_ml, static_cast<int64_t>(T) * nh, D, nsplit, out_f32, stream);
+    return launch_attention_combine(out, part_o, part_ml, static_cast<int64_t>(T) * nh, DV, nsplit, out_f32, stream);
   return kvc_check_launch("kvc_prefill_attention");
 }
 
-template <int D>
+template <int D, int DV>
 int launch_prefill(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t* k_cache,
                    const bf16_t* v_cache, const int32_t* table, int table_stride,
                    const int32_t* positions, const int32_t* q_start, const int32_t* slots, int T,
@@ -752,15 +759,18 @@ int launch_prefill(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t*
     single = mode[1] == 's';
     waves = (mode[1] && mode[2] == '8') ? 8 : 4;
   }
+  if (DV < 64) waves = 4;  // eight waves would stage the values of more key blocks than a tile has
   if (g > 16 * waves * ct) return kvc_fail("kvc_prefill_attention: too many query heads per kv head");
 #define KVC_LAUNCH_PREFILL(CT_, W_)                                                                      \
-  return launch_prefill_ct<D, CT_, W_>(out, q, q_stride, k_cache, v_cache, table, table_stride, positions, \
+  return launch_prefill_ct<D, DV, CT_, W_>(out, q, q_stride, k_cache, v_cache, table, table_stride, positions, \
                                        q_start, slots, T, R, nh, nkv, page_size, num_pages, scale, window, \
                                        slopes, chunk, sinks, part_o, part_ml, nsplit, single, cos_tab, sin_tab, rot_dim,     \
                                        interleaved, out_f32, stream)
-  if (waves == 8) {
-    if (ct == 2) KVC_LAUNCH_PREFILL(2, 8);
-    KVC_LAUNCH_PREFILL(1, 8);
+  if constexpr (DV >= 64) {
+    if (waves == 8) {
+      if (ct == 2) KVC_LAUNCH_PREFILL(2, 8);
+      KVC_LAUNCH_PREFILL(1, 8);
+    }
   }
   if (ct == 2) KVC_LAUNCH_PREFILL(2, 4);
   KVC_LAUNCH_PREFILL(1, 4);
@@ -769,8 +779,9 @@ int launch_prefill(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t*
 
 }  // namespace
 
-extern "C" int kvc_prefill_attention_supported(int nh, int nkv, int d, int page_size, int dtype) {
+extern "C" int kvc_prefill_attention_supported(int nh, int nkv, int d, int dv, int page_size, int dtype) {
   if (dtype != 1) return 0;
+  if (dv != d && 2 * dv != d) return 0;
   if (nkv <= 0 || nh % nkv || nh / nkv > 64) return 0;
   if (page_size % 16) return 0;
   return d == 64 || d == 128;
@@ -780,14 +791,14 @@ extern "C" int kvc_prefill_attention(void* out, const void* q, int64_t q_stride,
                                      const void* k_cache, const void* v_cache,
                                      const int32_t* table, int table_stride,
                                      const int32_t* positions, const int32_t* q_start,
-                                     const int32_t* slots, int T, int R, int nh, int nkv, int d,
+                                     const int32_t* slots, int T, int R, int nh, int nkv, int d, int dv,
                                      int page_size, int num_pages, float scale, int window,
                                      const float* slopes, int chunk, const float* sinks, void* part_o, void* part_ml, int nsplit, const float* cos_tab,
                                      const float* sin_tab, int rot_dim, int interleaved, int out_f32,
                                      kvc_stream stream) {
-  if (!kvc_prefill_attention_supported(nh, nkv, d, page_size, 1))
-    return kvc_fail("kvc_prefill_attention: unsupported shape (bfloat16, head size 64 or 128, at "
-                    "most 64 query heads per kv head, page size a multiple of 16)");
+  if (!kvc_prefill_attention_supported(nh, nkv, d, dv, page_size, 1))
+    return kvc_fail("kvc_prefill_attention: unsupported shape (bfloat16, head size 64 or 128, values as "
+                    "wide or half as wide, at most 64 query heads per kv head, page size a multiple of 16)");
   if (T < 0 || R <= 0 || nkv > 65535 || table_stride <= 0 || num_pages <= 0)
     return kvc_fail("kvc_prefill_attention: bad sizes");
   if (!(scale > 0.f)) return kvc_fail("kvc_prefill_attention: the scale must be positive");
@@ -809,12 +820,15 @@ extern "C" int kvc_prefill_attention(void* out, const void* q, int64_t q_stride,
   const bf16_t* qq = static_cast<const bf16_t*>(q);
   const bf16_t* kc = static_cast<const bf16_t*>(k_cache);
   const bf16_t* vc = static_cast<const bf16_t*>(v_cache);
-  if (d == 64)
-    return launch_prefill<64>(static_cast<bf16_t*>(out), qq, q_stride, kc, vc, table, table_stride,
-                              positions, q_start, slots, T, R, nh, nkv, page_size, num_pages, scale,
-                              window, slopes, chunk, sinks, po, pml, nsplit, cos_tab, sin_tab, rot_dim, interleaved, out_f32, s);
-  return launch_prefill<128>(static_cast<bf16_t*>(out), qq, q_stride, kc, vc, table, table_stride,
-                             positions, q_start, slots, T, R, nh, nkv, page_size, num_pages, scale,
-                             window, slopes, chunk, sinks, po, pml, nsplit, cos_tab, sin_tab, rot_dim, interleaved,
-                             out_f32, s);
+#define KVC_PREFILL(D_, DV_)                                                                                      \
+  return launch_prefill<D_, DV_>(static_cast<bf16_t*>(out), qq, q_stride, kc, vc, table, table_stride, positions, \
+                                 q_start, slots, T, R, nh, nkv, page_size, num_pages, scale, window, slopes, chunk, \
+                                 sinks, po, pml, nsplit, cos_tab, sin_tab, rot_dim, interleaved, out_f32, s)
+  if (d == 64) {
+    if (dv == d) KVC_PREFILL(64, 64);
+    KVC_PREFILL(64, 32);
+  }
+  if (dv == d) KVC_PREFILL(128, 128);
+  KVC_PREFILL(128, 64);
+#undef KVC_PREFILL
 }

@@ -48,13 +48,28 @@ __device__ __forceinline__ float rotate_second(float x0, float x1, float c, floa
   return __builtin_fmaf(x0, s, x1 * c);
 }
 
-// The activation of a gated feed-forward's gate: kGateSilu g * sigmoid(g), kGateGeluTanh the tanh
-// form of gelu, 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))).
+// min(g, limit) * sigmoid(alpha * min(g, limit)) * (clamp(u, -limit, limit) + shift)
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float shift) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.f + expf(-alpha * g)) * (u + shift);
+}
+
+// How a gated feed-forward joins its two branches: kGateSilu g * sigmoid(g) * u, kGateGeluTanh the
+// tanh form of gelu, 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))) * u, kGateClamped as above (the
+// three constants belong to it alone).
 constexpr int kGateSilu = 0;
 constexpr int kGateGeluTanh = 1;
-__device__ __forceinline__ float gate_act(float g, int act) {
-  if (act == kGateGeluTanh) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-  return g / (1.f + expf(-g));
+constexpr int kGateClamped = 2;
+struct GateRule {
+  int act;
+  float limit, alpha, shift;
+};
+__device__ __forceinline__ float gate_join(float g, float u, const GateRule& rule) {
+  if (rule.act == kGateClamped) return clamped_glu(g, u, rule.limit, rule.alpha, rule.shift);
+  if (rule.act == kGateGeluTanh)
+    return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
+  return g / (1.f + expf(-g)) * u;
 }
 
 __device__ __forceinline__ float wave_sum(float v) {

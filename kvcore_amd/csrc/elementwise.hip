@@ -90,6 +90,60 @@ extern "C" int kvc_embed(float* residual, const void* table, const int32_t* ids,
   return kvc_check_launch("kvc_embed");
 }
 
+// A token's row and the row of the pair (token before, token), a block a token.  The token before the
+// first one of a request's tokens in this step is the request's own, kept in its slot between steps; the
+// block of that first token reads it and, when all its threads have, leaves the last token of the
+// request's tokens there for the next step (nobody else touches the slot).
+template <typename T>
+__global__ void embed_pairs_kernel(float* __restrict__ residual, const T* __restrict__ table,
+                                   const T* __restrict__ pairs, const int32_t* __restrict__ ids,
+                                   int32_t* __restrict__ last, const int32_t* __restrict__ positions,
+                                   const int32_t* __restrict__ token_req, const int32_t* __restrict__ q_start,
+                                   const int32_t* __restrict__ slots, int H, int V, int64_t buckets,
+                                   int64_t mul_prev, int64_t mul_cur) {
+  const int t = blockIdx.x;
+  const int id = ids[t];
+  float* out = residual + static_cast<int64_t>(t) * H;
+  const int req = token_req[t];
+  if (req < 0) {  // a padding token: any row will do
+    for (int i = threadIdx.x; i < H; i += blockDim.x) out[i] = 0.f;
+    return;
+  }
+  const bool first = t == q_start[req];
+  int prev = 0;
+  int64_t pair = buckets;  // the first token of a sequence has a row of its own
+  if (positions[t] != 0) {
+    prev = first ? last[slots[req]] : ids[t - 1];
+    pair = (prev * mul_prev + id * mul_cur) % buckets;
+  }
+  if (first) {
+    __syncthreads();  // every thread has read the slot
+    if (threadIdx.x == 0) last[slots[req]] = ids[q_start[req + 1] - 1];
+  }
+  if (id < 0 || id >= V || prev < 0 || prev >= V) {
+    for (int i = threadIdx.x; i < H; i += blockDim.x) out[i] = __uint_as_float(0x7fc00000u);
+    return;
+  }
+  const T* a = table + static_cast<int64_t>(id) * H;
+  const T* b = pairs + pair * H;
+  for (int i = threadIdx.x; i < H; i += blockDim.x) out[i] = to_float(a[i]) + to_float(b[i]);
+}
+
+extern "C" int kvc_embed_pairs(float* residual, const void* table, const void* pairs, const int32_t* ids,
+                               int32_t* last, const int32_t* positions, const int32_t* token_req,
+                               const int32_t* q_start, const int32_t* slots, int T, int H, int V,
+                               int64_t buckets, int64_t mul_prev, int64_t mul_cur, int dtype, kvc_stream stream) {
+  if (T < 0 || H <= 0 || V <= 0 || buckets <= 0) return kvc_fail("kvc_embed_pairs: bad sizes");
+  if (mul_prev < 0 || mul_prev >= buckets || mul_cur < 0 || mul_cur >= buckets || buckets > 0x7fffffff)
+    return kvc_fail("kvc_embed_pairs: the multipliers must be reduced modulo the buckets");
+  if (T == 0) return 0;
+  KVC_DISPATCH_DTYPE(dtype, Tp,
+                     hipLaunchKernelGGL(embed_pairs_kernel<Tp>, dim3(T), dim3(256), 0, S(stream), residual,
+                                        static_cast<const Tp*>(table), static_cast<const Tp*>(pairs), ids, last,
+                                        positions, token_req, q_start, slots, H, V, buckets, mul_prev, mul_cur));
+  return kvc_check_launch("kvc_embed_pairs");
+}
+
 // ------------------------------------------------------------- logits after the head
 // x = logits + bias; x = cap * tanh(x / cap) when cap > 0; x *= scale.
 template <typename TB>
@@ -442,7 +496,7 @@ extern "C" int kvc_residual_add2(float* residual, const void* a, int a_dtype, co
 
 template <typename T>
 __global__ void silu_mul_kernel(T* __restrict__ out, const T* __restrict__ gate_up, int I,
-                                int64_t n, int act) {
+                                int64_t n, GateRule rule) {
   const int64_t idx = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (idx >= n) return;
   const int64_t t = idx / I;
@@ -450,12 +504,12 @@ __global__ void silu_mul_kernel(T* __restrict__ out, const T* __restrict__ gate_
   const T* row = gate_up + t * 2 * I;
   const float g = to_float(row[i]);
   const float u = to_float(row[I + i]);
-  out[idx] = from_float<T>(gate_act(g, act) * u);
+  out[idx] = from_float<T>(gate_join(g, u, rule));
 }
 
 template <typename T>
 __global__ void silu_mul_vec_kernel(T* __restrict__ out, const T* __restrict__ gate_up, int I8,
-                                    int64_t n8, int act) {
+                                    int64_t n8, GateRule rule) {
   const int64_t idx = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (idx >= n8) return;
   const int64_t t = idx / I8;
@@ -465,19 +519,20 @@ __global__ void silu_mul_vec_kernel(T* __restrict__ out, const T* __restrict__ g
   load8(gate_up + t * 2 * I + i, g);
   load8(gate_up + t * 2 * I + I + i, u);
 #pragma unroll
-  for (int e = 0; e < 8; ++e) y[e] = gate_act(g[e], act) * u[e];
+  for (int e = 0; e < 8; ++e) y[e] = gate_join(g[e], u[e], rule);
   store8(out + t * I + i, y);
 }
 
 extern "C" int kvc_silu_mul(void* out, const void* gate_up, int T, int I, int dtype,
                             kvc_stream stream) {
-  return kvc_gate_mul(out, gate_up, T, I, kGateSilu, dtype, stream);
+  return kvc_gate_mul(out, gate_up, T, I, kGateSilu, 0.f, 0.f, 0.f, dtype, stream);
 }
 
-extern "C" int kvc_gate_mul(void* out, const void* gate_up, int T, int I, int act, int dtype,
-                            kvc_stream stream) {
+extern "C" int kvc_gate_mul(void* out, const void* gate_up, int T, int I, int act, float limit, float alpha,
+                            float up_shift, int dtype, kvc_stream stream) {
   if (T < 0 || I <= 0) return kvc_fail("kvc_gate_mul: bad sizes");
-  if (act != kGateSilu && act != kGateGeluTanh) return kvc_fail("kvc_gate_mul: unknown activation");
+  if (act != kGateSilu && act != kGateGeluTanh && act != kGateClamped) return kvc_fail("kvc_gate_mul: unknown activation");
+  const GateRule rule{act, limit, alpha, up_shift};
   const int64_t n = static_cast<int64_t>(T) * I;
   if (n == 0) return 0;
   if (I % 8 == 0 && (reinterpret_cast<uintptr_t>(out) % 16) == 0 &&
@@ -487,14 +542,14 @@ extern "C" int kvc_gate_mul(void* out, const void* gate_up, int T, int I, int ac
     KVC_DISPATCH_DTYPE(dtype, Tp,
                        hipLaunchKernelGGL(silu_mul_vec_kernel<Tp>, dim3(vblocks), dim3(256), 0,
                                           S(stream), static_cast<Tp*>(out),
-                                          static_cast<const Tp*>(gate_up), I / 8, n8, act));
+                                          static_cast<const Tp*>(gate_up), I / 8, n8, rule));
     return kvc_check_launch("kvc_gate_mul");
   }
   const unsigned blocks = static_cast<unsigned>((n + 255) / 256);
   KVC_DISPATCH_DTYPE(dtype, Tp,
                      hipLaunchKernelGGL(silu_mul_kernel<Tp>, dim3(blocks), dim3(256), 0, S(stream),
                                         static_cast<Tp*>(out), static_cast<const Tp*>(gate_up), I,
-                                        n, act));
+                                        n, rule));
   return kvc_check_launch("kvc_gate_mul");
 }
 

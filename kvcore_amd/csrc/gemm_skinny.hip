@@ -42,7 +42,7 @@ struct SkinnyExtras {
   int64_t ldr;
   const float* gain;
   float* out_ss;
-  int act;  // the gate's activation in the gated form (kGateSilu, kGateGeluTanh)
+  GateRule rule;  // how the gated form joins its two branches
   int out_act;  // the plain form: 0 stores the product (+ bias); 1 stores the square of its relu, the
                 // product rounded to bfloat16 first as if it had been stored and read again
 };
@@ -320,7 +320,7 @@ __global__ __launch_bounds__(MAXW * 64) void gemm_skinny_kernel(OutT* __restrict
       for (int i = 0; i < 4; ++i) {
         const float gv = to_float(from_float<bf16_t>(acc[0][nt][i] * row_scale[nt] + bg[i]));
         const float uv = to_float(from_float<bf16_t>(acc[1][nt][i] * row_scale[nt] + bu[i]));
-        y[i] = gate_act(gv, ex.act) * uv;
+        y[i] = gate_join(gv, uv, ex.rule);
       }
       store4<OutT>(C + static_cast<int64_t>(tok) * ldc + n_first, y, n_left);
     }
@@ -526,7 +526,7 @@ int check_operands(const char* who, const void* A, const void* W, int M, int N, 
   return 0;
 }
 
-const SkinnyExtras kNoExtras = {nullptr, 0, 1.f, 0.f, nullptr, 0, nullptr, nullptr, kGateSilu, 0};
+const SkinnyExtras kNoExtras = {nullptr, 0, 1.f, 0.f, nullptr, 0, nullptr, nullptr, {kGateSilu, 0.f, 0.f, 0.f}, 0};
 
 }  // namespace
 
@@ -607,7 +607,7 @@ extern "C" int kvc_gemm_skinny_blocks(int N, int K, int gated, int packed) {
 
 extern "C" int kvc_gemm_skinny_fused_bf16(void* C, const void* A, const void* W, const void* bias,
                                           int M, int N, int K, int64_t lda, int64_t ldc, int gated,
-                                          const float* in_ss, int in_parts, int in_width,
+                                          float limit, float alpha, float up_shift, const float* in_ss, int in_parts, int in_width,
                                           float in_eps, float* residual, int64_t ldr,
                                           const float* gain, float* out_ss, int packed,
                                           kvc_stream stream) {
@@ -620,9 +620,10 @@ extern "C" int kvc_gemm_skinny_fused_bf16(void* C, const void* A, const void* W,
     return kvc_fail("kvc_gemm_skinny_fused_bf16: the residual form needs gain and out_ss, rows of "
                     "at least N, and is not gated");
   if (M == 0) return 0;
-  if (gated < 0 || gated > 2) return kvc_fail("kvc_gemm_skinny_fused_bf16: gated is 0, 1 (silu) or 2 (gelu, tanh form)");
+  if (gated < 0 || gated > 3)
+    return kvc_fail("kvc_gemm_skinny_fused_bf16: gated is 0, 1 (silu), 2 (gelu, tanh form) or 3 (clamped)");
   SkinnyExtras ex = {in_ss, in_parts, static_cast<float>(in_width), in_eps,
-                     residual, ldr, gain, out_ss, gated == 2 ? kGateGeluTanh : kGateSilu};
+                     residual, ldr, gain, out_ss, {gated > 0 ? gated - 1 : kGateSilu, limit, alpha, up_shift}, 0};
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   if (gated)
     return dispatch_gated(static_cast<bf16_t*>(C), static_cast<const bf16_t*>(A),

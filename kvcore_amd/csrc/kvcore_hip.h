@@ -82,9 +82,12 @@ int kvc_residual_add2(float* residual, const void* a, int a_dtype, const void* b
 
 // out[t, i] = silu(gate_up[t, i]) * gate_up[t, I + i].
 int kvc_silu_mul(void* out, const void* gate_up, int T, int I, int dtype, kvc_stream stream);
-// out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i]; act 0: silu, 1: gelu in its tanh form,
-// 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3))).
-int kvc_gate_mul(void* out, const void* gate_up, int T, int I, int act, int dtype, kvc_stream stream);
+// The two branches g = gate_up[t, i] and u = gate_up[t, I + i] of a gated feed-forward joined into
+// out[t, i]; act 0: silu(g) * u, 1: gelu in its tanh form, 0.5 g (1 + tanh(sqrt(2 / pi) (g + 0.044715 g^3)))
+// * u, 2: clamped, g' * sigmoid(alpha * g') * (clamp(u, -limit, limit) + up_shift) with g' = min(g, limit)
+// (limit, alpha and up_shift belong to this one alone, here and in the products below).
+int kvc_gate_mul(void* out, const void* gate_up, int T, int I, int act, float limit, float alpha, float up_shift,
+                 int dtype, kvc_stream stream);
 
 // out = act(x) elementwise over n values (in place is fine); act 0: the square of relu.
 int kvc_activation(void* out, const void* x, int64_t n, int act, int dtype, kvc_stream stream);
@@ -136,6 +139,16 @@ int kvc_paged_attention(void* out, const void* q, int64_t q_stride, const void* 
                         int num_pages, float scale, int window, const float* slopes, int chunk,
                         const float* sinks, int out_f32, int dtype, kvc_stream stream);
 
+// residual[t, :] = float(table[ids[t], :]) + float(pairs[row, :]): row = buckets for the token at position
+// 0, else (prev * mul_prev + ids[t] * mul_cur) mod buckets with prev the token before it, ids[t - 1] or,
+// for the first of a request's tokens in this step, last[slots[req]]; the request's last token is left
+// there for its next step.  pairs [buckets + 1, H]; mul_prev and mul_cur already modulo buckets.  A token
+// outside [0, V) on either place gives a NaN row, a padding token (token_req < 0) zeros.
+int kvc_embed_pairs(float* residual, const void* table, const void* pairs, const int32_t* ids, int32_t* last,
+                    const int32_t* positions, const int32_t* token_req, const int32_t* q_start,
+                    const int32_t* slots, int T, int H, int V, int64_t buckets, int64_t mul_prev,
+                    int64_t mul_cur, int dtype, kvc_stream stream);
+
 // What kvc_rope_kv_write does, for heads whose keys (d) and values (dv) may differ in size,
 // with a norm of every q and k head before the rotation: rows of qkv are [nh q heads of d |
 // nkv k heads of d | nkv v heads of dv], row_stride elements apart.  With q_gain and k_gain
@@ -146,6 +159,7 @@ int kvc_paged_attention(void* out, const void* q, int64_t q_stride, const void* 
 // num_v_planes (1 to 4) planes of dv / num_v_planes elements a head each (host_v_planes: a host
 // array of their device pointers): element i of a value head then lies in plane i / (dv /
 // num_v_planes), so that kernels whose keys and values are of one size can serve a plane each.
+// nkv 0 (without write_kv): the rows hold queries alone, for a layer that reads another's cache.
 int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_cache,
                               void* const* host_v_planes, int num_v_planes, const float* q_gain, const float* k_gain, float eps,
                               const float* cos_tab, const float* sin_tab, int rot_dim,
@@ -271,20 +285,23 @@ int kvc_head_rmsnorm_gate(void* out, int out_dtype, const float* o, const void* 
 // x row sorted[i] / in_div (in_div 0: row i itself) and writes out row i (out_sorted) or
 // sorted[i].  dtype is that of x and w.  packed: w is the copy kvc_pack_weight makes of the whole
 // stacked matrix (bfloat16, N a multiple of 16, K of 64).
-// score_fn 0: softmax over the experts, 1: sigmoid of each logit.  correction [E] (or null) is added
-// to the scores for the choice alone.  group_best 1 or 2: a group is worth its best choice score, or
+// bias [E] (or null) joins the logits.  score_fn 0: softmax over the experts, 1: sigmoid of each logit,
+// 2: the logit itself, the weights then being the softmax over the chosen logits.  correction [E] (or
+// null) is added to the scores for the choice alone.  group_best 1 or 2: a group is worth its best choice score, or
 // the sum of its best two.  The weights are multiplied by weight_scale.
 int kvc_moe_route(int32_t* choice, float* weight, const float* logits, int T, int E, int top,
-                  int groups, int keep, int score_fn, const float* correction, int group_best,
-                  float weight_scale, kvc_stream stream);
+                  int groups, int keep, int score_fn, const float* bias, const float* correction,
+                  int group_best, float weight_scale, kvc_stream stream);
 // Tiles hold up to tile_rows rows, 16 or 64 (kvc_moe_tile_rows says which a step's size asks
 // for; 64 is for bfloat16 with K a multiple of 32).
 int kvc_moe_tile_rows(int pairs, int E);
 // The router's logits (x [T, H] of x_dtype times router [E, H] float32, float32 sums in one fixed order)
-// and the choice of kvc_moe_route in one kernel.
+// and the choice of kvc_moe_route in one kernel.  With gate [T] (may be null) the matrix is [E + 1, H]
+// and gate[t] = sigmoid(x[t] . its last row).
 int kvc_moe_router(int32_t* choice, float* weight, const void* x, int64_t x_stride, int x_dtype,
-                   const float* router, int T, int H, int E, int top, int groups, int keep, int score_fn,
-                   const float* correction, int group_best, float weight_scale, kvc_stream stream);
+                   const float* router, float* gate, int T, int H, int E, int top, int groups, int keep,
+                   int score_fn, const float* bias, const float* correction, int group_best, float weight_scale,
+                   kvc_stream stream);
 int kvc_moe_max_tiles(int pairs, int E, int tile_rows);
 int kvc_moe_align(int32_t* sorted, int32_t* tiles, int32_t* num_tiles, const int32_t* choice,
                   int pairs, int E, int max_tiles, int tile_rows, kvc_stream stream);
@@ -293,18 +310,17 @@ int kvc_moe_gemm(void* out, int64_t out_stride, int out_dtype, const void* x, in
                  const int32_t* num_tiles, int max_tiles, int tile_rows, int N, int K, int in_div, int out_sorted,
                  int gated, float limit, float alpha, float up_shift, int packed, kvc_stream stream);
 // out[t] = sum_c weight[t, c] * y[t * top + c] + add0[t] + add1[t] (either may be null; add0 of
-// dtype add0_dtype, add1 float32), float32.
+// dtype add0_dtype, add1 float32), float32.  add1_gate [T] (or null): add1[t] is multiplied by it.
 // accumulate: the sum is added into out instead of stored.
 int kvc_moe_combine(float* out, const float* y, const float* weight, int top, const void* add0,
-                    int add0_dtype, const float* add1, int T, int H, int accumulate, kvc_stream stream);
-// out[t, i] = g * sigmoid(alpha * g) * (u + 1), g = min(gate_up[t, i], limit),
-// u = clamp(gate_up[t, I + i], -limit, limit).
-int kvc_clamped_glu(void* out, const void* gate_up, int T, int I, float limit, float alpha, int dtype,
+                    int add0_dtype, const float* add1, const float* add1_gate, int T, int H, int accumulate,
                     kvc_stream stream);
 
 // The same attention for bfloat16 steps of single tokens on the matrix cores, a block of
 // several waves per (token, kv head, split), which also does what kvc_rope_kv_write does for
-// its token: qkv rows are [nh q heads | nkv k heads | nkv v heads]; the first rot_dim elements
+// its token: qkv rows are [nh q heads of d | nkv k heads of d | nkv v heads of dv], dv d or d / 2 (out
+// [T, nh * dv], part_o likewise); with q_gain and k_gain ([d], or null) every head is normed as
+// kvc_qk_norm_rope_kv_write does; the first rot_dim elements
 // of every q head (and of the k head) are rotated by cos/sin [T, rot_dim / 2] on the way in
 // (rot_dim 0: taken as they are) and qkv itself is left unchanged; with write_kv the
 // token's key and value are stored in their cache slot and attended to (without write_kv
@@ -321,15 +337,16 @@ int kvc_clamped_glu(void* out, const void* gate_up, int T, int I, float limit, f
 // they are built.
 // slopes, sinks (float32 [nh] or null) and chunk as for kvc_paged_attention; the kernel for portions
 // (kvc_prefill_attention) takes them too.
-int kvc_decode_attention_supported(int nh, int nkv, int d, int page_size, int dtype);
+int kvc_decode_attention_supported(int nh, int nkv, int d, int dv, int page_size, int dtype);
 int kvc_decode_attention_waves(int nh, int nkv, int d);
 int kvc_decode_attention_max_table(int nh, int nkv, int d);
 int kvc_decode_attention(void* out, void* part_o, void* part_ml, const void* qkv,
                          int64_t qkv_stride, void* k_cache, void* v_cache, const int32_t* table,
                          int table_stride, const int32_t* positions, const int32_t* token_req,
                          const int32_t* slots, const int32_t* token_rows, const float* cos_tab,
-                         const float* sin_tab, int rot_dim, int interleaved, int write_kv, int T,
-                         int nh, int nkv, int d, int page_size, int num_pages, float scale,
+                         const float* sin_tab, int rot_dim, int interleaved, const float* q_gain,
+                         const float* k_gain, float norm_eps, int write_kv, int T,
+                         int nh, int nkv, int d, int dv, int page_size, int num_pages, float scale,
                          int window, const float* slopes, int chunk, const float* sinks, int nsplit,
                          int out_f32, kvc_stream stream);
 
@@ -338,15 +355,15 @@ int kvc_decode_attention(void* out, void* part_o, void* part_ml, const void* qkv
 // each request's tokens in the flattened batch; slots [R] names its block-table row;
 // positions must rise by one along a request's tokens.  With nsplit > 1 the keys of every
 // tile are dealt to that many blocks (for few query rows against many keys) and a second
-// kernel joins their results; part_o [T*nh*nsplit, d] and part_ml [T*nh*nsplit, 2] float32
+// kernel joins their results; values have dv elements, d or d / 2; part_o [T*nh*nsplit, dv] and part_ml [T*nh*nsplit, 2] float32
 // are its workspace.  With cos_tab and sin_tab [T, rot_dim / 2] the queries come unrotated
 // and are rotated on their way in, as kvc_rope_kv_write would have (rot_dim a multiple of 64,
 // or of 32 when interleaved); without, they are taken as they are.
-int kvc_prefill_attention_supported(int nh, int nkv, int d, int page_size, int dtype);
+int kvc_prefill_attention_supported(int nh, int nkv, int d, int dv, int page_size, int dtype);
 int kvc_prefill_attention(void* out, const void* q, int64_t q_stride, const void* k_cache,
                           const void* v_cache, const int32_t* table, int table_stride,
                           const int32_t* positions, const int32_t* q_start, const int32_t* slots,
-                          int T, int R, int nh, int nkv, int d, int page_size, int num_pages,
+                          int T, int R, int nh, int nkv, int d, int dv, int page_size, int num_pages,
                           float scale, int window, const float* slopes, int chunk, const float* sinks, void* part_o,
                           void* part_ml, int nsplit,
                           const float* cos_tab, const float* sin_tab, int rot_dim, int interleaved,
@@ -358,10 +375,14 @@ int kvc_prefill_attention(void* out, const void* q, int64_t q_stride, const void
 // behind a sublayer, the sum into the float32 stream and the norm before the next sublayer in one
 // pass.  delta is float32 (delta_dtype 0) or bfloat16 (1); out likewise (out_dtype).  slices > 1:
 // delta holds [slices, T, H] float32 partial sums of a product cut along K (kvc_gemm_mid_bf16 mode
-// 2) and a row of the result is their sum in slice order.
+// 2) and a row of the result is their sum in slice order.  weight [T, slices] (or null): delta instead
+// holds [T, slices, H] float32, the results of a token's experts, and a row of the result is their sum
+// in order, each times its weight, plus add[t] (float32 [T, H], or null) times add_gate[t] ([T], or null:
+// once): what kvc_moe_combine stores, added up on the way.
 int kvc_norm_add_norm(void* out, int out_dtype, float* residual, const void* delta, int delta_dtype,
                       const float* post_gain, float eps, const float* next_gain, float next_eps,
-                      int T, int H, int slices, kvc_stream stream);
+                      int T, int H, int slices, const float* weight, const float* add, const float* add_gate,
+                      kvc_stream stream);
 // Rows of attn are [heads][2][dv]: out[t, h] = (a1 - lambda * a2) / sqrt(mean((a1 - lambda * a2)^2) + eps)
 // * post over the head's dv values, out [T, heads * dv] of dtype; attn of attn_dtype (dtype, or float32);
 // float32 arithmetic.
@@ -403,15 +424,15 @@ int kvc_gemm_f32(float* C, const float* A, const float* W, const float* bias, in
 // The same product for 17 to 192 rows, where the waves of a block share the rows of A through
 // LDS (K a multiple of 512).  mode 0: C = A W^T (+ bias), float32 (out_dtype 0) or bfloat16
 // (1).  mode 1: C[M, N] = silu(A Wg^T + bg) * (A Wu^T + bu) in bfloat16, W [2N, K] holding Wg
-// then Wu (mode 4: the same with the tanh form of gelu for silu).  mode 2: narrow outputs are cut along K into kvc_gemm_mid_slices(N, K) slices and
+// then Wu (mode 4: the same with the tanh form of gelu for silu; mode 5: joined as kvc_gate_mul's act 2).  mode 2: narrow outputs are cut along K into kvc_gemm_mid_slices(N, K) slices and
 // only their float32 partial sums are stored, partial [slices, M, N] (no bias); the kernel
 // that consumes them adds them up in slice order.  mode 3: as mode 0, but cut along K like
 // mode 2 when `partial` is given, with a second kernel that sums the slices.  With `packed` W
 // is what kvc_pack_weight made of the matrix (the same sums, read in contiguous kilobytes).
 int kvc_gemm_mid_slices(int N, int K);
 int kvc_gemm_mid_bf16(void* C, void* partial, const void* A, const void* W, const void* bias, int M,
-                      int N, int K, int64_t lda, int64_t ldc, int out_dtype, int mode, int packed,
-                      kvc_stream stream);
+                      int N, int K, int64_t lda, int64_t ldc, int out_dtype, int mode, float limit, float alpha,
+                      float up_shift, int packed, kvc_stream stream);
 
 // C[M, N] = A[M, K] * W[N, K]^T (+ bias[N]) for M <= 64 rows of bfloat16 on the matrix
 // cores, float32 sums, weights streamed once; C is float32 (out_dtype 0) or bfloat16 (1).
@@ -451,12 +472,13 @@ int kvc_gemm_skinny_silu_mul_bf16(void* C, const void* A, const void* W, const v
 //    receives bfloat16(residual * gain[n]) and out_ss [M, blocks] the new residual's sums of
 //    squares per block of columns, blocks = kvc_gemm_skinny_blocks(N, K, 0, packed): the in_ss of the
 //    product that consumes C.
-// gated = 1 is kvc_gemm_skinny_silu_mul_bf16's product (N = the gate's rows).
+// gated = 1 is kvc_gemm_skinny_silu_mul_bf16's product (N = the gate's rows); 2 and 3 join the branches
+// as kvc_gate_mul's act 1 and 2.
 int kvc_gemm_skinny_blocks(int N, int K, int gated, int packed);
 int kvc_gemm_skinny_fused_bf16(void* C, const void* A, const void* W, const void* bias, int M, int N,
-                               int K, int64_t lda, int64_t ldc, int gated, const float* in_ss,
-                               int in_parts, int in_width, float in_eps, float* residual,
-                               int64_t ldr, const float* gain, float* out_ss, int packed,
+                               int K, int64_t lda, int64_t ldc, int gated, float limit, float alpha,
+                               float up_shift, const float* in_ss, int in_parts, int in_width, float in_eps,
+                               float* residual, int64_t ldr, const float* gain, float* out_ss, int packed,
                                kvc_stream stream);
 
 // table[triples[3i], triples[3i+1]] = triples[3i+2] for i < n.

@@ -5,13 +5,16 @@
 // tokens x choices, tiles <= pairs / 16 + experts), so a step neither waits for the routing nor
 // changes its launches with it: a captured step replays for any routing.
 //
-//   kvc_moe_route    scores = softmax(logits) or sigmoid(logits) in float32; the choice is made on the
-//                    scores plus an optional correction per expert: the `keep` groups that are worth
-//                    most (a group's best choice score, or the sum of its best two); the `top` best
-//                    experts of those groups (the lower index on a tie); weights = the chosen experts'
-//                    plain scores / (their sum + 1e-20) * weight_scale.  A wave a token.
+//   kvc_moe_route    scores = softmax(logits), sigmoid(logits) or the logits themselves in float32 (an
+//                    optional bias per expert joins the logits); the choice is made on the scores plus
+//                    an optional correction per expert: the `keep` groups that are worth most (a
+//                    group's best choice score, or the sum of its best two); the `top` best experts of
+//                    those groups (the lower index on a tie); weights = the chosen experts' plain
+//                    scores / (their sum + 1e-20) * weight_scale, or, where the scores are the logits,
+//                    the softmax over the chosen logits * weight_scale.  A wave a token.
 //   kvc_moe_router   the router's product (float32 sums in one fixed order over rows of either dtype)
-//                    and the choice in one kernel.
+//                    and the choice in one kernel; a further row of the router's matrix may give one
+//                    number a token, a sigmoid gate for an expert that every token runs.
 //   kvc_moe_align    pairs sorted by expert: sorted[i] = pair index (token * top + choice), and a
 //                    list of tiles of up to 16 (or 64) sorted rows that belong to one expert each.
 //   kvc_moe_gemm     for every tile, rows x that expert's matrix.  Gated: gate and up rows of the
@@ -21,9 +24,9 @@
 //                    bfloat16 operands go through the matrix cores (16 x 16 x 32, the expert's rows as
 //                    the A operand, the tokens as B) with float32 sums; float32 operands, and rows
 //                    that 16-byte loads do not divide, are summed in float32 in index order.  A row's sums do not depend on which tile it is in.
-//   kvc_moe_combine  out[t] = sum_c weight[t, c] * y[t * top + c] (+ up to two more row sets),
-//                    float32, in the order of the choices; or added into out (the residual stream).
-//   kvc_clamped_glu  the same activation for a feed-forward that every token runs.
+//   kvc_moe_combine  out[t] = sum_c weight[t, c] * y[t * top + c] (+ up to two more row sets, the second
+//                    times a number a token where one is given), float32, in the order of the
+//                    choices; or added into out (the residual stream).
 
 #include <hip/hip_runtime.h>
 
@@ -40,12 +43,6 @@ namespace {
 constexpr int kTileRows = 16;
 constexpr int kBigTileRows = 64;
 
-__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float shift) {
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g / (1.f + expf(-alpha * g)) * (u + shift);
-}
-
 // the lane that holds the largest value (the lowest index among equals) tells everyone
 __device__ __forceinline__ void wave_argmax(float& val, int& idx) {
 #pragma unroll
@@ -59,14 +56,16 @@ __device__ __forceinline__ void wave_argmax(float& val, int& idx) {
   }
 }
 
-// How a token's experts are chosen from its logits.  score_fn 0: softmax over the experts, 1: a
-// sigmoid of each logit.  The choice is made on score + correction[e] (correction may be null) and
-// may so be negative; the weights are the plain scores of the chosen, over their sum (+ 1e-20),
-// times weight_scale.  With keep < groups only the experts of the best `keep` of `groups` equal
+// How a token's experts are chosen from its logits (+ bias[e], which may be null).  score_fn 0: softmax
+// over the experts, 1: a sigmoid of each logit, 2: the logit itself.  The choice is made on score +
+// correction[e] (correction may be null) and may so be negative; the weights are the plain scores of
+// the chosen, over their sum (+ 1e-20), or (2) the softmax over the chosen logits, times weight_scale.
+// With keep < groups only the experts of the best `keep` of `groups` equal
 // groups of neighbours may be chosen; a group is worth the sum of its `group_best` (1 or 2) largest
 // choice scores.  The lower index wins a tie.
 struct RouteRule {
   int top, groups, keep, score_fn, group_best;
+  const float* bias;
   const float* correction;
   float weight_scale;
 };
@@ -76,21 +75,24 @@ struct RouteRule {
 __device__ __forceinline__ void route_one(int32_t* __restrict__ choice, float* __restrict__ weight, const float* z,
                                           float* sc, float* pk, float* gs, int lane, int E, const RouteRule& rule) {
   const int top = rule.top, groups = rule.groups, keep = rule.keep;
+  auto logit = [&](int e) -> float { return rule.bias != nullptr ? z[e] + rule.bias[e] : z[e]; };
   if (rule.score_fn == 0) {
     float mx = -INFINITY;
-    for (int e = lane; e < E; e += kWave) mx = fmaxf(mx, z[e]);
+    for (int e = lane; e < E; e += kWave) mx = fmaxf(mx, logit(e));
     mx = wave_max(mx);
     float sum = 0.f;
     for (int e = lane; e < E; e += kWave) {
-      const float p = expf(z[e] - mx);
+      const float p = expf(logit(e) - mx);
       sc[e] = p;
       sum += p;
     }
     sum = wave_sum(sum);
     const float inv = 1.f / sum;
     for (int e = lane; e < E; e += kWave) sc[e] *= inv;
+  } else if (rule.score_fn == 1) {
+    for (int e = lane; e < E; e += kWave) sc[e] = 1.f / (1.f + expf(-logit(e)));
   } else {
-    for (int e = lane; e < E; e += kWave) sc[e] = 1.f / (1.f + expf(-z[e]));
+    for (int e = lane; e < E; e += kWave) sc[e] = logit(e);
   }
   for (int e = lane; e < E; e += kWave) pk[e] = sc[e] + (rule.correction != nullptr ? rule.correction[e] : 0.f);
   __builtin_amdgcn_wave_barrier();
@@ -132,6 +134,7 @@ __device__ __forceinline__ void route_one(int32_t* __restrict__ choice, float* _
   float total = 0.f;
   float mine = 0.f;  // lane c keeps the c-th choice's score
   int mine_idx = 0;
+  bool mine_ok = false;
   for (int c = 0; c < top; ++c) {
     float val = -INFINITY;
     int idx = 0x7fffffff;
@@ -150,12 +153,18 @@ __device__ __forceinline__ void route_one(int32_t* __restrict__ choice, float* _
     if (lane == c) {
       mine = plain;
       mine_idx = idx;
+      mine_ok = val != -INFINITY;
     }
     __builtin_amdgcn_wave_barrier();
     if (lane == 0) pk[idx] = -INFINITY;
     __builtin_amdgcn_wave_barrier();
   }
-  const float norm = rule.weight_scale / (total + 1e-20f);
+  float norm = rule.weight_scale / (total + 1e-20f);
+  if (rule.score_fn == 2) {  // the softmax over the chosen logits alone
+    const float mx = wave_max(mine_ok ? mine : -INFINITY);
+    mine = mine_ok ? expf(mine - mx) : 0.f;
+    norm = rule.weight_scale / wave_sum(mine);
+  }
   if (lane < top) {
     choice[lane] = mine_idx;
     weight[lane] = mine * norm;
@@ -179,21 +188,23 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int32_t* __restrict__ ch
 // w sums the products of the values 4 l .. 4 l + 3 of the pieces of 256 that are the wave's (every
 // fourth piece) for each of up to 32 experts at a time (a fetched piece of the router's row meets all
 // TOK tokens); the 256 partial sums of a logit are added in wave and lane order through LDS: one
-// fixed order, whatever the batch.  The first wave then chooses.
+// fixed order, whatever the batch.  The first wave then chooses.  With `gate` the matrix has a row
+// behind the experts', whose product's sigmoid goes to gate[t].
 template <typename T, int TOK>
 __global__ __launch_bounds__(256) void moe_router_kernel(int32_t* __restrict__ choice, float* __restrict__ weight,
                                                          const T* __restrict__ x, int64_t x_stride,
-                                                         const float* __restrict__ wr, int T_, int H, int E,
-                                                         RouteRule rule, int vectors) {
+                                                         const float* __restrict__ wr, float* __restrict__ gate,
+                                                         int T_, int H, int E, RouteRule rule, int vectors) {
   constexpr int EB = 32, PR = EB + 1;
   extern __shared__ float lds[];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
   float* part = lds;                       // [256][EB + 1]
-  float* z = lds + 256 * PR;               // [TOK][2 E + groups]
-  const int zrow = 2 * E + rule.groups;
+  float* z = lds + 256 * PR;               // [TOK][rows + E + groups]
+  const int rows = gate != nullptr ? E + 1 : E;
+  const int zrow = rows + E + rule.groups;
   const int t0 = blockIdx.x * TOK;
-  for (int e0 = 0; e0 < E; e0 += EB) {
-    const int ne = (E - e0 < EB) ? E - e0 : EB;
+  for (int e0 = 0; e0 < rows; e0 += EB) {
+    const int ne = (rows - e0 < EB) ? rows - e0 : EB;
     float acc[TOK][EB];
 #pragma unroll
     for (int j = 0; j < TOK; ++j)
@@ -212,7 +223,7 @@ __global__ __launch_bounds__(256) void moe_router_kernel(int32_t* __restrict__ c
       float wv[EB][4];
 #pragma unroll
       for (int e = 0; e < EB; ++e) {
-        const float* wp = wr + static_cast<int64_t>(e < ne ? e0 + e : E - 1) * H + k;
+        const float* wp = wr + static_cast<int64_t>(e < ne ? e0 + e : rows - 1) * H + k;
         if (vectors) {
           const float4 v4 = *reinterpret_cast<const float4*>(wp);
           wv[e][0] = v4.x; wv[e][1] = v4.y; wv[e][2] = v4.z; wv[e][3] = v4.w;
@@ -247,8 +258,9 @@ __global__ __launch_bounds__(256) void moe_router_kernel(int32_t* __restrict__ c
     const int t = t0 + j;
     if (t >= T_) break;  // the whole wave
     float* zr = z + j * zrow;
-    route_one(choice + static_cast<int64_t>(t) * rule.top, weight + static_cast<int64_t>(t) * rule.top, zr, zr, zr + E,
-              zr + 2 * E, lane, E, rule);
+    if (gate != nullptr && lane == 0) gate[t] = 1.f / (1.f + expf(-zr[E]));
+    route_one(choice + static_cast<int64_t>(t) * rule.top, weight + static_cast<int64_t>(t) * rule.top, zr, zr,
+              zr + rows, zr + rows + E, lane, E, rule);
   }
 }
 
@@ -557,7 +569,8 @@ template <typename TA>
 __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ out, const float* __restrict__ y,
                                                           const float* __restrict__ weight, int top,
                                                           const TA* __restrict__ add0, const float* __restrict__ add1,
-                                                          int T, int H, int accumulate) {
+                                                          const float* __restrict__ add1_gate, int T, int H,
+                                                          int accumulate) {
   const int64_t idx = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (idx >= static_cast<int64_t>(T) * H) return;
   const int t = static_cast<int>(idx / H), c = static_cast<int>(idx - static_cast<int64_t>(t) * H);
@@ -565,31 +578,21 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ ou
   for (int j = 0; j < top; ++j)
     acc = fmaf(weight[static_cast<int64_t>(t) * top + j], y[(static_cast<int64_t>(t) * top + j) * H + c], acc);
   if (add0 != nullptr) acc += to_float(add0[idx]);
-  if (add1 != nullptr) acc += add1[idx];
+  if (add1 != nullptr) acc = add1_gate != nullptr ? fmaf(add1_gate[t], add1[idx], acc) : acc + add1[idx];
   out[idx] = accumulate ? out[idx] + acc : acc;
-}
-
-template <typename T>
-__global__ __launch_bounds__(256) void clamped_glu_kernel(T* __restrict__ out, const T* __restrict__ gate_up,
-                                                          int64_t n, int I, float limit, float alpha, float shift) {
-  const int64_t idx = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
-  if (idx >= n) return;
-  const int64_t t = idx / I, i = idx - t * I;
-  const T* row = gate_up + t * 2 * I;
-  out[idx] = from_float<T>(clamped_glu(to_float(row[i]), to_float(row[I + i]), limit, alpha, shift));
 }
 
 }  // namespace
 
 extern "C" int kvc_moe_route(int32_t* choice, float* weight, const float* logits, int T, int E, int top,
-                             int groups, int keep, int score_fn, const float* correction, int group_best,
-                             float weight_scale, kvc_stream stream) {
+                             int groups, int keep, int score_fn, const float* bias, const float* correction,
+                             int group_best, float weight_scale, kvc_stream stream) {
   if (T < 0 || E <= 0 || top <= 0 || top > E || top > kWave || groups <= 0 || E % groups || keep <= 0 ||
       keep > groups)
     return kvc_fail("kvc_moe_route: bad sizes (at most 64 choices; the experts in equal groups)");
-  if ((score_fn != 0 && score_fn != 1) || (group_best != 1 && group_best != 2))
-    return kvc_fail("kvc_moe_route: scores by softmax (0) or sigmoid (1); a group is worth its best 1 or 2");
-  const RouteRule rule{top, groups, keep, score_fn, group_best, correction, weight_scale};
+  if (score_fn < 0 || score_fn > 2 || (group_best != 1 && group_best != 2))
+    return kvc_fail("kvc_moe_route: scores by softmax (0), sigmoid (1) or logit (2); a group is worth its best 1 or 2");
+  const RouteRule rule{top, groups, keep, score_fn, group_best, bias, correction, weight_scale};
   const size_t lds = sizeof(float) * 4 * (2 * E + groups);
   if (lds > 60000) return kvc_fail("kvc_moe_route: too many experts for a wave's scores in LDS");
   if (T == 0) return 0;
@@ -599,20 +602,20 @@ extern "C" int kvc_moe_route(int32_t* choice, float* weight, const float* logits
 }
 
 extern "C" int kvc_moe_router(int32_t* choice, float* weight, const void* x, int64_t x_stride, int x_dtype,
-                              const float* router, int T, int H, int E, int top, int groups, int keep,
-                              int score_fn, const float* correction, int group_best, float weight_scale,
-                              kvc_stream stream) {
+                              const float* router, float* gate, int T, int H, int E, int top, int groups, int keep,
+                              int score_fn, const float* bias, const float* correction, int group_best,
+                              float weight_scale, kvc_stream stream) {
   if (T < 0 || H <= 0 || E <= 0 || top <= 0 || top > E || top > kWave || groups <= 0 || E % groups || keep <= 0 ||
       keep > groups || x_stride < H)
     return kvc_fail("kvc_moe_router: bad sizes (at most 64 choices; the experts in equal groups)");
-  if ((score_fn != 0 && score_fn != 1) || (group_best != 1 && group_best != 2))
-    return kvc_fail("kvc_moe_router: scores by softmax (0) or sigmoid (1); a group is worth its best 1 or 2");
-  const RouteRule rule{top, groups, keep, score_fn, group_best, correction, weight_scale};
+  if (score_fn < 0 || score_fn > 2 || (group_best != 1 && group_best != 2))
+    return kvc_fail("kvc_moe_router: scores by softmax (0), sigmoid (1) or logit (2); a group is worth its best 1 or 2");
+  const RouteRule rule{top, groups, keep, score_fn, group_best, bias, correction, weight_scale};
   if (T == 0) return 0;
   // four tokens a block where the blocks then still fill the chip several times over, else one
   const bool big = T >= 4 * 8 * kvc_device_compute_units();
   const int TOK = big ? 4 : 1;
-  const size_t lds = sizeof(float) * (static_cast<size_t>(256) * 33 + static_cast<size_t>(TOK) * (2 * E + groups));
+  const size_t lds = sizeof(float) * (static_cast<size_t>(256) * 33 + static_cast<size_t>(TOK) * (2 * E + 1 + groups));
   if (lds > 160 * 1024) return kvc_fail("kvc_moe_router: too many experts for a block's LDS");
   const dim3 grid((T + TOK - 1) / TOK);
   // 16-byte loads of the router's rows where the rows allow
@@ -625,7 +628,7 @@ extern "C" int kvc_moe_router(int32_t* choice, float* weight, const void* x, int
       if (attr != hipSuccess) return kvc_fail("kvc_moe_router: the kernel's LDS size was refused");            \
     }                                                                                                           \
     hipLaunchKernelGGL((moe_router_kernel<Tp, TOK_>), grid, dim3(256), lds, S(stream), choice, weight,          \
-                       static_cast<const Tp*>(x), x_stride, router, T, H, E, rule, vectors);             \
+                       static_cast<const Tp*>(x), x_stride, router, gate, T, H, E, rule, vectors);             \
   } while (0)
   if (x_dtype == 1 && big) KVC_ROUTER(bf16_t, 4);
   else if (x_dtype == 1) KVC_ROUTER(bf16_t, 1);
@@ -724,30 +727,18 @@ extern "C" int kvc_moe_gemm(void* out, int64_t out_stride, int out_dtype, const 
 }
 
 extern "C" int kvc_moe_combine(float* out, const float* y, const float* weight, int top, const void* add0,
-                               int add0_dtype, const float* add1, int T, int H, int accumulate,
-                               kvc_stream stream) {
+                               int add0_dtype, const float* add1, const float* add1_gate, int T, int H,
+                               int accumulate, kvc_stream stream) {
   if (T < 0 || H <= 0 || top < 0) return kvc_fail("kvc_moe_combine: bad sizes");
   if (T == 0) return 0;
   const int64_t n = static_cast<int64_t>(T) * H;
   const dim3 grid(static_cast<unsigned>((n + 255) / 256));
   if (add0_dtype == 1) {
     hipLaunchKernelGGL((moe_combine_kernel<bf16_t>), grid, dim3(256), 0, S(stream), out, y, weight, top,
-                       static_cast<const bf16_t*>(add0), add1, T, H, accumulate);
+                       static_cast<const bf16_t*>(add0), add1, add1_gate, T, H, accumulate);
   } else {
     hipLaunchKernelGGL((moe_combine_kernel<float>), grid, dim3(256), 0, S(stream), out, y, weight, top,
-                       static_cast<const float*>(add0), add1, T, H, accumulate);
+                       static_cast<const float*>(add0), add1, add1_gate, T, H, accumulate);
   }
   return kvc_check_launch("kvc_moe_combine");
-}
-
-extern "C" int kvc_clamped_glu(void* out, const void* gate_up, int T, int I, float limit, float alpha, int dtype,
-                               kvc_stream stream) {
-  if (T < 0 || I <= 0) return kvc_fail("kvc_clamped_glu: bad sizes");
-  if (T == 0) return 0;
-  const int64_t n = static_cast<int64_t>(T) * I;
-  const dim3 grid(static_cast<unsigned>((n + 255) / 256));
-  KVC_DISPATCH_DTYPE(dtype, Tp,
-                     hipLaunchKernelGGL((clamped_glu_kernel<Tp>), grid, dim3(256), 0, S(stream),
-                                        static_cast<Tp*>(out), static_cast<const Tp*>(gate_up), n, I, limit, alpha, 1.f));
-  return kvc_check_launch("kvc_clamped_glu");
 }

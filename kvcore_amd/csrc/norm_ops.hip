@@ -48,22 +48,60 @@ __device__ __forceinline__ void st8(bf16_t* p, const float* v) {
   *reinterpret_cast<uint4*>(p) = a;
 }
 
-// A chunk of 8 values of a sublayer's result: the value itself, or, where the product before left
-// partial sums of slices along K ([slices, T, H] float32), their sum in slice order.
+// Where a row of a sublayer's result comes from.  Plain: the row itself, or, where the product before
+// left partial sums of slices along K ([slices, T, H] float32), their sum in slice order.  Weighted
+// (`weight` is not null): the results of a token's experts ([T, slices, H] float32), each times its
+// weight, and a further row times a number a token.
+struct SumRule {
+  int slices;
+  int64_t row_stride, slice_stride;
+  const float* weight;    // [T, slices]
+  const float* add;       // [T, H] or null
+  const float* add_gate;  // [T] or null (one)
+};
+
+// A chunk of 8 values of token t's row from element e on.
 template <typename TD>
-__device__ __forceinline__ void ld8_sum(const TD* p, int slices, int64_t slice_stride, float* v) {
-  ld8(p, v);
-  for (int s = 1; s < slices; ++s) {
-    float u[8];
-    ld8(p + s * slice_stride, u);
+__device__ __forceinline__ void ld8_sum(const TD* delta, const SumRule& rule, int64_t t, int H, int e, float* v) {
+  const TD* p = delta + t * rule.row_stride + e;
+  if (rule.weight == nullptr) {
+    ld8(p, v);
+    for (int s = 1; s < rule.slices; ++s) {
+      float u[8];
+      ld8(p + s * rule.slice_stride, u);
 #pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] += u[i];
+      for (int i = 0; i < 8; ++i) v[i] += u[i];
+    }
+    return;
+  }
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = 0.f;
+  for (int s = 0; s < rule.slices; ++s) {
+    const float w = rule.weight[t * rule.slices + s];
+    float u[8];
+    ld8(p + s * rule.slice_stride, u);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = fmaf(w, u[i], v[i]);
+  }
+  if (rule.add != nullptr) {
+    const float w = rule.add_gate != nullptr ? rule.add_gate[t] : 1.f;
+    float u[8];
+    ld8(rule.add + t * H + e, u);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = fmaf(w, u[i], v[i]);
   }
 }
 template <typename TD>
-__device__ __forceinline__ float ld_sum(const TD* p, int slices, int64_t slice_stride) {
-  float v = to_float(p[0]);
-  for (int s = 1; s < slices; ++s) v += to_float(p[s * slice_stride]);
+__device__ __forceinline__ float ld_sum(const TD* delta, const SumRule& rule, int64_t t, int H, int e) {
+  const TD* p = delta + t * rule.row_stride + e;
+  if (rule.weight == nullptr) {
+    float v = to_float(p[0]);
+    for (int s = 1; s < rule.slices; ++s) v += to_float(p[s * rule.slice_stride]);
+    return v;
+  }
+  float v = 0.f;
+  for (int s = 0; s < rule.slices; ++s) v = fmaf(rule.weight[t * rule.slices + s], to_float(p[s * rule.slice_stride]), v);
+  if (rule.add != nullptr) v = fmaf(rule.add_gate != nullptr ? rule.add_gate[t] : 1.f, rule.add[t * H + e], v);
   return v;
 }
 
@@ -72,20 +110,19 @@ template <typename TD, typename TO>
 __global__ __launch_bounds__(256) void norm_add_norm_kernel(
     TO* __restrict__ out, float* __restrict__ residual, const TD* __restrict__ delta,
     const float* __restrict__ post_gain, float eps, const float* __restrict__ next_gain, float next_eps, int H,
-    int slices, int64_t slice_stride) {
+    SumRule rule) {
   __shared__ float scratch[16];
   const int64_t base = static_cast<int64_t>(blockIdx.x) * H;
   float* r = residual + base;
-  const TD* dl = delta + base;
   float sd = 0.f;
   for (int i = threadIdx.x; i < H; i += blockDim.x) {
-    const float v = ld_sum(dl + i, slices, slice_stride);
+    const float v = ld_sum(delta, rule, blockIdx.x, H, i);
     sd += v * v;
   }
   const float inv_d = rsqrtf(block_sum(sd, scratch) / static_cast<float>(H) + eps);
   float ss = 0.f;
   for (int i = threadIdx.x; i < H; i += blockDim.x) {
-    const float v = r[i] + post_gain[i] * (ld_sum(dl + i, slices, slice_stride) * inv_d);
+    const float v = r[i] + post_gain[i] * (ld_sum(delta, rule, blockIdx.x, H, i) * inv_d);
     r[i] = v;
     ss += v * v;
   }
@@ -101,7 +138,7 @@ template <typename TD, typename TO, int NCH>
 __global__ __launch_bounds__(256) void norm_add_norm_vec_kernel(
     TO* __restrict__ out, float* __restrict__ residual, const TD* __restrict__ delta,
     const float* __restrict__ post_gain, float eps, const float* __restrict__ next_gain, float next_eps, int H,
-    int slices, int64_t slice_stride) {
+    SumRule rule) {
   __shared__ float scratch[16];
   const int64_t base = static_cast<int64_t>(blockIdx.x) * H;
   float d[NCH][8], v[NCH][8];
@@ -110,7 +147,7 @@ __global__ __launch_bounds__(256) void norm_add_norm_vec_kernel(
   for (int c = 0; c < NCH; ++c) {
     const int e = (c * 256 + threadIdx.x) * 8;
     if (e < H) {
-      ld8_sum(delta + base + e, slices, slice_stride, d[c]);
+      ld8_sum(delta, rule, blockIdx.x, H, e, d[c]);
       ld8(residual + base + e, v[c]);
 #pragma unroll
       for (int i = 0; i < 8; ++i) sd += d[c][i] * d[c][i];
@@ -149,16 +186,15 @@ __global__ __launch_bounds__(256) void norm_add_norm_vec_kernel(
 
 template <typename TD, typename TO>
 void launch_norm_add_norm(TO* out, float* residual, const TD* delta, const float* post_gain, float eps,
-                          const float* next_gain, float next_eps, int T, int H, int slices, hipStream_t stream) {
-  const int64_t slice_stride = static_cast<int64_t>(T) * H;
+                          const float* next_gain, float next_eps, int T, int H, const SumRule& rule, hipStream_t stream) {
   const auto misaligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) % 16) != 0; };
   const bool vec = H % 8 == 0 && H <= 8 * 2048 && !misaligned(out) && !misaligned(residual) && !misaligned(delta) &&
-                   !misaligned(post_gain) && !misaligned(next_gain);
+                   !misaligned(post_gain) && !misaligned(next_gain) && !misaligned(rule.add);
   if (vec) {
     const int nch = (H + 2047) / 2048;
 #define KVC_NAN_CASE(NN)                                                                                   \
   hipLaunchKernelGGL((norm_add_norm_vec_kernel<TD, TO, NN>), dim3(T), dim3(256), 0, stream, out, residual, \
-                     delta, post_gain, eps, next_gain, next_eps, H, slices, slice_stride)
+                     delta, post_gain, eps, next_gain, next_eps, H, rule)
     if (nch <= 1) KVC_NAN_CASE(1);
     else if (nch <= 2) KVC_NAN_CASE(2);
     else if (nch <= 4) KVC_NAN_CASE(4);
@@ -167,7 +203,7 @@ void launch_norm_add_norm(TO* out, float* residual, const TD* delta, const float
     return;
   }
   hipLaunchKernelGGL((norm_add_norm_kernel<TD, TO>), dim3(T), dim3(256), 0, stream, out, residual, delta,
-                     post_gain, eps, next_gain, next_eps, H, slices, slice_stride);
+                     post_gain, eps, next_gain, next_eps, H, rule);
 }
 
 // One block a token.  The sums of squares of the two sections first (the raw keys copied behind
@@ -281,16 +317,25 @@ __global__ __launch_bounds__(256) void diff_heads_norm_kernel(T* __restrict__ ou
 
 extern "C" int kvc_norm_add_norm(void* out, int out_dtype, float* residual, const void* delta, int delta_dtype,
                                  const float* post_gain, float eps, const float* next_gain, float next_eps,
-                                 int T, int H, int slices, kvc_stream stream) {
+                                 int T, int H, int slices, const float* weight, const float* add,
+                                 const float* add_gate, kvc_stream stream) {
   if (T < 0 || H <= 0 || slices < 1) return kvc_fail("kvc_norm_add_norm: bad sizes");
-  if (slices > 1 && delta_dtype != 0) return kvc_fail("kvc_norm_add_norm: partial sums are float32");
+  if ((slices > 1 || weight != nullptr) && delta_dtype != 0)
+    return kvc_fail("kvc_norm_add_norm: partial sums and weighted rows are float32");
+  if (weight == nullptr && (add != nullptr || add_gate != nullptr))
+    return kvc_fail("kvc_norm_add_norm: a further row joins weighted rows only");
   if (residual == nullptr || delta == nullptr || post_gain == nullptr) return kvc_fail("kvc_norm_add_norm: null operand");
   if (out != nullptr && next_gain == nullptr) return kvc_fail("kvc_norm_add_norm: the second norm needs its gain");
   if (T == 0) return 0;
   if (out == nullptr) next_gain = post_gain;  // never read
+  SumRule rule{slices, H, static_cast<int64_t>(T) * H, weight, add, add_gate};
+  if (weight != nullptr) {  // a token's rows lie one after the other
+    rule.row_stride = static_cast<int64_t>(slices) * H;
+    rule.slice_stride = H;
+  }
 #define KVC_NAN(TD, TO)                                                                                         \
   launch_norm_add_norm<TD, TO>(static_cast<TO*>(out), residual, static_cast<const TD*>(delta), post_gain, eps, \
-                               next_gain, next_eps, T, H, slices, S(stream))
+                               next_gain, next_eps, T, H, rule, S(stream))
   if (delta_dtype == 0 && out_dtype == 0) {
     KVC_NAN(float, float);
   } else if (delta_dtype == 0 && out_dtype == 1) {

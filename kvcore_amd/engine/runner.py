@@ -229,13 +229,12 @@ class ModelRunner:
     # -------------------------------------------------------------------- bookkeeping
     def forget(self, slot: int) -> None:
         """A request left its slot.  The next owner's pages are synced from scratch.  With
-        ``poison_pages`` the slot's rows of every state array become NaN (on the stream, behind
-        the steps launched so far), so that a next owner that read them would show."""
+        ``poison_pages`` the slot's rows of every state array become NaN (integers -1; on the stream,
+        behind the steps launched so far), so that a next owner that read them would show."""
         self._slot_owner[slot] = None
         if self.poison_pages:
             for state in self.states:
-                if state.dtype.is_floating_point:
-                    state[slot].fill_(float("nan"))
+                state[slot].fill_(float("nan") if state.dtype.is_floating_point else -1)
 
     def poison(self, pages: Sequence[Sequence[int]]) -> None:
         """Fill the listed pages (one list per cache group) with NaN on the stream, behind the
@@ -259,6 +258,8 @@ class ModelRunner:
         for state in self.states:
             if state.dtype.is_floating_point:
                 state.fill_(value)
+            elif value != value:
+                state.fill_(-1)  # no token, no row: as good as a NaN
 
     def cache_bytes(self) -> int:
         return sum(p.numel() * p.element_size() for g in self.groups for p in g.storage)

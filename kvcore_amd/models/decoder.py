@@ -153,6 +153,9 @@ class DecoderModel:
                 raise ValueError(f"schedule entry {e} names stream op {entry.before}, which does not exist")
             calls.append(LayerCall(e, entry.layer, g, plane, write,
                                    state_indices[0] if state_indices else None, tuple(state_indices)))
+        needs_of_embedding = self.embed.state_needs()
+        self.embed_states = tuple(range(len(states), len(states) + len(needs_of_embedding)))
+        states.extend(StateArraySpec(need) for need in needs_of_embedding)
         self.calls = calls
         self.schedule = schedule
         self.cache_groups = [CacheGroupSpec(n, c) for n, c in zip(needs, planes)]
@@ -165,7 +168,7 @@ class DecoderModel:
             local: dict[str, torch.Tensor] = {}
             for ps in part.param_specs():
                 t = torch.empty(ps.shape, dtype=kinds[ps.kind], device=self.device)
-                full = f"{prefix}.{ps.name}"
+                full = checkpoint_name(prefix, ps.name)
                 if full in self.params:
                     raise ValueError(f"parameter {full} is declared twice")
                 self.params[full] = BoundParam(full, prefix, ps, t)
@@ -271,10 +274,10 @@ class DecoderModel:
         H = self.spec.hidden_size
         if self.stream_copies == 1:
             residual = ctx.buf("residual", H, torch.float32)
-            self.embed.forward(residual, ctx.token_ids[: ctx.num_tokens])
+            self.embed.forward_step(residual, ctx, self.embed_states)
         else:  # every copy starts as the embedding's row
             first = ctx.buf("embedded_rows", H, torch.float32)
-            self.embed.forward(first, ctx.token_ids[: ctx.num_tokens])
+            self.embed.forward_step(first, ctx, self.embed_states)
             residual = ctx.buf(f"residual:{self.stream_copies}", self.stream_copies * H, torch.float32)
             ops.spread_streams(residual, first, self.stream_copies)
         for pe in self.positions:

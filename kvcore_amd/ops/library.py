@@ -9,6 +9,7 @@ products for bfloat16 excepted, which is where the reference uses a library too:
 
 from __future__ import annotations
 
+import math
 import os
 
 import ctypes
@@ -33,6 +34,7 @@ def _declare(lib: ctypes.CDLL) -> None:
     P, I, L, F = c_void_p, c_int, c_int64, c_float
     sigs = {
         "kvc_embed": [P, P, P, I, I, I, I, F, P],
+        "kvc_embed_pairs": [P, P, P, P, P, P, P, P, P, I, I, I, L, L, L, I, P],
         "kvc_logits_finish": [P, I, I, L, P, I, F, F, P],
         "kvc_fill_pages": [P, P, I, I, I, I, L, I, ctypes.c_uint32, P],
         "kvc_fill_normal": [P, L, I, ctypes.c_uint32, ctypes.c_uint32, F, F, P],
@@ -42,12 +44,12 @@ def _declare(lib: ctypes.CDLL) -> None:
         "kvc_residual_add": [P, P, I, I, I, P],
         "kvc_residual_add2": [P, P, I, P, I, I, I, P],
         "kvc_silu_mul": [P, P, I, I, I, P],
-        "kvc_gate_mul": [P, P, I, I, I, I, P],
+        "kvc_gate_mul": [P, P, I, I, I, F, F, F, I, P],
         "kvc_activation": [P, P, L, I, I, P],
         "kvc_hyper_step": [P, I, P, P, I, I, P, I, P, P, F, P, P, F, I, I, I, P],
         "kvc_spread_streams": [P, P, I, I, I, P],
         "kvc_diff_heads_norm": [P, P, L, I, F, F, F, I, I, I, I, P],
-        "kvc_norm_add_norm": [P, I, P, P, I, P, F, P, F, I, I, I, P],
+        "kvc_norm_add_norm": [P, I, P, P, I, P, F, P, F, I, I, I, P, P, P, P],
         "kvc_wide_qk_norm": [P, L, P, P, F, I, I, I, I, I, P],
         "kvc_head_gate": [P, P, L, P, L, I, I, I, I, I, I, P],
         "kvc_latent_rows": [P, L, P, P, L, P, L, P, P, F, I, I, I, I, I, P],
@@ -64,14 +66,13 @@ def _declare(lib: ctypes.CDLL) -> None:
         "kvc_decay_and_write_gates": [P, P, P, L, P, L, P, P, I, I, P],
         "kvc_unit_heads": [P, L, I, I, I, F, F, I, F, P],
         "kvc_head_rmsnorm_gate": [P, I, P, P, L, I, P, F, I, I, I, P],
-        "kvc_moe_route": [P, P, P, I, I, I, I, I, I, P, I, F, P],
-        "kvc_moe_router": [P, P, P, L, I, P, I, I, I, I, I, I, I, P, I, F, P],
+        "kvc_moe_route": [P, P, P, I, I, I, I, I, I, P, P, I, F, P],
+        "kvc_moe_router": [P, P, P, L, I, P, P, I, I, I, I, I, I, I, P, P, I, F, P],
         "kvc_moe_max_tiles": [I, I, I],
         "kvc_moe_tile_rows": [I, I],
         "kvc_moe_align": [P, P, P, P, I, I, I, I, P],
         "kvc_moe_gemm": [P, L, I, P, L, P, I, P, P, P, I, I, I, I, I, I, I, F, F, F, I, P],
-        "kvc_moe_combine": [P, P, P, I, P, I, P, I, I, I, P],
-        "kvc_clamped_glu": [P, P, I, I, F, F, I, P],
+        "kvc_moe_combine": [P, P, P, I, P, I, P, P, I, I, I, P],
         "kvc_qk_norm_rope_kv_write": [P, L, P, P, I, P, P, F, P, P, I, I, P, I, I, I, I, I, I, I, I, P],
         "kvc_add_layernorm": [P, P, P, P, P, F, I, I, I, P],
         "kvc_rms_branches_mean": [P, P, P, I, F, I, I, I, P],
@@ -82,23 +83,23 @@ def _declare(lib: ctypes.CDLL) -> None:
         "kvc_rglru_scan": [P, I, P, P, P, L, I, P, P, P, P, P, I, I, I, P, L, P],
         "kvc_ssm_scan": [P, P, L, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
         "kvc_gated_group_rmsnorm": [P, I, P, P, L, I, P, F, I, I, I, P],
-        "kvc_decode_attention": [P, P, P, P, L, P, P, P, I, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I,
-                                 F, I, P, I, P, I, I, P],
+        "kvc_decode_attention": [P, P, P, P, L, P, P, P, I, P, P, P, P, P, P, I, I, P, P, F, I, I, I, I, I, I,
+                                 I, I, F, I, P, I, P, I, I, P],
         "kvc_decode_attention_waves": [I, I, I],
         "kvc_decode_attention_max_table": [I, I, I],
-        "kvc_decode_attention_supported": [I, I, I, I, I],
-        "kvc_prefill_attention": [P, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, P, I, P, P, P, I,
+        "kvc_decode_attention_supported": [I, I, I, I, I, I],
+        "kvc_prefill_attention": [P, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, I, I, F, I, P, I, P, P, P, I,
                                   P, P, I, I, I, P],
-        "kvc_prefill_attention_supported": [I, I, I, I, I],
+        "kvc_prefill_attention_supported": [I, I, I, I, I, I],
         "kvc_gemm_mid_slices": [I, I],
-        "kvc_gemm_mid_bf16": [P, P, P, P, P, I, I, I, L, L, I, I, I, P],
+        "kvc_gemm_mid_bf16": [P, P, P, P, P, I, I, I, L, L, I, I, F, F, F, I, P],
         "kvc_gemm_f32": [P, P, P, P, I, I, I, L, L, P],
         "kvc_gemm_skinny_bf16": [P, P, P, P, I, I, I, L, L, I, I, P],
         "kvc_gemm_skinny_act_bf16": [P, P, P, P, I, I, I, L, L, I, I, P],
         "kvc_gemm_skinny_silu_mul_bf16": [P, P, P, P, I, I, I, L, L, I, P],
         "kvc_pack_weight": [P, P, I, I, P],
         "kvc_gemm_skinny_blocks": [I, I, I, I],
-        "kvc_gemm_skinny_fused_bf16": [P, P, P, P, I, I, I, L, L, I, P, I, I, F, P, L, P, P, I, P],
+        "kvc_gemm_skinny_fused_bf16": [P, P, P, P, I, I, I, L, L, I, F, F, F, P, I, I, F, P, L, P, P, I, P],
         "kvc_table_update": [P, I, I, P, I, P],
         "kvc_argmax": [P, P, I, I, L, P, P, I, P],
         "kvc_argmax_static": [P, P, I, I, L, P],
@@ -195,6 +196,26 @@ def embed(residual: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, scale:
                             _stream()), "kvc_embed")
 
 
+def embed_pairs(residual: torch.Tensor, table: torch.Tensor, pairs: torch.Tensor, ids: torch.Tensor,
+                last: torch.Tensor, *, mul_prev: int, mul_cur: int, positions: torch.Tensor,
+                token_req: torch.Tensor, q_start: torch.Tensor, slots: torch.Tensor) -> None:
+    """``residual[t] = table[ids[t]] + pairs[row]`` in float32, ``pairs [buckets + 1, H]``: the last row for
+    the token at position 0, else row ``(prev * mul_prev + ids[t] * mul_cur) % buckets`` with ``prev`` the
+    token before it; between steps a request's last token waits in ``last [slots]`` (int32)."""
+    T, H = residual.shape
+    V, buckets = table.shape[0], pairs.shape[0] - 1
+    if table.shape[1] != H or pairs.shape[1] != H or buckets < 1 or ids.numel() < T or pairs.dtype != table.dtype:
+        raise KernelError("embed_pairs: shapes do not match")
+    if positions.numel() < T or token_req.numel() < T or last.dim() < 1 or last.numel() != last.shape[0]:
+        raise KernelError("embed_pairs: index arrays too short, or not a token a slot")
+    i32 = torch.int32
+    _check(load().kvc_embed_pairs(
+        _dev(residual, "residual", torch.float32), _dev(table, "table"), _dev(pairs, "pairs"), _dev(ids, "ids", i32),
+        _dev(last, "last", i32), _dev(positions, "positions", i32), _dev(token_req, "token_req", i32),
+        _dev(q_start, "q_start", i32), _dev(slots, "slots", i32), T, H, V, buckets, int(mul_prev) % buckets,
+        int(mul_cur) % buckets, _code(table, "table"), _stream()), "kvc_embed_pairs")
+
+
 def logits_finish(logits: torch.Tensor, bias: torch.Tensor | None = None, soft_cap: float = 0.0,
                   scale: float = 1.0) -> None:
     """In place on float32 ``logits [S, V]``: ``+ bias``, then ``soft_cap * tanh(x / soft_cap)``
@@ -289,22 +310,35 @@ def residual_add2(residual: torch.Tensor, a: torch.Tensor, b: torch.Tensor) -> N
                                     _dev(b, "b"), _code(b, "b"), T, H, _stream()), "kvc_residual_add2")
 
 
-GATE_ACTS = {"silu": 0, "gelu_tanh": 1}  # the activations of a gated feed-forward's gate
+GATE_ACTS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}  # how a gated feed-forward joins its branches
 
 
-def _gate_act(act: str) -> int:
-    try:
-        return GATE_ACTS[act]
-    except KeyError:
-        raise KernelError(f"unknown gate activation {act!r} (known: {sorted(GATE_ACTS)})") from None
+@dataclass(frozen=True)
+class GateAct:
+    """How a gated feed-forward joins its branches g and u: ``silu`` ``g sigmoid(g) u``, ``gelu_tanh``
+    ``gelu(g) u`` (the tanh form), ``clamped`` ``g' sigmoid(alpha g') (clamp(u, -limit, limit) + up_shift)``
+    with ``g' = min(g, limit)``.  Functions that take one take the bare name of the first two as well."""
+
+    kind: str
+    limit: float = math.inf
+    alpha: float = 1.0
+    up_shift: float = 0.0
 
 
-def silu_mul(out: torch.Tensor, gate_up: torch.Tensor, act: str = "silu") -> None:
-    """``out = act(gate) * up`` for rows ``[gate | up]``; ``act`` is ``silu`` or ``gelu_tanh``."""
+def _gate_rule(act: "str | GateAct") -> tuple[int, float, float, float]:
+    if isinstance(act, str):
+        act = GateAct(act)
+    if act.kind not in GATE_ACTS:
+        raise KernelError(f"unknown gate activation {act.kind!r} (known: {sorted(GATE_ACTS)})")
+    return GATE_ACTS[act.kind], float(act.limit), float(act.alpha), float(act.up_shift)
+
+
+def silu_mul(out: torch.Tensor, gate_up: torch.Tensor, act: "str | GateAct" = "silu") -> None:
+    """``out = act(gate) * up`` for rows ``[gate | up]``; ``act``: see :class:`GateAct`."""
     T, I2 = gate_up.shape
     if I2 % 2 or out.shape != (T, I2 // 2) or out.dtype != gate_up.dtype:
         raise KernelError("silu_mul: shapes or dtypes do not match")
-    _check(load().kvc_gate_mul(_dev(out, "out"), _dev(gate_up, "gate_up"), T, I2 // 2, _gate_act(act),
+    _check(load().kvc_gate_mul(_dev(out, "out"), _dev(gate_up, "gate_up"), T, I2 // 2, *_gate_rule(act),
                                _code(out, "out"), _stream()), "kvc_gate_mul")
 
 
@@ -517,16 +551,19 @@ def qk_norm_rope_kv_write(qkv: torch.Tensor, k_cache: torch.Tensor,
                           cos: torch.Tensor, sin: torch.Tensor, *, rot_dim: int, interleaved: bool,
                           kv_slot: torch.Tensor, nh: int, nkv: int, d: int, dv: int,
                           q_gain: torch.Tensor | None = None, k_gain: torch.Tensor | None = None,
-                          eps: float = 0.0, write_kv: bool = True) -> None:
+                          eps: float = 0.0, write_kv: bool = True, queries_only: bool = False) -> None:
     """Rows of ``qkv`` are ``[nh heads of d | nkv heads of d | nkv heads of dv]``.  With gains
     (float32 ``[d]``, shared by all heads) every q and k head is first divided by its root mean
     square (``eps`` inside the root) and multiplied by the gain; then the first ``rot_dim``
     elements are rotated; q and k are rewritten in place, k and v stored at ``kv_slot``
     (``k_cache [pages, nkv, page_size, d]``, ``v_cache [pages, nkv, dv, page_size]``, or a list of
     up to four planes ``[pages, nkv, dv / n, page_size]`` that each hold a slice of every value
-    head)."""
+    head).  ``queries_only``: the rows hold the query heads alone and nothing is stored."""
     T = qkv.shape[0]
-    if qkv.dim() != 2 or qkv.stride(1) != 1 or qkv.shape[1] < (nh + nkv) * d + nkv * dv:
+    row_kv = 0 if queries_only else nkv
+    if queries_only and write_kv:
+        raise KernelError("qk_norm_rope_kv_write: rows of queries alone have nothing to store")
+    if qkv.dim() != 2 or qkv.stride(1) != 1 or qkv.shape[1] < (nh + row_kv) * d + row_kv * dv:
         raise KernelError(f"qk_norm_rope_kv_write: qkv shape {tuple(qkv.shape)} does not fit the heads")
     planes = list(v_cache) if isinstance(v_cache, (list, tuple)) else [v_cache]
     if not 1 <= len(planes) <= 4 or dv % len(planes):
@@ -550,7 +587,7 @@ def qk_norm_rope_kv_write(qkv: torch.Tensor, k_cache: torch.Tensor,
         qkv.data_ptr(), qkv.stride(0), _dev(k_cache, "k_cache"), pointers, len(planes),
         None if q_gain is None else _dev(q_gain, "q_gain"), None if k_gain is None else _dev(k_gain, "k_gain"),
         float(eps), _dev(cos, "cos", torch.float32), _dev(sin, "sin", torch.float32), int(rot_dim),
-        int(bool(interleaved)), _dev(kv_slot, "kv_slot", torch.int32), T, nh, nkv, d, dv, page_size,
+        int(bool(interleaved)), _dev(kv_slot, "kv_slot", torch.int32), T, nh, row_kv, d, dv, page_size,
         int(write_kv), _code(qkv, "qkv"), _stream()), "kvc_qk_norm_rope_kv_write")
 
 
@@ -572,8 +609,10 @@ def _sinks(sinks: torch.Tensor | None, nh: int) -> int | None:
     return _dev(sinks, "sinks", torch.float32)
 
 
-def decode_attention_supported(nh: int, nkv: int, d: int, page_size: int, dtype: torch.dtype) -> bool:
-    return bool(load().kvc_decode_attention_supported(nh, nkv, d, page_size, DTYPE_CODE.get(dtype, -1)))
+def decode_attention_supported(nh: int, nkv: int, d: int, page_size: int, dtype: torch.dtype,
+                               dv: int | None = None) -> bool:
+    return bool(load().kvc_decode_attention_supported(nh, nkv, d, d if dv is None else dv, page_size,
+                                                      DTYPE_CODE.get(dtype, -1)))
 
 
 KERNEL_FAMILIES = {"prefill_attention": 0, "rope_kv_write": 1, "decode_attention": 2}
@@ -657,21 +696,30 @@ def decode_attention(out: torch.Tensor, qkv: torch.Tensor, k_cache: torch.Tensor
                      sin: torch.Tensor | None = None, rot_dim: int = 0, interleaved: bool = False,
                      write_kv: bool = False, token_rows: torch.Tensor | None = None,
                      slopes: torch.Tensor | None = None, chunk: int = 0,
-                     sinks: torch.Tensor | None = None) -> None:
+                     sinks: torch.Tensor | None = None, dv: int | None = None,
+                     q_gain: torch.Tensor | None = None, k_gain: torch.Tensor | None = None,
+                     eps: float = 0.0) -> None:
     """bfloat16 attention of single tokens on the matrix cores (see the C header), with the
     rotation of each token's query and key and the write of its key and value into the cache
     (``write_kv``) in the same kernel; ``qkv`` is not changed.  With ``rot_dim = 0`` and
     ``write_kv = False`` it is the attention alone over queries as they are.  ``token_rows``
     (``slots[token_req]``, -1 for padding) may be given to save the kernel a lookup.  ``part_o`` and
-    ``part_ml`` are float32 workspaces of at least ``T*nh*nsplit*d`` and ``T*nh*nsplit*2``
-    elements when ``nsplit > 1``."""
+    ``part_ml`` are float32 workspaces of at least ``T*nh*nsplit*dv`` and ``T*nh*nsplit*2``
+    elements when ``nsplit > 1``.  ``dv``: the size of a value head, ``d`` (the default) or half of
+    it.  ``q_gain`` and ``k_gain`` (float32 ``[d]``): every query head, and the key head that is
+    written, is divided by its root mean square (``eps`` inside the root) and multiplied by the
+    gain before the rotation."""
     T = out.shape[0]
-    if out.shape != (T, nh * d) or not out.is_contiguous() or out.dtype not in (torch.bfloat16, torch.float32):
-        raise KernelError("decode_attention: out must be contiguous bfloat16 (or float32) [T, nh*d]")
-    need = (nh + 2 * nkv) * d if write_kv else nh * d
+    dv = d if dv is None else dv
+    if out.shape != (T, nh * dv) or not out.is_contiguous() or out.dtype not in (torch.bfloat16, torch.float32):
+        raise KernelError("decode_attention: out must be contiguous bfloat16 (or float32) [T, nh*dv]")
+    need = (nh + nkv) * d + nkv * dv if write_kv else nh * d
+    for gain in (q_gain, k_gain):
+        if gain is not None and gain.shape != (d,):
+            raise KernelError("decode_attention: a gain must be float32 [d]")
     if qkv.shape[0] != T or qkv.stride(1) != 1 or qkv.shape[1] < need or qkv.dtype != torch.bfloat16:
         raise KernelError("decode_attention: qkv does not fit")
-    num_pages, page_size = _check_cache(k_cache, v_cache, nkv, d, "decode_attention")
+    num_pages, page_size = _check_cache(k_cache, v_cache, nkv, d, "decode_attention", dv)
     if k_cache.dtype != qkv.dtype:
         raise KernelError("decode_attention: cache dtype differs from the queries'")
     if positions.numel() < T or token_req.numel() < T:
@@ -684,7 +732,7 @@ def decode_attention(out: torch.Tensor, qkv: torch.Tensor, k_cache: torch.Tensor
         c, s_ = _dev(cos, "cos", torch.float32), _dev(sin, "sin", torch.float32)
     po = pm = None
     if nsplit > 1:
-        if part_o is None or part_ml is None or part_o.numel() < T * nh * nsplit * d \
+        if part_o is None or part_ml is None or part_o.numel() < T * nh * nsplit * dv \
                 or part_ml.numel() < T * nh * nsplit * 2:
             raise KernelError("decode_attention: workspace missing or too small")
         po, pm = _dev(part_o, "part_o", torch.float32), _dev(part_ml, "part_ml", torch.float32)
@@ -695,14 +743,18 @@ def decode_attention(out: torch.Tensor, qkv: torch.Tensor, k_cache: torch.Tensor
         _dev(slots, "slots", torch.int32),
         None if token_rows is None else _dev(token_rows, "token_rows", torch.int32),
         c, s_, int(rot_dim), int(bool(interleaved)),
-        int(bool(write_kv)), T, nh, nkv, d, page_size, num_pages, float(scale),
+        None if q_gain is None else _dev(q_gain, "q_gain", torch.float32),
+        None if k_gain is None else _dev(k_gain, "k_gain", torch.float32), float(eps),
+        int(bool(write_kv)), T, nh, nkv, d, dv, page_size, num_pages, float(scale),
         int(window), _slopes(slopes, nh), int(chunk), _sinks(sinks, nh), int(nsplit),
         int(out.dtype == torch.float32), _stream()),
         "kvc_decode_attention")
 
 
-def prefill_attention_supported(nh: int, nkv: int, d: int, page_size: int, dtype: torch.dtype) -> bool:
-    return bool(load().kvc_prefill_attention_supported(nh, nkv, d, page_size, DTYPE_CODE.get(dtype, -1)))
+def prefill_attention_supported(nh: int, nkv: int, d: int, page_size: int, dtype: torch.dtype,
+                                dv: int | None = None) -> bool:
+    return bool(load().kvc_prefill_attention_supported(nh, nkv, d, d if dv is None else dv, page_size,
+                                                       DTYPE_CODE.get(dtype, -1)))
 
 
 def prefill_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
@@ -712,25 +764,27 @@ def prefill_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
                       part_ml: torch.Tensor | None = None, cos: torch.Tensor | None = None,
                       sin: torch.Tensor | None = None, rot_dim: int = 0, interleaved: bool = False,
                       slopes: torch.Tensor | None = None, chunk: int = 0,
-                      sinks: torch.Tensor | None = None) -> None:
+                      sinks: torch.Tensor | None = None, dv: int | None = None) -> None:
     """bfloat16 attention of portions of prompts on the matrix cores (see the C header).
     ``nsplit > 1`` deals every tile's keys to that many blocks; ``part_o`` (float32,
-    ``T*nh*nsplit*d`` values) and ``part_ml`` (``T*nh*nsplit*2``) are then the workspace.
+    ``T*nh*nsplit*dv`` values) and ``part_ml`` (``T*nh*nsplit*2``) are then the workspace.
+    ``dv``: the size of a value head, ``d`` (the default) or half of it.
     With ``cos`` and ``sin`` (``[T, rot_dim / 2]`` float32) the queries come unrotated and
     the kernel rotates them (``prefill_attention_rotates`` says for which shapes)."""
     T = out.shape[0]
-    if out.shape != (T, nh * d) or not out.is_contiguous() or out.dtype not in (torch.bfloat16, torch.float32):
-        raise KernelError("prefill_attention: out must be contiguous bfloat16 (or float32) [T, nh*d]")
+    dv = d if dv is None else dv
+    if out.shape != (T, nh * dv) or not out.is_contiguous() or out.dtype not in (torch.bfloat16, torch.float32):
+        raise KernelError("prefill_attention: out must be contiguous bfloat16 (or float32) [T, nh*dv]")
     if q.shape[0] != T or q.stride(1) != 1 or q.shape[1] < nh * d or q.dtype != torch.bfloat16:
         raise KernelError("prefill_attention: q does not fit")
-    num_pages, page_size = _check_cache(k_cache, v_cache, nkv, d, "prefill_attention")
+    num_pages, page_size = _check_cache(k_cache, v_cache, nkv, d, "prefill_attention", dv)
     if k_cache.dtype != q.dtype:
         raise KernelError("prefill_attention: cache dtype differs from the queries'")
     if positions.numel() < T or q_start.numel() < num_reqs + 1 or slots.numel() < num_reqs:
         raise KernelError("prefill_attention: index arrays too short")
     po = pml = None
     if nsplit > 1:
-        if part_o is None or part_ml is None or part_o.numel() < T * nh * nsplit * d or \
+        if part_o is None or part_ml is None or part_o.numel() < T * nh * nsplit * dv or \
                 part_ml.numel() < T * nh * nsplit * 2:
             raise KernelError("prefill_attention: the workspace for splits is missing or too small")
         po, pml = _dev(part_o, "part_o", torch.float32), _dev(part_ml, "part_ml", torch.float32)
@@ -744,7 +798,7 @@ def prefill_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
         out.data_ptr(), q.data_ptr(), q.stride(0), _dev(k_cache, "k_cache"), _dev(v_cache, "v_cache"),
         _dev(table, "table", torch.int32), table.shape[1], _dev(positions, "positions", torch.int32),
         _dev(q_start, "q_start", torch.int32), _dev(slots, "slots", torch.int32), T, num_reqs,
-        nh, nkv, d, page_size, num_pages, float(scale), int(window), _slopes(slopes, nh), int(chunk),
+        nh, nkv, d, dv, page_size, num_pages, float(scale), int(window), _slopes(slopes, nh), int(chunk),
         _sinks(sinks, nh), po, pml, int(nsplit), cs, sn, int(rot_dim) if cs is not None else 0, int(interleaved),
         int(out.dtype == torch.float32), _stream()),
         "kvc_prefill_attention")
@@ -914,6 +968,27 @@ class SlicedRows:
     bias: torch.Tensor | None = None
 
 
+@dataclass
+class WeightedRows:
+    """The results of a token's experts, not yet added up: ``data [>= T * n, H]`` float32 (token t's ``n``
+    rows one after the other), ``weight [T, n]``; row t is ``sum_c weight[t, c] * data[t * n + c]``, plus
+    ``add[t]`` (float32, or None) times ``add_gate[t]`` (``[T, 1]``, or None: once).  ``norm_add_norm`` takes
+    it in place of the summed rows (``moe_combine`` makes those)."""
+
+    data: torch.Tensor
+    weight: torch.Tensor
+    add: torch.Tensor | None = None
+    add_gate: torch.Tensor | None = None
+
+    def check(self, T: int, H: int) -> int:
+        n = self.weight.shape[1]
+        if self.weight.shape[0] != T or n < 1 or self.data.shape[1] != H or self.data.shape[0] < T * n \
+                or (self.add is not None and self.add.shape != (T, H)) \
+                or (self.add_gate is not None and (self.add is None or self.add_gate.numel() != T)):
+            raise KernelError("weighted rows do not fit")
+        return n
+
+
 # The most rows the kernel that shares its rows through LDS takes (twelve tiles of 16 a wave).
 # Measured on the 8B shape against the vendor's products with a norm kernel between them, a
 # whole decode step: 72 rows 5.93 against 6.66 ms, 96 rows 6.53 against 7.72, 128 rows 7.57
@@ -968,7 +1043,7 @@ def skinny_blocks(N: int, K: int, gated: bool = False, packed: bool = False) -> 
 
 
 def _fused_skinny(out: torch.Tensor | ResidualSink, x: torch.Tensor | ScaledRows, w: torch.Tensor,
-                  bias: torch.Tensor | None, gated: bool, act: str = "silu") -> ScaledRows | None:
+                  bias: torch.Tensor | None, gated: bool, act: "str | GateAct" = "silu") -> ScaledRows | None:
     """The weight-streaming product with a norm on either side folded in (see the C header);
     ``act`` is the gate's activation of the gated form."""
     data = x.data if isinstance(x, ScaledRows) else x
@@ -1012,9 +1087,10 @@ def _fused_skinny(out: torch.Tensor | ResidualSink, x: torch.Tensor | ScaledRows
         ldr = 0
     if M:
         w_ptr, packed = _streamed(w, N)
+        code, *constants = _gate_rule(act)
         _check(load().kvc_gemm_skinny_fused_bf16(
             c_ptr, data.data_ptr(), w_ptr, None if bias is None else _dev(bias, "bias"), M, N, K,
-            data.stride(0), ldc, (1 + _gate_act(act)) if gated else 0, in_ss or None, in_parts, in_width, float(in_eps),
+            data.stride(0), ldc, 1 + code if gated else 0, *constants, in_ss or None, in_parts, in_width, float(in_eps),
             residual, ldr, gain, out_ss, packed, _stream()), "kvc_gemm_skinny_fused_bf16")
     return result
 
@@ -1048,13 +1124,15 @@ def mid_operands_ok(x: torch.Tensor, w: torch.Tensor) -> bool:
 
 
 def gemm_mid(out: torch.Tensor | None, x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None,
-             *, mode: int = 0, partial: torch.Tensor | None = None) -> None:
+             *, mode: int = 0, partial: torch.Tensor | None = None, act: "GateAct | None" = None) -> None:
     """The weight-streaming product for up to 192 rows of bfloat16 whose waves share the rows
     through LDS, the faster one from 9 rows on (see the C header for the
     modes: 0 plain, 1 ``silu(gate) * up``, 2 partial sums of slices along K only, 3 plain
-    with slices and a kernel that sums them, 4 ``gelu_tanh(gate) * up``)."""
+    with slices and a kernel that sums them, 4 ``gelu_tanh(gate) * up``, 5 the clamped ``act``)."""
     M, K = x.shape
-    N = w.shape[0] // 2 if mode in (1, 4) else w.shape[0]
+    N = w.shape[0] // 2 if mode in (1, 4, 5) else w.shape[0]
+    if (mode == 5) != (act is not None and act.kind == "clamped"):
+        raise KernelError("gemm_mid: mode 5 goes with a clamped activation")
     if w.shape[1] != K or x.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 or not x.is_cuda:
         raise KernelError("gemm_mid: operands must be bfloat16 GPU tensors with matching K")
     if not mid_operands_ok(x, w):
@@ -1074,7 +1152,8 @@ def gemm_mid(out: torch.Tensor | None, x: torch.Tensor, w: torch.Tensor, bias: t
     w_ptr, packed = _streamed(w, N)
     _check(load().kvc_gemm_mid_bf16(out_ptr, part_ptr, x.data_ptr(), w_ptr,
                                     None if bias is None else _dev(bias, "bias"), M, N, K, x.stride(0),
-                                    ldc, code, mode, packed, _stream()), "kvc_gemm_mid_bf16")
+                                    ldc, code, mode, *(_gate_rule(act)[1:] if act is not None else (0.0, 0.0, 0.0)),
+                                    packed, _stream()), "kvc_gemm_mid_bf16")
 
 
 def add_slices_rmsnorm(out: torch.Tensor, residual: torch.Tensor, partial: torch.Tensor, slices: int,
@@ -1146,9 +1225,9 @@ def _slices_mid(sink: SliceSink, x: torch.Tensor, w: torch.Tensor, bias: torch.T
 
 
 def linear_silu_mul(out: torch.Tensor, x: torch.Tensor | ScaledRows, w: torch.Tensor,
-                    bias: torch.Tensor | None, scratch, act: str = "silu") -> None:
+                    bias: torch.Tensor | None, scratch, act: "str | GateAct" = "silu") -> None:
     """``out = act(x @ wg.T) * (x @ wu.T)`` with ``wg`` the first half of ``w``'s rows and
-    ``wu`` the second (biases likewise); ``act`` is ``silu`` or ``gelu_tanh``.  Few rows of
+    ``wu`` the second (biases likewise); ``act``: see :class:`GateAct`.  Few rows of
     bfloat16 run as one weight-streaming kernel; otherwise ``scratch()`` gives the ``[M, 2I]``
     buffer for the two-kernel form."""
     if isinstance(x, ScaledRows):
@@ -1165,7 +1244,7 @@ def linear_silu_mul(out: torch.Tensor, x: torch.Tensor | ScaledRows, w: torch.Te
             return
         if bias is not None and (bias.dtype != torch.bfloat16 or bias.shape != (2 * I,)):
             raise KernelError("linear_silu_mul: bias must be bfloat16 [2I]")
-        if act != "silu":
+        if _gate_rule(act)[0] != 0:
             _fused_skinny(out, x, w, bias, gated=True, act=act)
             return
         w_ptr, packed = _streamed(w, I)
@@ -1177,7 +1256,8 @@ def linear_silu_mul(out: torch.Tensor, x: torch.Tensor | ScaledRows, w: torch.Te
             and x.is_cuda and mid_operands_ok(x, w) and out.stride(1) == 1
             and mid_rows_ok(M, bool(_streamed(w, I)[1]), MID_ROWS_GATED)):
         # 17 to 128 rows: the waves of a block share the rows through LDS
-        gemm_mid(out, x, w, bias, mode=4 if _gate_act(act) == 1 else 1)
+        code = _gate_rule(act)[0]
+        gemm_mid(out, x, w, bias, mode=(1, 4, 5)[code], act=act if code == 2 else None)
         return
     gate_up = scratch()
     linear(gate_up, x, w, bias)
@@ -1610,16 +1690,21 @@ def max_gated_finish(out: torch.Tensor, o: torch.Tensor, m: torch.Tensor, gate: 
         "kvc_max_gated_finish")
 
 
-def norm_add_norm(out: torch.Tensor | None, residual: torch.Tensor, delta: "torch.Tensor | SlicedRows",
+def norm_add_norm(out: torch.Tensor | None, residual: torch.Tensor, delta: "torch.Tensor | SlicedRows | WeightedRows",
                   post_gain: torch.Tensor, eps: float, next_gain: torch.Tensor | None = None,
                   next_eps: float | None = None) -> None:
     """``residual += post_gain * delta / rms(delta)``, then, given ``out``, ``out = next_gain *
     residual / rms(residual)``: the norm behind a sublayer, the sum into the float32 stream and the
     norm before the next sublayer in one pass (both roots hold their eps).  ``delta`` is float32
-    or bfloat16, or the :class:`SlicedRows` that a product left (their sum is the result)."""
+    or bfloat16, or the :class:`SlicedRows` that a product left (their sum is the result), or the
+    :class:`WeightedRows` of a feed-forward of routed experts."""
     T, H = residual.shape
     slices = 1
-    if isinstance(delta, SlicedRows):
+    weight = add = add_gate = None
+    if isinstance(delta, WeightedRows):
+        slices = delta.check(T, H)
+        weight, add, add_gate, delta = delta.weight, delta.add, delta.add_gate, delta.data
+    elif isinstance(delta, SlicedRows):
         if delta.bias is not None:
             raise KernelError("norm_add_norm: partial sums whose bias is still to be added")
         if (delta.rows, delta.width) != (T, H) or delta.data.dtype != torch.float32 \
@@ -1638,7 +1723,9 @@ def norm_add_norm(out: torch.Tensor | None, residual: torch.Tensor, delta: "torc
         _dev(residual, "residual", torch.float32), _dev(delta, "delta"), _code(delta, "delta"),
         _dev(post_gain, "post_gain", torch.float32), float(eps),
         None if out is None else _dev(next_gain, "next_gain", torch.float32),
-        float(eps if next_eps is None else next_eps), T, H, slices, _stream()), "kvc_norm_add_norm")
+        float(eps if next_eps is None else next_eps), T, H, slices,
+        *(None if t is None else _dev(t, "a weight", torch.float32) for t in (weight, add, add_gate)), _stream()),
+        "kvc_norm_add_norm")
 
 
 def wide_qk_norm(qkv: torch.Tensor, q_gain: torch.Tensor, k_gain: torch.Tensor, eps: float, *,
@@ -1695,27 +1782,31 @@ def head_gate(out: torch.Tensor, x: torch.Tensor, gate: torch.Tensor, *, heads: 
                                 _code(out, "out"), _stream()), "kvc_head_gate")
 
 
-ROUTE_SCORES = {"softmax": 0, "sigmoid": 1}  # how a router's logits become scores
+# how a router's logits become scores ("logit": they are the scores, and the weights are the softmax over
+# the chosen ones)
+ROUTE_SCORES = {"softmax": 0, "sigmoid": 1, "logit": 2}
 
 
-def _route_rule(E: int, score: str, correction: torch.Tensor | None, group_best: int,
-                weight_scale: float) -> tuple[int, int | None, int, float]:
+def _route_rule(E: int, score: str, bias: torch.Tensor | None, correction: torch.Tensor | None, group_best: int,
+                weight_scale: float) -> tuple[int, int | None, int | None, int, float]:
     if score not in ROUTE_SCORES:
         raise KernelError(f"unknown router score {score!r} (known: {sorted(ROUTE_SCORES)})")
-    if correction is not None and (correction.shape != (E,) or correction.dtype != torch.float32):
-        raise KernelError("moe routing: the correction is float32 [experts]")
+    for t, what in ((bias, "bias"), (correction, "correction")):
+        if t is not None and (t.shape != (E,) or t.dtype != torch.float32):
+            raise KernelError(f"moe routing: the {what} is float32 [experts]")
     if group_best not in (1, 2):
         raise KernelError("moe routing: a group is worth its best choice score or the sum of its best two")
-    return (ROUTE_SCORES[score], None if correction is None else _dev(correction, "correction"), int(group_best),
-            float(weight_scale))
+    return (ROUTE_SCORES[score], None if bias is None else _dev(bias, "bias"),
+            None if correction is None else _dev(correction, "correction"), int(group_best), float(weight_scale))
 
 
 def moe_route(choice: torch.Tensor, weight: torch.Tensor, logits: torch.Tensor, *, top: int, groups: int = 1,
               keep: int = 1, score: str = "softmax", correction: torch.Tensor | None = None, group_best: int = 1,
-              weight_scale: float = 1.0) -> None:
+              weight_scale: float = 1.0, bias: torch.Tensor | None = None) -> None:
     """The router's choice from float32 ``logits [T, E]``: ``choice`` (int32) and ``weight``
-    (float32), both ``[T, top]``.  ``score``: ``softmax`` over the experts or a ``sigmoid`` of each
-    logit; ``correction`` (float32 ``[E]``) joins the scores for the choice alone; a group is worth
+    (float32), both ``[T, top]``.  ``bias`` (float32 ``[E]``) joins the logits.  ``score``: ``softmax`` over the
+    experts, a ``sigmoid`` of each logit, or the ``logit`` itself (the weights are then the softmax over the
+    chosen logits); ``correction`` (float32 ``[E]``) joins the scores for the choice alone; a group is worth
     its ``group_best`` (1 or 2) best choice scores; the weights (the chosen experts' plain scores
     over their sum) are multiplied by ``weight_scale``."""
     T, E = logits.shape
@@ -1723,23 +1814,27 @@ def moe_route(choice: torch.Tensor, weight: torch.Tensor, logits: torch.Tensor, 
         raise KernelError("moe_route: shapes do not match")
     _check(load().kvc_moe_route(_dev(choice, "choice", torch.int32), _dev(weight, "weight", torch.float32),
                                 _dev(logits, "logits", torch.float32), T, E, top, groups, keep,
-                                *_route_rule(E, score, correction, group_best, weight_scale), _stream()),
+                                *_route_rule(E, score, bias, correction, group_best, weight_scale), _stream()),
            "kvc_moe_route")
 
 
 def moe_router(choice: torch.Tensor, weight: torch.Tensor, x: torch.Tensor, router: torch.Tensor, *, top: int,
                groups: int = 1, keep: int = 1, score: str = "softmax", correction: torch.Tensor | None = None,
-               group_best: int = 1, weight_scale: float = 1.0) -> None:
+               group_best: int = 1, weight_scale: float = 1.0, bias: torch.Tensor | None = None,
+               gate: torch.Tensor | None = None) -> None:
     """``moe_route`` of the logits ``x @ router.T`` (float32 sums in one fixed order; ``x [T, H]`` of
-    either dtype, ``router [E, H]`` float32) without storing the logits."""
+    either dtype, ``router [E, H]`` float32) without storing the logits.  With ``gate`` (float32, a
+    value a token) the router has one row more, and ``gate[t] = sigmoid(x[t] . that row)``."""
     T, H = x.shape
-    E = router.shape[0]
-    if router.shape != (E, H) or choice.shape != (T, top) or weight.shape != (T, top) or x.stride(1) != 1:
+    E = router.shape[0] - (1 if gate is not None else 0)
+    if gate is not None and gate.numel() != T:
+        raise KernelError("moe_router: a gate value a token")
+    if router.dim() != 2 or router.shape[1] != H or E < 1 or choice.shape != (T, top) or weight.shape != (T, top) or x.stride(1) != 1:
         raise KernelError("moe_router: shapes do not match")
     _check(load().kvc_moe_router(_dev(choice, "choice", torch.int32), _dev(weight, "weight", torch.float32),
                                  x.data_ptr(), x.stride(0), _code(x, "x"), _dev(router, "router", torch.float32),
-                                 T, H, E, top, groups, keep,
-                                 *_route_rule(E, score, correction, group_best, weight_scale), _stream()),
+                                 None if gate is None else _dev(gate, "gate", torch.float32), T, H, E, top, groups, keep,
+                                 *_route_rule(E, score, bias, correction, group_best, weight_scale), _stream()),
            "kvc_moe_router")
 
 
@@ -1790,9 +1885,10 @@ def moe_gemm(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, sorted_pairs: 
 
 
 def moe_combine(out: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, add0: torch.Tensor | None = None,
-                add1: torch.Tensor | None = None, accumulate: bool = False) -> None:
+                add1: torch.Tensor | None = None, accumulate: bool = False,
+                add1_gate: torch.Tensor | None = None) -> None:
     """``out[t] = sum_c weight[t, c] * y[t * top + c] (+ add0[t]) (+ add1[t])``, float32; ``add0``
-    of either dtype, ``add1`` float32.  ``accumulate``: the sum is added into ``out``."""
+    of either dtype, ``add1`` float32, times ``add1_gate`` (a value a token) if given.  ``accumulate``: the sum is added into ``out``."""
     T, H = out.shape
     top = weight.shape[1] if weight.dim() == 2 else 0
     if out.dtype != torch.float32 or (top and (y.shape[0] < T * top or y.shape[1] != H)):
@@ -1800,10 +1896,13 @@ def moe_combine(out: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, add0: 
     for a in (add0, add1):
         if a is not None and a.shape != (T, H):
             raise KernelError("moe_combine: an added row set does not fit")
+    if add1_gate is not None and (add1 is None or add1_gate.numel() != T):
+        raise KernelError("moe_combine: a gate value a token, for the second added row set")
     _check(load().kvc_moe_combine(_dev(out, "out"), _dev(y, "y", torch.float32), _dev(weight, "weight", torch.float32),
                                   top, None if add0 is None else _dev(add0, "add0"),
                                   0 if add0 is None else _code(add0, "add0"),
-                                  None if add1 is None else _dev(add1, "add1", torch.float32), T, H,
+                                  None if add1 is None else _dev(add1, "add1", torch.float32),
+                                  None if add1_gate is None else _dev(add1_gate, "add1_gate", torch.float32), T, H,
                                   int(bool(accumulate)), _stream()), "kvc_moe_combine")
 
 
@@ -1811,10 +1910,9 @@ def clamped_glu(out: torch.Tensor, gate_up: torch.Tensor, limit: float, alpha: f
     """``out = g * sigmoid(alpha * g) * (u + 1)`` with ``g = min(gate, limit)``, ``u = clamp(up,
     -limit, limit)`` from ``gate_up [T, 2I]`` (gate columns first)."""
     T, I = out.shape
-    if gate_up.shape != (T, 2 * I) or gate_up.dtype != out.dtype:
+    if gate_up.shape != (T, 2 * I):
         raise KernelError("clamped_glu: shapes do not match")
-    _check(load().kvc_clamped_glu(_dev(out, "out"), _dev(gate_up, "gate_up"), T, I, float(limit), float(alpha),
-                                  _code(out, "out"), _stream()), "kvc_clamped_glu")
+    silu_mul(out, gate_up, GateAct("clamped", limit, alpha, 1.0))
 
 
 def table_update(table: torch.Tensor, triples: torch.Tensor, n: int) -> None:

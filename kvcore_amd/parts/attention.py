@@ -117,8 +117,8 @@ class PagedAttention(Mixer):
                  tensor_names: dict[str, str] | None = None, float32_result: bool = False,
                  qk_norm_gain: bool = True, distance_slopes: tuple[float, ...] | None = None,
                  chunk: int = 0, qk_norm_span: str = "head", values_are_keys: bool = False,
-                 sinks: bool = False, sized_buffers: bool = False,
-                 position: PositionEncoding | None = None) -> None:
+                 sinks: bool | float = False, sized_buffers: bool = False, o_bias: bool | None = None,
+                 own_kv: bool = True, position: PositionEncoding | None = None) -> None:
         """``v_head_dim``: the size of a value head where it differs from ``head_dim``, the
         size of a query and key head.  ``qk_norm_eps`` (None: no such norm): every query and
         key head is divided by its root mean square, eps inside the root, and multiplied by a
@@ -134,7 +134,11 @@ class PagedAttention(Mixer):
         heads at once), with a gain of that whole size each, instead of every head alone.
         ``values_are_keys``: there is no value projection; a token's values are its keys as
         projected, before norm and rotation.  ``sinks``: a learned score per query head (tensor
-        ``sink``) that joins the softmax's denominator without a key or a value, unscaled.
+        ``sink``) that joins the softmax's denominator without a key or a value, unscaled; a number
+        instead is that score for every head, and there is no tensor.  ``o_bias`` None: the output
+        product has a bias iff the others do (``bias``).  ``own_kv`` False: the layer has no
+        projections of keys and values and reads the cache that another layer with the same head
+        counts and sizes has written (its schedule entry says ``cache_from``).
         ``sized_buffers``: name the step buffers by their width, for a model whose attention layers
         differ in size."""
         if qk_norm_span not in ("head", "projection"):
@@ -143,13 +147,17 @@ class PagedAttention(Mixer):
             raise ValueError("a norm over the whole projection needs its eps and has gains")
         if values_are_keys and v_head_dim not in (None, head_dim):
             raise ValueError("values that are the keys have the keys' size")
+        if not own_kv and (values_are_keys or qk_norm_span == "projection"):
+            raise ValueError("a layer that reads another's cache projects queries alone, normed head by head")
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} kv heads")
         v_head_dim = head_dim if v_head_dim is None else v_head_dim
         self.head_norm = qk_norm_eps is not None and qk_norm_span == "head"
         self.wide_norm = qk_norm_eps is not None and qk_norm_span == "projection"
         plain = v_head_dim == head_dim and not self.head_norm
-        if plain and (head_dim % 16 or head_dim > 256):
+        if not own_kv:
+            plain = False  # rows of queries alone
+        elif plain and (head_dim % 16 or head_dim > 256):
             if qk_norm_eps is None and not values_are_keys and not self.any_head_size:
                 raise ValueError(f"head size {head_dim} is not supported (multiples of 16 up to 256)")
             plain = False  # the kernel that rotates and writes heads of any size, and the general attention
@@ -163,7 +171,9 @@ class PagedAttention(Mixer):
         self.qk_norm_eps = qk_norm_eps
         self.qk_norm_gain = bool(qk_norm_gain)
         self.values_are_keys = bool(values_are_keys)
-        self.has_sinks = bool(sinks)
+        self.has_sinks = sinks is True  # a learned score a head
+        self.fixed_sink = float(sinks) if not isinstance(sinks, bool) else None  # the same for every head
+        self.own_kv = bool(own_kv)
         if distance_slopes is not None and len(distance_slopes) != num_heads:
             raise ValueError(f"{len(distance_slopes)} distance slopes for {num_heads} heads")
         if chunk < 0:
@@ -172,6 +182,7 @@ class PagedAttention(Mixer):
         self.chunk = int(chunk)
         self.scale = scale
         self.bias = bias
+        self.o_bias = bias if o_bias is None else bool(o_bias)
         self.window = window
         self.page_size = page_size  # None: the engine's block size
         self.position = position
@@ -180,6 +191,8 @@ class PagedAttention(Mixer):
         self.kv_size = num_kv_heads * head_dim
         self.v_size = num_kv_heads * v_head_dim
         self.o_size = num_heads * v_head_dim
+        # the width of a projected row
+        self.row_size = self.q_size + (self.kv_size + self.v_size if own_kv else 0)
         self.plain = plain
         # layers that are all alike share one step buffer a role; others name theirs by width
         self.shared_buffers = plain and not sized_buffers and not self.any_head_size
@@ -194,13 +207,15 @@ class PagedAttention(Mixer):
                       "o_bias": "o_proj.bias", "sink": "sinks", **(tensor_names or {})}
 
     def param_specs(self) -> list[ParamSpec]:
-        total = self.q_size + self.kv_size + self.v_size
+        total = self.row_size
         n = self.names
 
         if self.values_are_keys:  # no value projection: q and k alone
             total = self.q_size + self.kv_size
 
         def stacked(q: str, k: str, v: str) -> tuple[ParamSource, ...]:
+            if not self.own_kv:
+                return (ParamSource(n[q], 0, self.q_size),)
             qk = (ParamSource(n[q], 0, self.q_size), ParamSource(n[k], self.q_size, self.kv_size))
             if self.values_are_keys:
                 return qk
@@ -214,10 +229,11 @@ class PagedAttention(Mixer):
         if self.bias:
             specs.append(ParamSpec("qkv_proj.bias", (total,), init="zeros",
                                    sources=stacked("q_bias", "k_bias", "v_bias")))
+        if self.o_bias:
             specs.append(ParamSpec("o_proj.bias", (self.hidden_size,), init="zeros",
                                    sources=(ParamSource(n["o_bias"], 0, self.hidden_size),)))
         if self.qk_norm_eps is not None and self.qk_norm_gain:
-            for key, whole in (("q_norm", self.q_size), ("k_norm", self.kv_size)):
+            for key, whole in (("q_norm", self.q_size), ("k_norm", self.kv_size))[: 2 if self.own_kv else 1]:
                 size = whole if self.wide_norm else self.head_dim
                 specs.append(ParamSpec(key, (size,), kind="vector", init="gain",
                                        sources=(ParamSource(n[key], 0, size),)))
@@ -228,7 +244,9 @@ class PagedAttention(Mixer):
 
     def setup(self, runtime) -> None:
         super().setup(runtime)
-        self._slopes = self._unit_gain = None
+        self._slopes = self._unit_gain = self._sinks = None
+        if self.fixed_sink is not None:
+            self._sinks = torch.full((self.num_heads,), self.fixed_sink, dtype=torch.float32, device=runtime.device)
         if self.distance_slopes is not None:
             self._slopes = torch.tensor(self.distance_slopes, dtype=torch.float32, device=runtime.device)
         if self.head_norm and not self.qk_norm_gain:
@@ -248,8 +266,7 @@ class PagedAttention(Mixer):
             raise ValueError(
                 f"{type(self).__name__} keeps its cache in {need.dtype} beside a model in "
                 f"{self.runtime.dtype}: the attention kernels read keys and values in the model's dtype")
-        if not self._same_sizes() or self.runtime.dtype != torch.bfloat16 or not ops.decode_attention_supported(
-                self.num_heads, self.num_kv_heads, self.head_dim, limits.page_size, self.runtime.dtype):
+        if not self._decode_kernel(limits.page_size, self.runtime.dtype):
             return
         widest = ops.decode_attention_max_table(self.num_heads, self.num_kv_heads, self.head_dim)
         if limits.max_pages_per_seq > widest:
@@ -262,20 +279,26 @@ class PagedAttention(Mixer):
     def product_weights(self) -> tuple[str, ...]:
         return ("qkv_proj.weight", "o_proj.weight")
 
-    def _same_sizes(self) -> bool:
-        """Keys and values of one size in every plane: what the matrix-core kernels serve."""
-        return self.v_plane_dim == self.head_dim
+    def _decode_kernel(self, page_size: int, dtype) -> bool:
+        """Whether the matrix-core kernel for single tokens serves these heads (a plane of values as
+        wide as the keys or half as wide)."""
+        return ops.decode_attention_supported(self.num_heads, self.num_kv_heads, self.head_dim, page_size, dtype,
+                                              self.v_plane_dim)
+
+    def _prefill_kernel(self, page_size: int, dtype) -> bool:
+        """The same for the matrix-core kernel for portions of prompts."""
+        return self.scale > 0 and ops.prefill_attention_supported(
+            self.num_heads, self.num_kv_heads, self.head_dim, page_size, dtype, self.v_plane_dim)
 
     def forward(self, x, ctx, call, sink=None):
         return self._output(self._attention(self._project(x, ctx), ctx, call), ctx, sink)
 
     def _project(self, x, ctx):
-        """Rows ``[q heads | k heads | v heads]`` for the step's tokens, normed over the whole
+        """Rows ``[q heads | k heads | v heads]`` (queries alone without ``own_kv``) for the step's tokens, normed over the whole
         projection where the layer says so (norms of single heads and rotation come later)."""
         p = self.params
         # step buffers are named by their width: layers of one model may differ in size
-        qkv = ctx.buf(_sized("attn_qkv", self.q_size + self.kv_size + self.v_size, self.shared_buffers),
-                      self.q_size + self.kv_size + self.v_size)
+        qkv = ctx.buf(_sized("attn_qkv", self.row_size, self.shared_buffers), self.row_size)
         if self.values_are_keys:
             ops.linear(qkv[:, : self.q_size + self.kv_size], x, p["qkv_proj.weight"], p.get("qkv_proj.bias"))
             if not self.wide_norm:  # the values are the keys as projected
@@ -309,21 +332,26 @@ class PagedAttention(Mixer):
             attn = ctx.buf(f"attn_out_f32:{self.o_size}", self.o_size, torch.float32)
         else:
             attn = ctx.buf(_sized("attn_out", self.o_size, self.shared_buffers), self.o_size)
+        q_gain = p.get("q_norm", self._unit_gain) if self.head_norm else None
+        k_gain = p.get("k_norm", self._unit_gain) if self.head_norm else None
         # with a norm of the heads, or values of another size than the keys, one kernel norms,
         # rotates and writes the cache; the attention kernels then take q and the cache as they are
-        prepared = not self.plain
+        # (the kernel for single tokens does all of that itself)
+        single = ctx.max_query_len == 1 and self.v_planes == 1 and self._decode_kernel(group.page_size, qkv.dtype)
+        prepared = not self.plain and not single
         if prepared:
             kv_slot = self._kv_slots(ctx, call, group, k_cache)
             ops.qk_norm_rope_kv_write(qkv, k_cache, v_planes, cos, sin, rot_dim=rot_dim,
                                       interleaved=interleaved, kv_slot=kv_slot, nh=self.num_heads,
                                       nkv=self.num_kv_heads, d=self.head_dim, dv=self.v_head_dim,
-                                      q_gain=p.get("q_norm", self._unit_gain) if self.head_norm else None,
-                                      k_gain=p.get("k_norm", self._unit_gain) if self.head_norm else None,
-                                      eps=self.qk_norm_eps or 0.0, write_kv=call.write_cache)
+                                      q_gain=q_gain, k_gain=k_gain if self.own_kv else q_gain,
+                                      eps=self.qk_norm_eps or 0.0, write_kv=call.write_cache and self.own_kv,
+                                      queries_only=not self.own_kv)
             rot_dim, interleaved = 0, False
             cos = sin = ctx.buffers.get("rope_none", ctx.num_tokens, 0, torch.float32)
         if self.v_planes == 1:
-            self._attend(attn, qkv, k_cache, v_planes[0], ctx, call, group, cos, sin, rot_dim, interleaved, prepared)
+            self._attend(attn, qkv, k_cache, v_planes[0], ctx, call, group, cos, sin, rot_dim, interleaved, prepared,
+                         q_gain, k_gain)
         else:
             # the same scores against each plane of the values; the planes' results, each [T, heads
             # * plane size], are then laid side by side within every head
@@ -332,7 +360,7 @@ class PagedAttention(Mixer):
                                     reserve=m * ctx.buffers.token_capacity)
             for c in range(m):
                 self._attend(parts[c * T: (c + 1) * T], qkv, k_cache, v_planes[c], ctx, call, group, cos, sin,
-                             rot_dim, interleaved, prepared)
+                             rot_dim, interleaved, prepared, q_gain, k_gain)
             attn.view(T, self.num_heads, m, self.v_plane_dim).copy_(
                 parts.view(m, T, self.num_heads, self.v_plane_dim).permute(1, 2, 0, 3))
         return attn
@@ -348,22 +376,21 @@ class PagedAttention(Mixer):
         ops.linear(out, attn, p["o_proj.weight"], p.get("o_proj.bias"))
         return out
 
-    def _attend(self, attn, qkv, k_cache, v_cache, ctx, call, group, cos, sin, rot_dim, interleaved, prepared):
+    def _attend(self, attn, qkv, k_cache, v_cache, ctx, call, group, cos, sin, rot_dim, interleaved, prepared,
+                q_gain=None, k_gain=None):
         """The attention itself into ``attn [T, heads * plane size]`` over one plane of values,
         by the kernel that serves the step's shape.  ``prepared``: q is ready and the cache is
         written; otherwise the kernels chosen here rotate and write on their way."""
         common = dict(table=group.table, positions=ctx.positions, token_req=ctx.token_req,
                       slots=ctx.slots, nh=self.num_heads, nkv=self.num_kv_heads, d=self.head_dim,
-                      scale=self.scale, window=self.window)
+                      dv=self.v_plane_dim, scale=self.scale, window=self.window)
         x_dtype = qkv.dtype
         # a distance bias and a chunked view are options of every attention kernel
-        common.update(slopes=self._slopes, chunk=self.chunk, sinks=self.params.get("sinks"))
+        sinks = self.params.get("sinks", self._sinks)
+        common.update(slopes=self._slopes, chunk=self.chunk, sinks=sinks)
         # a token never sees more keys than its window or its chunk holds: what the launch plans count
         reach = min((n for n in (self.window, self.chunk) if n > 0), default=0)
-        if not self._same_sizes():
-            ops.paged_attention(attn, qkv, k_cache, v_cache, dv=self.v_plane_dim, **common)
-        elif ctx.max_query_len == 1 and ops.decode_attention_supported(
-                self.num_heads, self.num_kv_heads, self.head_dim, group.page_size, x_dtype):
+        if ctx.max_query_len == 1 and self._decode_kernel(group.page_size, x_dtype):
             # single tokens: rotation, cache write and attention in one kernel on the matrix
             # cores, a block per (token, kv head, split)
             T = ctx.num_tokens
@@ -375,18 +402,18 @@ class PagedAttention(Mixer):
                 # for the largest at once, since a buffer that grows drops the graphs
                 most = (decode_target_blocks() // self.num_kv_heads + 1 + max(T, ctx.buffers.seq_capacity)) \
                     * self.num_heads
-                part_o = ctx.buffers.get(_sized("attn_part_o", self.head_dim, self.shared_buffers),
-                                         T * self.num_heads * nsplit, self.head_dim,
+                part_o = ctx.buffers.get(_sized("attn_part_o", self.v_plane_dim, self.shared_buffers),
+                                         T * self.num_heads * nsplit, self.v_plane_dim,
                                          torch.float32, reserve=most)
                 part_ml = ctx.buffers.get("attn_part_ml", T * self.num_heads * nsplit, 2, torch.float32,
                                           reserve=most)
             ops.decode_attention(attn, qkv, k_cache, v_cache, nsplit=nsplit, part_o=part_o,
                                  part_ml=part_ml, cos=cos, sin=sin, rot_dim=rot_dim,
-                                 interleaved=interleaved, write_kv=call.write_cache and not prepared,
-                                 token_rows=ctx.token_rows, **common)
+                                 interleaved=interleaved, write_kv=call.write_cache and self.own_kv and not prepared,
+                                 token_rows=ctx.token_rows, **({} if prepared or not self.head_norm else dict(
+                                     q_gain=q_gain, k_gain=k_gain, eps=self.qk_norm_eps)), **common)
         else:
-            on_matrix_cores = ctx.max_query_len > 1 and self.scale > 0 and ops.prefill_attention_supported(
-                self.num_heads, self.num_kv_heads, self.head_dim, group.page_size, x_dtype)
+            on_matrix_cores = ctx.max_query_len > 1 and self._prefill_kernel(group.page_size, x_dtype)
             # the kernel for portions rotates the queries on their way in where it can, which
             # saves writing them and reading them again
             rotates = on_matrix_cores and ops.prefill_attention_rotates(rot_dim, interleaved)
@@ -405,16 +432,16 @@ class PagedAttention(Mixer):
                 if nsplit > 1:
                     # asked for at their largest at once: a buffer that grows drops the graphs
                     most = prefill_split_rows(self.num_kv_heads, self.num_heads // self.num_kv_heads) * self.num_heads
-                    part_o = ctx.buffers.get(_sized("attn_prefill_part_o", self.head_dim, self.shared_buffers),
+                    part_o = ctx.buffers.get(_sized("attn_prefill_part_o", self.v_plane_dim, self.shared_buffers),
                                              T * self.num_heads * nsplit,
-                                             self.head_dim, torch.float32, reserve=most)
+                                             self.v_plane_dim, torch.float32, reserve=most)
                     part_ml = ctx.buffers.get("attn_prefill_part_ml", T * self.num_heads * nsplit, 2,
                                               torch.float32, reserve=most)
                 ops.prefill_attention(attn, qkv, k_cache, v_cache, table=group.table,
                                       positions=ctx.positions, q_start=ctx.q_start, slots=ctx.slots,
                                       num_reqs=ctx.num_reqs, nh=self.num_heads, nkv=self.num_kv_heads,
-                                      d=self.head_dim, scale=self.scale, window=self.window,
-                                      slopes=self._slopes, chunk=self.chunk, sinks=self.params.get("sinks"),
+                                      d=self.head_dim, dv=self.v_plane_dim, scale=self.scale, window=self.window,
+                                      slopes=self._slopes, chunk=self.chunk, sinks=sinks,
                                       nsplit=nsplit, part_o=part_o, part_ml=part_ml,
                                       **(dict(cos=cos, sin=sin, rot_dim=rot_dim, interleaved=interleaved)
                                          if rotates else {}))

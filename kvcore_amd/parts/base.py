@@ -35,8 +35,9 @@ class ParamSource:
 
 def checkpoint_name(prefix: str, name: str) -> str:
     """The checkpoint tensor that a source names: ``prefix.name``, or the prefix itself for an
-    empty name (a part whose one tensor is called as the part is)."""
-    return f"{prefix}.{name}" if name else prefix
+    empty name (a part whose one tensor is called as the part is), or the name itself for an empty
+    prefix (a part whose tensors stand at the top)."""
+    return f"{prefix}.{name}" if name and prefix else prefix or name
 
 
 @dataclass(frozen=True)
@@ -215,10 +216,18 @@ class RotaryTables:
 class Embedding(Part):
     """Token ids to rows of the residual stream: ``forward`` writes ``residual [T, H]``
     (float32) for ``token_ids [T]`` (int32 on the device).  A parameter named ``weight`` of
-    shape ``[vocab, hidden]`` is what a tied head shares."""
+    shape ``[vocab, hidden]`` is what a tied head shares.  An embedding that needs more of the step than
+    its tokens, or keeps per-request state (``state_needs``, as for :class:`Mixer`), overrides
+    ``forward_step``; ``state_indices`` name its arrays in ``ctx.states``."""
+
+    def state_needs(self) -> tuple[StateNeed, ...]:
+        return ()
 
     def forward(self, residual: torch.Tensor, token_ids: torch.Tensor) -> None:
         raise NotImplementedError
+
+    def forward_step(self, residual: torch.Tensor, ctx: "StepContext", state_indices: tuple[int, ...]) -> None:
+        self.forward(residual, ctx.token_ids[: ctx.num_tokens])
 
 
 class Head(Part):
@@ -276,11 +285,14 @@ class StreamOp(Part):
 
 
 class FeedForward(Part):
-    """``takes_scaled_rows``, ``takes_sink`` and ``takes_slice_sink`` as for :class:`Mixer`."""
+    """``takes_scaled_rows``, ``takes_sink`` and ``takes_slice_sink`` as for :class:`Mixer`.
+    ``gives_weighted_rows``: the part has a method ``forward_weighted`` that returns its result as
+    ``ops.WeightedRows``, for a block whose next kernel adds them up."""
 
     takes_scaled_rows = False
     takes_sink = False
     takes_slice_sink = False
+    gives_weighted_rows = False
 
     def forward(self, x: torch.Tensor, ctx: "StepContext", call: "LayerCall") -> torch.Tensor:
         raise NotImplementedError

@@ -180,7 +180,8 @@ class SandwichNormBlock(Block):
     def _join(self, result, residual, ctx, post, following, name: str):
         """``residual += post(result)``, and the rows of the norm ``following`` (a (gain, eps) or
         None) into the step buffer ``name``.  ``result`` is a tensor or the partial sums that a
-        part's last product left (``ops.SlicedRows``)."""
+        part's last product left (``ops.SlicedRows``), or the results of a feed-forward's experts
+        (``ops.WeightedRows``)."""
         post_gain, post_eps = post
         if following is None:
             ops.norm_add_norm(None, residual, result, post_gain, post_eps)
@@ -215,7 +216,10 @@ class SandwichNormBlock(Block):
             return None if rows is None else ops.NormedRows(rows)
         x2 = self._join(a, residual, ctx, self._gain(1), self._gain(2), "block_x2")
         sink = self._slice_sink(self.ffn, residual, ctx)
-        f = self.ffn.forward(x2, ctx, call) if sink is None else self.ffn.forward(x2, ctx, call, sink=sink)
+        if self.ffn.gives_weighted_rows:  # the norm behind the experts adds their results up
+            f = self.ffn.forward_weighted(x2, ctx, call)
+        else:
+            f = self.ffn.forward(x2, ctx, call) if sink is None else self.ffn.forward(x2, ctx, call, sink=sink)
         rows = self._join(f, residual, ctx, self._gain(3), following, "block_x")
         return None if rows is None else ops.NormedRows(rows)
 

@@ -13,7 +13,7 @@ import torch
 
 from kvcore_amd.ops import library as ops
 
-from .base import Embedding, Head, ParamSource, ParamSpec, register_embedding, register_head
+from .base import Embedding, Head, ParamSource, ParamSpec, StateNeed, register_embedding, register_head
 
 
 class TokenEmbedding(Embedding):
@@ -37,6 +37,35 @@ class TokenEmbedding(Embedding):
         ops.embed(residual, self.params["weight"], token_ids, self.scale)
 
 
+class PairEmbedding(Embedding):
+    """A token's row plus the row of the pair (token before, token): ``table[token] + pairs[(prev *
+    mul_prev + token * mul_cur) mod buckets]``, the sum in float32; a sequence's first token takes the
+    row behind the buckets.  The token before the first of a step's tokens is the request's state: one
+    int32 a slot."""
+
+    def __init__(self, *, vocab_size: int, hidden_size: int, buckets: int, mul_prev: int, mul_cur: int,
+                 weight_name: str = "weight", pairs_name: str = "pairs.weight") -> None:
+        """``weight_name`` and ``pairs_name``: the two checkpoint tensors relative to the part's prefix."""
+        if buckets < 1 or mul_prev < 0 or mul_cur < 0:
+            raise ValueError(f"{buckets} buckets, multipliers {mul_prev} and {mul_cur}")
+        self.vocab_size, self.hidden_size = vocab_size, hidden_size
+        self.buckets, self.mul_prev, self.mul_cur = int(buckets), int(mul_prev), int(mul_cur)
+        self.names = (weight_name, pairs_name)
+
+    def param_specs(self) -> list[ParamSpec]:
+        shapes = (("weight", self.names[0], self.vocab_size), ("pairs", self.names[1], self.buckets + 1))
+        return [ParamSpec(name, (rows, self.hidden_size), sources=(ParamSource(tensor, 0, rows),))
+                for name, tensor, rows in shapes]
+
+    def state_needs(self) -> tuple[StateNeed, ...]:
+        return (StateNeed((1,), torch.int32),)
+
+    def forward_step(self, residual: torch.Tensor, ctx, state_indices: tuple[int, ...]) -> None:
+        ops.embed_pairs(residual, self.params["weight"], self.params["pairs"], ctx.token_ids,
+                        ctx.states[state_indices[0]], mul_prev=self.mul_prev, mul_cur=self.mul_cur,
+                        positions=ctx.positions, token_req=ctx.token_req, q_start=ctx.q_start, slots=ctx.slots)
+
+
 class LinearHead(Head):
     """``logits = hidden @ W.T (+ bias)``, then ``soft_cap * tanh(logits / soft_cap)`` if
     ``soft_cap > 0``, then ``* logit_scale``.  ``tied`` heads own no matrix; the model binds
@@ -44,6 +73,7 @@ class LinearHead(Head):
 
     def __init__(self, *, vocab_size: int, hidden_size: int, tied: bool = False, bias: bool = False,
                  logit_scale: float = 1.0, soft_cap: float = 0.0, weight_name: str = "weight") -> None:
+        """``weight_name``: the checkpoint tensor relative to the part's prefix (empty: the prefix itself)."""
         if soft_cap < 0:
             raise ValueError(f"soft_cap must be positive when set, got {soft_cap}")
         self.vocab_size = vocab_size
@@ -80,4 +110,5 @@ class LinearHead(Head):
 OutputHead = LinearHead
 
 register_embedding("token_embedding", TokenEmbedding)
+register_embedding("pair_embedding", PairEmbedding)
 register_head("linear_head", LinearHead)

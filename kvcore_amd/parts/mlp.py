@@ -1,11 +1,13 @@
 """Gated feed-forward: ``down(act(gate(x)) * up(x))`` with gate and up stacked; ``act`` is silu
-unless the layer names another (``gelu_tanh``).
+unless the layer names another (``gelu_tanh``, or ``clamped``, which bounds both branches).
 
 Reference: kvcore/model/models/llama3.py:25-45 (gate rows first, then up rows) and
 kvcore/model/layer/activation.py:14-16.
 """
 
 from __future__ import annotations
+
+import math
 
 import torch
 
@@ -30,16 +32,18 @@ class SwiGLU(FeedForward):
     def __init__(self, *, hidden_size: int, intermediate_size: int, bias: bool = False,
                  gate_name: str = "gate_proj", up_name: str = "up_proj", down_name: str = "down_proj",
                  suffix: str = ".weight", sized_buffers: bool = False, activation: str = "silu",
-                 float32_result: bool = False) -> None:
+                 float32_result: bool = False, limit: float = math.inf, alpha: float = 1.0,
+                 up_shift: float = 0.0) -> None:
         """``gate_name``, ``up_name`` and ``down_name`` are the checkpoint's names of the three
         matrices relative to the part's prefix, ``suffix`` what follows each (biases end in
         ``.bias``).  ``sized_buffers``: name the step buffers by their width, for a model whose
         layers may differ in width (a buffer whose width changed from layer to layer would be
-        allocated anew at every layer).  ``activation``: the gate's, ``silu`` or ``gelu_tanh``.
+        allocated anew at every layer).  ``activation``: the gate's, ``silu``, ``gelu_tanh`` or
+        ``clamped`` (``ops.GateAct``; ``limit``, ``alpha`` and ``up_shift`` are its constants).
         ``float32_result``: the output rows are float32 sums, for a consumer that normalises them."""
         if activation not in ops.GATE_ACTS:
             raise ValueError(f"gate activation {activation!r} is not supported (supported: {sorted(ops.GATE_ACTS)})")
-        self.activation = activation
+        self.activation = ops.GateAct(activation, float(limit), float(alpha), float(up_shift))
         self.float32_result = float32_result
         self.hidden_size = hidden_size
         self.intermediate_size = intermediate_size

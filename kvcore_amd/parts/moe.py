@@ -1,15 +1,19 @@
 """A feed-forward of routed experts: every token runs the few experts its router chooses.
 
-    scores = softmax(W_r h), or sigmoid(W_r h) element by element            (float32)
+    logits = W_r h (+ a learned bias per expert, where the layer has one)      (float32)
+    scores = softmax(logits), sigmoid(logits) element by element, or the logits as they are
     choice = the `top` best experts, by score (+ a learned correction per expert, where the layer
              has one), among those of the `keep` best of `groups` equal groups of neighbouring
              experts (a group is as good as its best expert, or as the sum of its best two)
-    weight = scores[choice] / (sum of them + 1e-20) * weight_scale    (the scores without the correction)
-    out    = sum_c weight_c * expert_choice_c(h)  (+ shared(h), an expert that every token runs)
+    weight = scores[choice] / (sum of them + 1e-20) * weight_scale    (the scores without the correction);
+             where the scores are the logits, the softmax over the chosen logits * weight_scale
+    out    = sum_c weight_c * expert_choice_c(h)  (+ shared(h), an expert that every token runs, times
+             sigmoid(w_sg . h), one number a token, where the layer has that vector)
 
 An expert is a gated feed-forward with a clamped activation: ``g = min(W_gate h, limit)``, ``u =
 clamp(W_up h, -limit, limit)``, ``W_down (g * sigmoid(alpha g) * (u + up_shift))``; an infinite
-limit, ``alpha`` 1 and ``up_shift`` 0 make it ``W_down (silu(W_gate h) * W_up h)``.  The experts' matrices are
+limit, ``alpha`` 1 and ``up_shift`` 0 make it ``W_down (silu(W_gate h) * W_up h)``; the shared expert has
+the same form with a size and a limit of its own.  The experts' matrices are
 stacked along a leading expert dimension (each expert's gate rows, then its up rows), the routing
 stays on the device and every launch is sized by the step's token count alone, so a step may be
 captured into a graph.  The result is float32 rows: the weighted sum is not rounded before it
@@ -32,18 +36,21 @@ GLU_ALPHA = 1.702
 class RoutedExperts(FeedForward):
     """``experts`` experts of ``expert_size`` hidden units, ``top`` a token; ``groups`` and
     ``keep`` as above (1 and 1: every expert may be chosen); ``shared_size`` > 0 adds the shared
-    expert (``shared_limit`` its clamp).  ``limit`` None: no clamp.  ``score``: ``softmax`` or
-    ``sigmoid``; ``correction``: the layer has a learned value per expert (tensor ``correction``)
+    expert (``shared_limit`` its clamp), ``shared_gate`` its gate (tensor ``shared_gate``, a row behind the
+    router's in memory).  ``limit`` None: no clamp.  ``score``: ``softmax``, ``sigmoid`` or ``logit``;
+    ``router_bias``: the logits have a bias (tensor ``router_bias``); ``correction``: the layer has a learned value per expert (tensor ``correction``)
     that joins the scores for the choice alone; ``group_best``: a group is worth its best 1 or 2
     choice scores; ``weight_scale`` multiplies the weights; ``up_shift`` is added to the up branch.
-    ``tensor_names`` renames checkpoint tensors (keys: router, correction, expert (a pattern with
-    ``{e}``), shared, gate, up, down)."""
+    ``tensor_names`` renames checkpoint tensors (keys: router, router_bias, correction, expert (a
+    pattern with ``{e}``), shared, shared_gate, gate, up, down)."""
+
+    gives_weighted_rows = True
 
     def __init__(self, *, hidden_size: int, experts: int, top: int, expert_size: int, limit: float | None,
                  groups: int = 1, keep: int = 1, shared_size: int = 0, shared_limit: float | None = None,
                  alpha: float = GLU_ALPHA, score: str = "softmax", correction: bool = False, group_best: int = 1,
-                 weight_scale: float = 1.0, up_shift: float = 1.0,
-                 tensor_names: dict[str, str] | None = None) -> None:
+                 weight_scale: float = 1.0, up_shift: float = 1.0, router_bias: bool = False,
+                 shared_gate: bool = False, tensor_names: dict[str, str] | None = None) -> None:
         if experts <= 0 or not 0 < top <= experts or expert_size <= 0:
             raise ValueError(f"{top} of {experts} experts of {expert_size} units")
         if groups <= 0 or experts % groups or not 0 < keep <= groups:
@@ -54,15 +61,20 @@ class RoutedExperts(FeedForward):
         if score not in ops.ROUTE_SCORES or group_best not in (1, 2):
             raise ValueError(f"router scores by {sorted(ops.ROUTE_SCORES)}, groups by their best 1 or 2; "
                              f"got {score!r} and {group_best}")
-        if shared_size and (limit is None or up_shift != 1.0):
-            raise ValueError("the shared expert's kernel has the clamped activation with an up branch plus one")
+        if shared_gate and not shared_size:
+            raise ValueError("a gate for a shared expert that the layer does not have")
         limit = math.inf if limit is None else float(limit)
         self.limit, self.groups, self.keep, self.alpha = limit, groups, keep, float(alpha)
         self.score, self.has_correction, self.group_best = score, bool(correction), int(group_best)
         self.weight_scale, self.up_shift = float(weight_scale), float(up_shift)
         self.shared_size = shared_size
         self.shared_limit = float(limit if shared_limit is None else shared_limit)
-        self.names = {"router": "router.weight", "correction": "correction", "expert": "experts.{e}", "shared": "shared",
+        self.has_shared_gate, self.has_router_bias = bool(shared_gate), bool(router_bias)
+        plain = math.isinf(self.shared_limit) and self.alpha == 1.0 and self.up_shift == 0.0
+        self.shared_act = ops.GateAct("silu") if plain else ops.GateAct("clamped", self.shared_limit, self.alpha,
+                                                                        self.up_shift)
+        self.names = {"router": "router.weight", "router_bias": "router.bias", "correction": "correction",
+                      "expert": "experts.{e}", "shared": "shared", "shared_gate": "shared_gate.weight",
                       "gate": "gate.weight", "up": "up.weight", "down": "down.weight", **(tensor_names or {})}
 
     def param_specs(self) -> list[ParamSpec]:
@@ -73,11 +85,17 @@ class RoutedExperts(FeedForward):
             gate_up.append(ParamSource(f"{prefix}.{n['gate']}", 2 * I * e, I))
             gate_up.append(ParamSource(f"{prefix}.{n['up']}", 2 * I * e + I, I))
             down.append(ParamSource(f"{prefix}.{n['down']}", H * e, H))
+        router = [ParamSource(n["router"], 0, E)]
+        if self.has_shared_gate:  # one more row: its product with the token is the shared expert's gate
+            router.append(ParamSource(n["shared_gate"], E, 1))
         specs = [
-            ParamSpec("router.weight", (E, H), kind="vector", init="normal", sources=(ParamSource(n["router"], 0, E),)),
+            ParamSpec("router.weight", (E + len(router) - 1, H), kind="vector", init="normal", sources=tuple(router)),
             ParamSpec("experts.gate_up", (2 * I * E, H), sources=tuple(gate_up)),
             ParamSpec("experts.down", (H * E, I), sources=tuple(down)),
         ]
+        if self.has_router_bias:
+            specs.append(ParamSpec("router.bias", (E,), kind="vector", init="normal",
+                                   sources=(ParamSource(n["router_bias"], 0, E),)))
         if self.has_correction:
             specs.append(ParamSpec("correction", (E,), kind="vector", init="normal",
                                    sources=(ParamSource(n["correction"], 0, E),)))
@@ -99,15 +117,24 @@ class RoutedExperts(FeedForward):
         self.forward(x, ctx, call, into=residual, add=add)
 
     def forward(self, x, ctx, call, sink=None, into=None, add=None):
+        rows = self.forward_weighted(x, ctx, call)
+        out = ctx.buf("ffn_out_f32", self.hidden_size, torch.float32) if into is None else into
+        ops.moe_combine(out, rows.data, rows.weight, add if into is not None else None, rows.add,
+                        accumulate=into is not None, add1_gate=rows.add_gate)
+        return out
+
+    def forward_weighted(self, x, ctx, call) -> "ops.WeightedRows":
+        """The experts' results with their weights, and the shared expert's with its gate."""
         p, H, E, I, top = self.params, self.hidden_size, self.experts, self.expert_size, self.top
         T = ctx.num_tokens
         pairs = T * top
         # the router reads the rows as they are and sums in float32; logits and choice in one kernel
         choice = ctx.buf(f"moe_choice:{top}", top, torch.int32)
         weight = ctx.buf(f"moe_weight:{top}", top, torch.float32)
+        gate = ctx.buf("moe_shared_gate", 1, torch.float32) if self.has_shared_gate else None
         ops.moe_router(choice, weight, x, p["router.weight"], top=top, groups=self.groups, keep=self.keep,
                        score=self.score, correction=p.get("correction"), group_best=self.group_best,
-                       weight_scale=self.weight_scale)
+                       weight_scale=self.weight_scale, bias=p.get("router.bias"), gate=gate)
         cap = ctx.buffers.token_capacity
         sorted_pairs = ctx.buffers.get(f"moe_sorted:{top}", pairs, 1, torch.int32, reserve=cap * top).view(-1)
         # portions of prompts give the experts rows enough for tiles of 64, single tokens tiles of 16
@@ -127,18 +154,12 @@ class RoutedExperts(FeedForward):
         shared = None
         if self.shared_size:
             S = self.shared_size
-            gate_up = ctx.buf(f"moe_shared_gu:{2 * S}", 2 * S)
-            ops.linear(gate_up, x, p["shared.gate_up"])
             sact = ctx.buf(f"moe_shared_act:{S}", S)
-            ops.clamped_glu(sact, gate_up, self.shared_limit, self.alpha)
+            ops.linear_silu_mul(sact, x, p["shared.gate_up"], None, lambda: ctx.buf(f"moe_shared_gu:{2 * S}", 2 * S),
+                                act=self.shared_act)
             shared = ctx.buf(f"moe_shared_out:{H}", H, torch.float32)
             ops.linear(shared, sact, p["shared.down"])
-        if into is not None:
-            ops.moe_combine(into, y, weight, shared, add, accumulate=True)
-            return into
-        out = ctx.buf("ffn_out_f32", H, torch.float32)
-        ops.moe_combine(out, y, weight, shared, None)
-        return out
+        return ops.WeightedRows(y, weight, shared, gate)
 
 
 register_feed_forward("routed_experts", RoutedExperts)

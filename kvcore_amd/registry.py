@@ -82,5 +82,10 @@ def _register_builtin() -> None:
 
     register_architecture("Darovik", DarovikConfig.from_dict, darovik_spec)
 
+    from kvcore_amd.config.sopulorn_config import SopulornConfig
+    from kvcore_amd.models.sopulorn import sopulorn_spec
+
+    register_architecture("Sopulorn", SopulornConfig.from_dict, sopulorn_spec)
+
 
 _register_builtin()
