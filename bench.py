@@ -20,7 +20,8 @@ Other workloads print a line of their own: ``--only-prefill``, ``--mixed`` (64 r
 with prompts of 16 to 2,048 tokens in portions of 512), ``--long-prompt N`` (time to the
 first token of one N-token prompt in portions of 2,048), ``--sweep`` (decode at further
 batch sizes and context lengths, a line each with its share of the memory bandwidth);
-``--model 1b|70b`` and ``--batch`` change the shape.  ``--darovik s|m`` times the Darovik decoder
+``--model 1b|70b`` and ``--batch`` change the shape.  ``--sopulorn s|m`` times the Sopulorn decoder
+beside the Vovalix and the Llama of equal width and depth.  ``--darovik s|m`` times the Darovik decoder
 beside the Tazunex, the Vovalix and the Llama of equal width and depth.  ``--tazunex s|m`` times the Tazunex
 decoder beside the Vovalix and the Llama of equal width and depth.  ``--vovalix s|m`` times the Vovalix
 decoder beside the Dirulorn of equal size.  ``--dirulorn s|m`` times the Dirulorn
@@ -169,6 +170,40 @@ DAROVIK_SHAPES = {
     "m": {"architecture": "Darovik", "vocab": 32000, "width": 2048, "norm": {"eps": 1e-5}, "residual_mult": 0.7,
           "streams": 4, "layers": _darovik_layers(16, 2048, 16, 4, 8192, 32, 4, 8, 4, 1024)},
 }
+
+
+def _sopulorn_layers(n, width, heads, kv, ff, experts, top):
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": experts, "top": top}, "shared": {"ff": ff // 4}}
+    mixer = {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 64, "scale": 0.09,
+             "rot": {"dims": 128, "base": 500000.0}}
+    own = n // 2
+    return [{"type": "attention", "mixer": dict(mixer, kv_from=own - 1) if i >= own else mixer,
+             "mlp": moe if i else dense} for i in range(n)]
+
+
+# Sopulorn at the layer sizes of a real model: attention with keys of 128 and values of 64 in every
+# layer, the second half of the layers reading the cache of the last layer before them; the first
+# layer with the dense feed-forward of the Llama of the same width, the rest with routed experts and
+# a shared one as the Vovalix of the same width has them
+SOPULORN_SHAPES = {
+    "s": {"architecture": "Sopulorn", "vocab": 32000, "width": 1024, "norm": {"eps": 1e-5},
+          "embedding": {"bigram": {"buckets": 60013, "mul_prev": 8191, "mul_cur": 131}},
+          "layers": _sopulorn_layers(8, 1024, 8, 2, 4096, 16, 4)},
+    "m": {"architecture": "Sopulorn", "vocab": 32000, "width": 2048, "norm": {"eps": 1e-5},
+          "embedding": {"bigram": {"buckets": 60013, "mul_prev": 8191, "mul_cur": 131}},
+          "layers": _sopulorn_layers(16, 2048, 16, 4, 8192, 32, 4)},
+}
+
+
+def bench_sopulorn(args) -> int:
+    """The workloads of ``bench_dirulorn`` for a Sopulorn shape beside the Vovalix of the same width
+    and depth (the closest model the engine has: routed experts and a shared one in every layer) and
+    the Llama (attention over every earlier token)."""
+    shapes = (SOPULORN_SHAPES[args.sopulorn], VOVALIX_SHAPES[args.sopulorn], DIRULORN_SHAPES[args.sopulorn][1])
+    names = (f"sopulorn-{args.sopulorn}", f"vovalix-of-sopulorn-{args.sopulorn}", f"llama-of-sopulorn-{args.sopulorn}")
+    which = {"all": (0, 1, 2), "sopulorn": (0,), "vovalix": (1,), "llama": (2,)}[args.sopulorn_only]
+    return _bench_design(args, shapes, names, which, args.sopulorn_workload)
 
 
 def bench_darovik(args) -> int:
@@ -326,6 +361,13 @@ def parse_args():
                    help="with --dirulorn: run one of the two models only (for profiling)")
     p.add_argument("--dirulorn-workload", default="all", choices=["all", "prefill", "decode8", "decode64"],
                    help="with --dirulorn: run one of the workloads only (for profiling)")
+    p.add_argument("--sopulorn", default=None, choices=sorted(SOPULORN_SHAPES),
+                   help="instead of the default run: prefill and decode of the Sopulorn decoder at this size, and "
+                        "of the Vovalix and the Llama of the same width and depth; a line each")
+    p.add_argument("--sopulorn-only", default="all", choices=["all", "sopulorn", "vovalix", "llama"],
+                   help="with --sopulorn: run one of the models only (for profiling)")
+    p.add_argument("--sopulorn-workload", default="all", choices=["all", "prefill", "decode8", "decode64"],
+                   help="with --sopulorn: run one of the workloads only (for profiling)")
     p.add_argument("--darovik", default=None, choices=sorted(DAROVIK_SHAPES),
                    help="instead of the default run: prefill and decode of the Darovik decoder at this size, and "
                         "of the Tazunex, the Vovalix and the Llama of the same width and depth; a line each")
@@ -498,6 +540,8 @@ def main() -> int:
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")
         return 2
+    if args.sopulorn:
+        return bench_sopulorn(args)
     if args.darovik:
         return bench_darovik(args)
     if args.tazunex:
