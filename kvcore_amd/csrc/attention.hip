@@ -365,6 +365,94 @@ __global__ __launch_bounds__(256) void qk_norm_rope_k_write_small_kernel(
   }
 }
 
+// The same in bfloat16 for heads of D = 32, 64, 128 or 256 elements: D / 8 lanes a (token, head), two
+// pieces of four elements a lane, chosen so that both elements of a rotary pair are in one lane: pieces
+// half the rotated width apart (half layout; that half a multiple of 4), or neighbours.
+template <int D>
+__global__ __launch_bounds__(256) void qk_norm_rope_k_write_vec_kernel(
+    bf16_t* __restrict__ qkv, int64_t row_stride, bf16_t* __restrict__ k_cache, const float* __restrict__ q_gain,
+    const float* __restrict__ k_gain, float eps, const float* __restrict__ cos_tab, const float* __restrict__ sin_tab,
+    int rot_dim, int interleaved, const int32_t* __restrict__ kv_slot, int num_tokens, int nh, int nkv, int page_size,
+    int write_kv) {
+  constexpr int L = D / 8;
+  const int sub = threadIdx.x % L;
+  const int heads = nh + nkv;
+  const int64_t item = static_cast<int64_t>(blockIdx.x) * (256 / L) + threadIdx.x / L;
+  const bool there = item < static_cast<int64_t>(num_tokens) * heads;
+  const int t = there ? static_cast<int>(item / heads) : 0;
+  const int head = there ? static_cast<int>(item - static_cast<int64_t>(t) * heads) : 0;
+  const int slot = kv_slot[t];
+  const int half = rot_dim / 2;
+  // first elements of the lane's two pieces: lanes 0 .. half / 4 hold the pairs of the half layout; what
+  // is left (everything, of neighbouring pairs) is dealt out in runs of eight
+  const bool apart = !interleaved && 4 * sub < half;
+  const int p0 = apart ? 4 * sub : 8 * sub;
+  const int p1 = apart ? p0 + half : p0 + 4;
+  bf16_t* hp = qkv + static_cast<int64_t>(t) * row_stride + static_cast<int64_t>(head) * D;
+  float x[2][4];
+#pragma unroll
+  for (int c = 0; c < 2; ++c) {
+    const uint2 w = *reinterpret_cast<const uint2*>(hp + (c ? p1 : p0));
+    x[c][0] = __uint_as_float(w.x << 16);
+    x[c][1] = __uint_as_float(w.x & 0xffff0000u);
+    x[c][2] = __uint_as_float(w.y << 16);
+    x[c][3] = __uint_as_float(w.y & 0xffff0000u);
+  }
+  if (q_gain != nullptr) {  // both or neither; every lane takes part in the exchange
+    const float* gain = head < nh ? q_gain : k_gain;
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) ss = fmaf(x[c][i], x[c][i], ss);
+#pragma unroll
+    for (int o = L / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, kWave);
+    const float inv = 1.f / sqrtf(ss / static_cast<float>(D) + eps);
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x[c][i] = x[c][i] * inv * gain[(c ? p1 : p0) + i];
+  }
+  const float* cs = cos_tab + static_cast<int64_t>(t) * half;
+  const float* sn = sin_tab + static_cast<int64_t>(t) * half;
+  float y[2][4];
+  if (apart) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float c = cs[p0 + i], s = sn[p0 + i];
+      y[0][i] = rotate_first(x[0][i], x[1][i], c, s);
+      y[1][i] = rotate_second(x[0][i], x[1][i], c, s);
+    }
+  } else {
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        const int j = (c ? p1 : p0) / 2 + i;  // a neighbouring pair's angle
+        const float a = x[c][2 * i], b = x[c][2 * i + 1];
+        const bool turned = interleaved && j < half;
+        const float cc = turned ? cs[j] : 1.f, s = turned ? sn[j] : 0.f;
+        y[c][2 * i] = turned ? rotate_first(a, b, cc, s) : a;
+        y[c][2 * i + 1] = turned ? rotate_second(a, b, cc, s) : b;
+      }
+  }
+  if (!there || slot == -2) return;  // a padding token is left alone
+  bf16_t* kc = nullptr;
+  if (head >= nh && write_kv && slot >= 0) {
+    const int page = slot / page_size, off = slot - page * page_size;
+    kc = k_cache + ((static_cast<int64_t>(page) * nkv + (head - nh)) * page_size + off) * D;
+  }
+#pragma unroll
+  for (int c = 0; c < 2; ++c) {
+    uint2 r;
+    r.x = f32_to_bf16_bits(y[c][0]) | (static_cast<uint32_t>(f32_to_bf16_bits(y[c][1])) << 16);
+    r.y = f32_to_bf16_bits(y[c][2]) | (static_cast<uint32_t>(f32_to_bf16_bits(y[c][3])) << 16);
+    const int p = c ? p1 : p0;
+    *reinterpret_cast<uint2*>(hp + p) = r;
+    if (kc != nullptr) *reinterpret_cast<uint2*>(kc + p) = r;
+  }
+}
+
 // The values of eight consecutive tokens a block, for steps of many tokens.  A V page keeps the
 // keys side by side, so a token alone stores its values two or four bytes at a time, page_size
 // elements apart; when the block's eight tokens lie side by side in one page (a portion of a
@@ -441,6 +529,31 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
   const bool queries_only = !write_kv && nkv == 0 && T >= 16;
   for (int c = 0; c < num_v_planes; ++c)
     tiled_values = tiled_values && (reinterpret_cast<uintptr_t>(host_v_planes[c]) & 15) == 0;
+  if ((tiled_values || queries_only) && dtype == 1 && (d == 32 || d == 64 || d == 128 || d == 256) &&
+      rot_dim % (interleaved ? 2 : 8) == 0 && row_stride % 8 == 0 && (reinterpret_cast<uintptr_t>(qkv) & 15) == 0 &&
+      (reinterpret_cast<uintptr_t>(k_cache) & 15) == 0) {
+    // many tokens in bfloat16: two pieces of four elements a lane, then the values
+    const int64_t groups = static_cast<int64_t>(T) * (nh + nkv) * (d / 8);
+    const dim3 grid(static_cast<unsigned>((groups + 255) / 256));
+    hipStream_t s = reinterpret_cast<hipStream_t>(stream);
+#define KVC_QK_VEC(D_)                                                                                              \
+  hipLaunchKernelGGL(qk_norm_rope_k_write_vec_kernel<D_>, grid, dim3(256), 0, s, static_cast<bf16_t*>(qkv), row_stride, \
+                     static_cast<bf16_t*>(k_cache), q_gain, k_gain, eps, cos_tab, sin_tab, rot_dim, interleaved,    \
+                     kv_slot, T, nh, nkv, page_size, write_kv)
+    if (d == 32) KVC_QK_VEC(32);
+    else if (d == 64) KVC_QK_VEC(64);
+    else if (d == 128) KVC_QK_VEC(128);
+    else KVC_QK_VEC(256);
+#undef KVC_QK_VEC
+    if (tiled_values) {
+      ValuePlanes<bf16_t> planes{};
+      for (int c = 0; c < num_v_planes; ++c) planes.plane[c] = static_cast<bf16_t*>(host_v_planes[c]);
+      hipLaunchKernelGGL(value_planes_write_tile_kernel<bf16_t>, dim3((T + 7) / 8), dim3(256), 0, s,
+                         static_cast<const bf16_t*>(qkv), row_stride, planes, v_chunk, kv_slot, T, (nh + nkv) * d, nkv,
+                         dv, page_size);
+    }
+    return kvc_check_launch("kvc_qk_norm_rope_kv_write");
+  }
   if ((tiled_values || queries_only) && d <= kWave) {
     // many tokens and heads of up to 64 elements: a wave a head, then the values
     const int64_t waves = static_cast<int64_t>(T) * (nh + nkv);

@@ -750,7 +750,8 @@ int launch_prefill(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t*
     }
   } else {
     single = 1;
-    if (D == 64 && pairs1 > cu / 2 && long_requests) waves = 8;
+    // keys of 128 with values of 64, one request: 2,048 tokens 45.8 against 40.8 us (16 heads over 4)
+    if (long_requests && ((D == 64 && pairs1 > cu / 2) || (D == 128 && DV < D))) waves = 8;
   }
   // KVC_PREFILL_MODE = 1p | 1s | 2p | 2s, then 4 or 8 (waves), overrides the choice for tuning
   static const char* mode = getenv("KVC_PREFILL_MODE");

@@ -183,96 +183,139 @@ __global__ __launch_bounds__(256) void moe_route_kernel(int32_t* __restrict__ ch
             logits + static_cast<int64_t>(t) * E, sc, sc + E, sc + 2 * E, lane, E, rule);
 }
 
-// The router whole: logits = x W^T in float32 (x of either dtype, its values as they are), then the
-// choice as in moe_route_kernel.  A block takes TOK tokens.  Its four waves share K: lane l of wave
-// w sums the products of the values 4 l .. 4 l + 3 of the pieces of 256 that are the wave's (every
-// fourth piece) for each of up to 32 experts at a time (a fetched piece of the router's row meets all
-// TOK tokens); the 256 partial sums of a logit are added in wave and lane order through LDS: one
-// fixed order, whatever the batch.  The first wave then chooses.  With `gate` the matrix has a row
-// behind the experts', whose product's sigmoid goes to gate[t].
-template <typename T, int TOK>
-__global__ __launch_bounds__(256) void moe_router_kernel(int32_t* __restrict__ choice, float* __restrict__ weight,
-                                                         const T* __restrict__ x, int64_t x_stride,
-                                                         const float* __restrict__ wr, float* __restrict__ gate,
-                                                         int T_, int H, int E, RouteRule rule, int vectors) {
-  constexpr int EB = 32, PR = EB + 1;
-  extern __shared__ float lds[];
-  const int wave = threadIdx.x / kWave, lane = threadIdx.x & (kWave - 1);
-  float* part = lds;                       // [256][EB + 1]
-  float* z = lds + 256 * PR;               // [TOK][rows + E + groups]
-  const int rows = gate != nullptr ? E + 1 : E;
-  const int zrow = rows + E + rule.groups;
-  const int t0 = blockIdx.x * TOK;
-  for (int e0 = 0; e0 < rows; e0 += EB) {
-    const int ne = (rows - e0 < EB) ? rows - e0 : EB;
-    float acc[TOK][EB];
+// The router whole: logits = x W^T with float32 products and sums (x of either dtype, its values as
+// they are) on the matrix cores, then the choice as in moe_route_kernel.  A block of sixteen waves takes
+// 16 tokens (the B operand's columns) and up to kRouterRows experts at a time (two A tiles of 16).  The
+// waves share K: wave w takes the pieces of 32 values w, w + 16, ..., of which lane (expert or token li,
+// lk) holds the values from 8 lk on (both operands are dealt the same way, so the eight 16 x 16 x 4
+// products of a piece sum over all of it).  The waves' partial sums are added in wave order through LDS:
+// one fixed order, whatever the batch.  Every wave then chooses for one token.  With `gate` the matrix
+// has a row behind the experts', whose product's sigmoid goes to gate[t]; the lanes multiply that one
+// themselves.
+constexpr int kRouterWaves = 16;
+constexpr int kRouterTokens = 16;
+constexpr int kRouterRows = 32;
+constexpr int kRouterPad = kRouterTokens + 1;
+
+// Eight values of a row from k on.  VEC: rows of a multiple of 8 values, 16-byte aligned, so a piece is in
+// or out as a whole; a piece that is out reads the row's last one (no branch around a load) and the
+// caller drops it.  Otherwise element by element, zeros beyond H.
+template <int VEC, typename T>
+__device__ __forceinline__ void router_load(const T* row, int k, int H, float* v) {
+  if constexpr (VEC) {
+    const T* p = row + (k < H ? k : H - 8);
+    if constexpr (sizeof(T) == 2) {
+      const uint4 a = *reinterpret_cast<const uint4*>(p);
+      const uint32_t w[4] = {a.x, a.y, a.z, a.w};
 #pragma unroll
-    for (int j = 0; j < TOK; ++j)
-#pragma unroll
-      for (int e = 0; e < EB; ++e) acc[j][e] = 0.f;
-    for (int k = 4 * lane + 4 * kWave * wave; k < H; k += 16 * kWave) {
-      float xv[TOK][4];
-#pragma unroll
-      for (int j = 0; j < TOK; ++j) {
-        const T* xr = x + static_cast<int64_t>(t0 + j < T_ ? t0 + j : t0) * x_stride + k;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) xv[j][i] = (k + i < H) ? to_float(xr[i]) : 0.f;
+      for (int i = 0; i < 4; ++i) {
+        v[2 * i] = __uint_as_float(w[i] << 16);
+        v[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
       }
-      // every expert's piece is asked for before any is used, with no branch between the loads
-      // (an expert beyond the last reads the last one's row again; its sums are dropped)
-      float wv[EB][4];
-#pragma unroll
-      for (int e = 0; e < EB; ++e) {
-        const float* wp = wr + static_cast<int64_t>(e < ne ? e0 + e : rows - 1) * H + k;
-        if (vectors) {
-          const float4 v4 = *reinterpret_cast<const float4*>(wp);
-          wv[e][0] = v4.x; wv[e][1] = v4.y; wv[e][2] = v4.z; wv[e][3] = v4.w;
-        } else {
-#pragma unroll
-          for (int i = 0; i < 4; ++i) wv[e][i] = (k + i < H) ? wp[i] : 0.f;
-        }
-      }
-#pragma unroll
-      for (int e = 0; e < EB; ++e)
-#pragma unroll
-        for (int j = 0; j < TOK; ++j)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) acc[j][e] = fmaf(xv[j][i], wv[e][i], acc[j][e]);
+    } else {
+      const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+      v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+      v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
     }
+  } else {
 #pragma unroll
-    for (int j = 0; j < TOK; ++j) {
-      __syncthreads();  // the partial sums of the token before have been added up
-#pragma unroll
-      for (int e = 0; e < EB; ++e) part[threadIdx.x * PR + e] = acc[j][e];
-      __syncthreads();
-      if (threadIdx.x < ne) {
-        float sum = 0.f;
-        for (int l = 0; l < 256; ++l) sum += part[l * PR + threadIdx.x];
-        z[j * zrow + e0 + threadIdx.x] = sum;
-      }
-    }
-  }
-  __syncthreads();
-  if (wave != 0) return;
-  for (int j = 0; j < TOK; ++j) {
-    const int t = t0 + j;
-    if (t >= T_) break;  // the whole wave
-    float* zr = z + j * zrow;
-    if (gate != nullptr && lane == 0) gate[t] = 1.f / (1.f + expf(-zr[E]));
-    route_one(choice + static_cast<int64_t>(t) * rule.top, weight + static_cast<int64_t>(t) * rule.top, zr, zr,
-              zr + rows, zr + rows + E, lane, E, rule);
+    for (int i = 0; i < 8; ++i) v[i] = (k + i < H) ? to_float(row[k + i]) : 0.f;
   }
 }
 
-// One block.  counts -> offsets -> sorted pairs -> tiles.
+template <typename T, int VEC>
+__global__ __launch_bounds__(kRouterWaves * 64) void moe_router_kernel(
+    int32_t* __restrict__ choice, float* __restrict__ weight, const T* __restrict__ x, int64_t x_stride,
+    const float* __restrict__ wr, float* __restrict__ gate, int T_, int H, int E, RouteRule rule) {
+  constexpr int NT = kRouterRows / 16;
+  extern __shared__ float lds[];
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave), lane = threadIdx.x & (kWave - 1);
+  const int li = lane & 15, lk = lane >> 4;
+  float* part = lds;                                         // [waves][kRouterRows][kRouterPad]
+  float* part_g = lds + kRouterWaves * kRouterRows * kRouterPad;  // [waves][kRouterTokens]
+  float* z = part_g + kRouterWaves * kRouterTokens;          // [kRouterTokens][2 E + groups]
+  const int zrow = 2 * E + rule.groups;
+  const int t0 = blockIdx.x * kRouterTokens;
+  const T* xr = x + static_cast<int64_t>(t0 + li < T_ ? t0 + li : T_ - 1) * x_stride;  // rows beyond are dropped
+  float acc_g = 0.f;
+  for (int e0 = 0; e0 < E; e0 += kRouterRows) {
+    const int ne = (E - e0 < kRouterRows) ? E - e0 : kRouterRows;
+    const bool with_gate = gate != nullptr && e0 == 0;
+    const float* wp[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) wp[n] = wr + static_cast<int64_t>(e0 + (16 * n + li < ne ? 16 * n + li : 0)) * H;
+    const float* wg = wr + static_cast<int64_t>(with_gate ? E : e0) * H;
+    f32x4_t acc[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) acc[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    float xn[8], wn[NT][8], gn[8];
+    auto fetch = [&](int k) {
+      router_load<VEC>(xr, k + 8 * lk, H, xn);
+#pragma unroll
+      for (int n = 0; n < NT; ++n) router_load<VEC>(wp[n], k + 8 * lk, H, wn[n]);
+      router_load<VEC>(wg, k + 8 * lk, H, gn);
+    };
+    int k = 32 * wave;
+    if (k < H) fetch(k);
+    for (; k < H; k += 32 * kRouterWaves) {  // the same for the whole wave
+      float xc[8], wc[NT][8];
+      const bool in = !VEC || k + 8 * lk < H;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        xc[i] = in ? xn[i] : 0.f;
+#pragma unroll
+        for (int n = 0; n < NT; ++n) wc[n][i] = wn[n][i];
+        if (with_gate) acc_g = fmaf(xc[i], gn[i], acc_g);
+      }
+      if (k + 32 * kRouterWaves < H) fetch(k + 32 * kRouterWaves);
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+#pragma unroll
+        for (int n = 0; n < NT; ++n) acc[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(wc[n][i], xc[i], acc[n], 0, 0, 0);
+    }
+    if (e0 > 0) __syncthreads();  // the partial sums of the experts before have been added up
+    // lane holds token li, experts 16 n + 4 lk + i
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) part[(wave * kRouterRows + 16 * n + 4 * lk + i) * kRouterPad + li] = acc[n][i];
+    if (with_gate) {
+      acc_g += __shfl_xor(acc_g, 16, kWave);
+      acc_g += __shfl_xor(acc_g, 32, kWave);
+      if (lk == 0) part_g[wave * kRouterTokens + li] = acc_g;
+    }
+    __syncthreads();
+    for (int idx = threadIdx.x; idx < ne * kRouterTokens; idx += kRouterWaves * kWave) {
+      const int e = idx / kRouterTokens, j = idx - e * kRouterTokens;
+      float sum = 0.f;
+#pragma unroll
+      for (int w = 0; w < kRouterWaves; ++w) sum += part[(w * kRouterRows + e) * kRouterPad + j];
+      z[j * zrow + e0 + e] = sum;
+    }
+  }
+  __syncthreads();
+  const int t = t0 + wave;
+  if (t >= T_) return;  // the whole wave
+  if (gate != nullptr && lane == 0) {
+    float sum = 0.f;
+    for (int w = 0; w < kRouterWaves; ++w) sum += part_g[w * kRouterTokens + wave];
+    gate[t] = 1.f / (1.f + expf(-sum));
+  }
+  float* zr = z + wave * zrow;
+  route_one(choice + static_cast<int64_t>(t) * rule.top, weight + static_cast<int64_t>(t) * rule.top, zr, zr, zr + E,
+            zr + 2 * E, lane, E, rule);
+}
+
+// One block.  counts -> offsets and tiles (a thread an expert, which adds up the counts before its own)
+// -> sorted pairs.
 __global__ __launch_bounds__(1024) void moe_align_kernel(int32_t* __restrict__ sorted, int32_t* __restrict__ tiles,
                                                          int32_t* __restrict__ num_tiles,
                                                          const int32_t* __restrict__ choice, int pairs, int E,
                                                          int max_tiles, int tile_rows) {
   extern __shared__ int32_t ilds[];
   int32_t* count = ilds;           // [E]
-  int32_t* offset = count + E;     // [E + 1]
-  int32_t* cursor = offset + E + 1;  // [E]
+  int32_t* offset = count + E;     // [E]
+  int32_t* cursor = offset + E;    // [E]
   for (int e = threadIdx.x; e < E; e += blockDim.x) count[e] = 0;
   __syncthreads();
   for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
@@ -280,20 +323,20 @@ __global__ __launch_bounds__(1024) void moe_align_kernel(int32_t* __restrict__ s
     if (e >= 0 && e < E) atomicAdd(&count[e], 1);
   }
   __syncthreads();
-  if (threadIdx.x == 0) {
+  for (int e = threadIdx.x; e < E; e += blockDim.x) {
     int at = 0, nt = 0;
-    for (int e = 0; e < E; ++e) {
-      offset[e] = at;
-      cursor[e] = 0;
-      for (int r = 0; r < count[e] && nt < max_tiles; r += tile_rows, ++nt) {
-        tiles[3 * nt] = e;
-        tiles[3 * nt + 1] = at + r;
-        tiles[3 * nt + 2] = (count[e] - r < tile_rows) ? count[e] - r : tile_rows;
-      }
-      at += count[e];
+    for (int p = 0; p < e; ++p) {
+      at += count[p];
+      nt += (count[p] + tile_rows - 1) / tile_rows;
     }
-    offset[E] = at;
-    *num_tiles = nt;
+    offset[e] = at;
+    cursor[e] = 0;
+    for (int r = 0; r < count[e] && nt < max_tiles; r += tile_rows, ++nt) {
+      tiles[3 * nt] = e;
+      tiles[3 * nt + 1] = at + r;
+      tiles[3 * nt + 2] = (count[e] - r < tile_rows) ? count[e] - r : tile_rows;
+    }
+    if (e == E - 1) *num_tiles = nt;
   }
   __syncthreads();
   // an expert's pairs take their places in the order in which their threads arrive: a row's sums
@@ -612,28 +655,27 @@ extern "C" int kvc_moe_router(int32_t* choice, float* weight, const void* x, int
     return kvc_fail("kvc_moe_router: scores by softmax (0), sigmoid (1) or logit (2); a group is worth its best 1 or 2");
   const RouteRule rule{top, groups, keep, score_fn, group_best, bias, correction, weight_scale};
   if (T == 0) return 0;
-  // four tokens a block where the blocks then still fill the chip several times over, else one
-  const bool big = T >= 4 * 8 * kvc_device_compute_units();
-  const int TOK = big ? 4 : 1;
-  const size_t lds = sizeof(float) * (static_cast<size_t>(256) * 33 + static_cast<size_t>(TOK) * (2 * E + 1 + groups));
+  const size_t lds = sizeof(float) * (static_cast<size_t>(kRouterWaves) * (kRouterRows * kRouterPad + kRouterTokens) +
+                                      static_cast<size_t>(kRouterTokens) * (2 * E + groups));
   if (lds > 160 * 1024) return kvc_fail("kvc_moe_router: too many experts for a block's LDS");
-  const dim3 grid((T + TOK - 1) / TOK);
-  // 16-byte loads of the router's rows where the rows allow
-  const int vectors = H % 4 == 0 && (reinterpret_cast<uintptr_t>(router) & 15) == 0;
-#define KVC_ROUTER(Tp, TOK_)                                                                                    \
+  const dim3 grid((T + kRouterTokens - 1) / kRouterTokens);
+  // 16-byte loads where the rows allow
+  const bool vectors = H % 8 == 0 && x_stride % 8 == 0 && (reinterpret_cast<uintptr_t>(router) & 15) == 0 &&
+                       (reinterpret_cast<uintptr_t>(x) & 15) == 0;
+#define KVC_ROUTER(Tp, VEC)                                                                                     \
   do {                                                                                                          \
     if (lds > 64 * 1024) {                                                                                      \
-      const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&moe_router_kernel<Tp, TOK_>),  \
+      const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(&moe_router_kernel<Tp, VEC>),   \
                                                   hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)); \
       if (attr != hipSuccess) return kvc_fail("kvc_moe_router: the kernel's LDS size was refused");            \
     }                                                                                                           \
-    hipLaunchKernelGGL((moe_router_kernel<Tp, TOK_>), grid, dim3(256), lds, S(stream), choice, weight,          \
-                       static_cast<const Tp*>(x), x_stride, router, gate, T, H, E, rule, vectors);             \
+    hipLaunchKernelGGL((moe_router_kernel<Tp, VEC>), grid, dim3(kRouterWaves * kWave), lds, S(stream), choice,  \
+                       weight, static_cast<const Tp*>(x), x_stride, router, gate, T, H, E, rule);               \
   } while (0)
-  if (x_dtype == 1 && big) KVC_ROUTER(bf16_t, 4);
-  else if (x_dtype == 1) KVC_ROUTER(bf16_t, 1);
-  else if (x_dtype == 0 && big) KVC_ROUTER(float, 4);
-  else if (x_dtype == 0) KVC_ROUTER(float, 1);
+  if (x_dtype == 1 && vectors) KVC_ROUTER(bf16_t, 1);
+  else if (x_dtype == 1) KVC_ROUTER(bf16_t, 0);
+  else if (x_dtype == 0 && vectors) KVC_ROUTER(float, 1);
+  else if (x_dtype == 0) KVC_ROUTER(float, 0);
   else return kvc_fail("kvc_moe_router: unknown dtype code");
 #undef KVC_ROUTER
   return kvc_check_launch("kvc_moe_router");
@@ -652,7 +694,7 @@ extern "C" int kvc_moe_align(int32_t* sorted, int32_t* tiles, int32_t* num_tiles
   if (tile_rows != kTileRows && tile_rows != kBigTileRows) return kvc_fail("kvc_moe_align: tiles of 16 or 64 rows");
   if (pairs < 0 || E <= 0 || max_tiles < kvc_moe_max_tiles(pairs, E, tile_rows))
     return kvc_fail("kvc_moe_align: bad sizes, or room for fewer tiles than the routing may need");
-  const size_t lds = sizeof(int32_t) * (3 * E + 1);
+  const size_t lds = sizeof(int32_t) * 3 * E;
   if (lds > 60000) return kvc_fail("kvc_moe_align: too many experts");
   hipLaunchKernelGGL(moe_align_kernel, dim3(1), dim3(1024), lds, S(stream), sorted, tiles, num_tiles, choice,
                      pairs, E, max_tiles, tile_rows);
