@@ -116,8 +116,8 @@ def random_config(rng) -> dict:
             f = moe(rng.choice([16, 24, 32, 64, 40]), experts, rng.randint(1, min(experts, 5)),
                     rng.choice([None, 16, 32, 64, 40]))
         layers.append(layer(m, f))
-    bigram = None if rng.random() < 0.15 else (rng.choice([1, 37, 128, 1000]), rng.choice([1, 31, 100003, 0]),
-                                               rng.choice([1, 17, 65537]))
+    bigram = None if rng.random() < 0.15 else (rng.choice([1, 37, 128, 1000]), rng.choice([1, 43, 100003, 0]),
+                                               rng.choice([1, 19, 65537]))
     return model(rng.choice([97, 256, 512, 1000]), width, rng.choice([1e-6, 1e-5]), bigram, layers)
 
 
