@@ -3,7 +3,7 @@
 ``build()`` always compiles; ``ensure_built()`` compiles only when no library that
 matches the sources is there.  The library is written next to this file when that
 folder is writable, else under the temporary folder, so that a read-only checkout
-still works.  Progress lines go to stderr while the compiler runs.
+still works.  A line goes to stderr as each source is compiled.
 """
 
 from __future__ import annotations
@@ -14,8 +14,6 @@ import shutil
 import subprocess
 import sys
 import tempfile
-import threading
-import time
 from concurrent.futures import ThreadPoolExecutor
 from pathlib import Path
 
@@ -105,15 +103,6 @@ def build(verbose: bool = True) -> Path:
             print(f"[kvcore_amd build] {msg}", file=sys.stderr, flush=True)
 
     log(f"compiling {len(sources)} sources for {ARCH} with {hipcc}")
-    done = threading.Event()
-
-    def heartbeat() -> None:
-        start = time.time()
-        while not done.wait(15.0):
-            log(f"still compiling ({time.time() - start:.0f} s)")
-
-    beat = threading.Thread(target=heartbeat, daemon=True)
-    beat.start()
 
     def compile_one(src: Path) -> Path:
         obj = obj_dir / (src.stem + ".o")
@@ -124,19 +113,16 @@ def build(verbose: bool = True) -> Path:
         log(f"compiled {src.name}")
         return obj
 
-    try:
-        with ThreadPoolExecutor(max_workers=min(8, len(sources))) as pool:
-            objects = list(pool.map(compile_one, sources))
-        lib = out_dir / LIB_NAME
-        tmp_lib = out_dir / (LIB_NAME + f".tmp{os.getpid()}")
-        cmd = [hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objects), "-o", str(tmp_lib)]
-        proc = subprocess.run(cmd, capture_output=True, text=True)
-        if proc.returncode != 0:
-            raise RuntimeError(f"hipcc link failed:\n{proc.stderr[-4000:]}")
-        os.replace(tmp_lib, lib)
-        (out_dir / (LIB_NAME + ".srchash")).write_text(source_hash() + "\n")
-    finally:
-        done.set()
+    with ThreadPoolExecutor(max_workers=min(8, len(sources))) as pool:
+        objects = list(pool.map(compile_one, sources))
+    lib = out_dir / LIB_NAME
+    tmp_lib = out_dir / (LIB_NAME + f".tmp{os.getpid()}")
+    cmd = [hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", *map(str, objects), "-o", str(tmp_lib)]
+    proc = subprocess.run(cmd, capture_output=True, text=True)
+    if proc.returncode != 0:
+        raise RuntimeError(f"hipcc link failed:\n{proc.stderr[-4000:]}")
+    os.replace(tmp_lib, lib)
+    (out_dir / (LIB_NAME + ".srchash")).write_text(source_hash() + "\n")
     log(f"built {lib}")
     return lib
 
