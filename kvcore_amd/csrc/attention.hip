@@ -11,7 +11,9 @@
 // only: not on the batch it is in nor on how its request was cut into steps.  Two options:
 // `slopes` (a value per query head) takes slope * (position - key position) off every score, and
 // `chunk` lets a token see only the keys of its own chunk of that many positions; `sinks` (a value
-// per query head) adds exp(sink) to the softmax's denominator and nothing to the weighted sum.
+// per query head) adds exp(sink) to the softmax's denominator and nothing to the weighted sum; `softcap`
+// replaces a scaled score s by softcap * tanh(s / softcap); `gate` (rows as wide as the result) multiplies
+// the result by its sigmoid, element by element.
 
 #include <hip/hip_runtime.h>
 
@@ -51,7 +53,7 @@ __global__ __launch_bounds__(kWavesPerBlock* kWave) void paged_attention_wave_ke
     const int32_t* __restrict__ positions, const int32_t* __restrict__ token_req,
     const int32_t* __restrict__ slots, int nh, int nkv, int d, int dv, int page_size, int num_pages,
     float scale, int window, const float* __restrict__ slopes, int chunk, const float* __restrict__ sinks,
-    int out_f32) {
+    float softcap, const T* __restrict__ gate, int64_t gate_stride, int out_f32) {
   __shared__ float q_s[kWavesPerBlock][MAXD];
   __shared__ float p_s[kWavesPerBlock][kWave];
   __shared__ int64_t off_s[kWavesPerBlock][kWave];   // K row of each key of the tile
@@ -128,6 +130,7 @@ __global__ __launch_bounds__(kWavesPerBlock* kWave) void paged_attention_wave_ke
           for (int i = 0; i < d; ++i) dot = fmaf(q_s[wave][i], to_float(kr[i]), dot);
         }
         s = dot * scale - slope * static_cast<float>(pos - key);
+        if (softcap > 0.f) s = softcap * tanhf(s / softcap);  // the same for the whole grid
       }
     }
     const float tile_max = wave_max(s);
@@ -164,8 +167,10 @@ __global__ __launch_bounds__(kWavesPerBlock* kWave) void paged_attention_wave_ke
   for (int i = 0; i < MAXD / kWave; ++i) {
     const int e = lane + i * kWave;
     if (e < dv) {
-      if (out_f32) o32[e] = acc[i] * inv;
-      else o[e] = from_float<T>(acc[i] * inv);
+      float y = acc[i] * inv;
+      if (gate != nullptr) y *= sigmoid_of(to_float(gate[t * gate_stride + static_cast<int64_t>(h) * dv + e]));
+      if (out_f32) o32[e] = y;
+      else o[e] = from_float<T>(y);
     }
   }
 }
@@ -177,7 +182,8 @@ extern "C" int kvc_paged_attention(void* out, const void* q, int64_t q_stride, c
                                    const int32_t* positions, const int32_t* token_req,
                                    const int32_t* slots, int T, int nh, int nkv, int d, int dv,
                                    int page_size, int num_pages, float scale, int window,
-                                   const float* slopes, int chunk, const float* sinks, int out_f32, int dtype,
+                                   const float* slopes, int chunk, const float* sinks, float softcap,
+                                   const void* gate, int64_t gate_stride, int out_f32, int dtype,
                                    kvc_stream stream) {
   if (T < 0 || nh <= 0 || nkv <= 0 || page_size <= 0 || num_pages <= 0 || table_stride <= 0)
     return kvc_fail("kvc_paged_attention: bad sizes");
@@ -188,6 +194,10 @@ extern "C" int kvc_paged_attention(void* out, const void* q, int64_t q_stride, c
     return kvc_fail("kvc_paged_attention: value size must be positive, at most 512");
   if (q_stride < static_cast<int64_t>(nh) * d)
     return kvc_fail("kvc_paged_attention: q stride too small");
+  if (softcap < 0.f || (softcap > 0.f && slopes != nullptr))
+    return kvc_fail("kvc_paged_attention: a soft cap is positive and does not go with distance slopes");
+  if (gate != nullptr && gate_stride < static_cast<int64_t>(nh) * dv)
+    return kvc_fail("kvc_paged_attention: gate rows too short");
   if (T == 0) return 0;
   const dim3 grid(T, (nh + kWavesPerBlock - 1) / kWavesPerBlock);
   if (d > kUsualHeadDim || dv > kUsualHeadDim) {
@@ -198,7 +208,7 @@ extern "C" int kvc_paged_attention(void* out, const void* q, int64_t q_stride, c
                            static_cast<const Tp*>(q), q_stride, static_cast<const Tp*>(k_cache),
                            static_cast<const Tp*>(v_cache), table, table_stride, positions,
                            token_req, slots, nh, nkv, d, dv, page_size, num_pages, scale, window, slopes,
-                           chunk, sinks, out_f32));
+                           chunk, sinks, softcap, static_cast<const Tp*>(gate), gate_stride, out_f32));
     return kvc_check_launch("kvc_paged_attention");
   }
   KVC_DISPATCH_DTYPE(
@@ -208,7 +218,7 @@ extern "C" int kvc_paged_attention(void* out, const void* q, int64_t q_stride, c
                          static_cast<const Tp*>(q), q_stride, static_cast<const Tp*>(k_cache),
                          static_cast<const Tp*>(v_cache), table, table_stride, positions,
                          token_req, slots, nh, nkv, d, dv, page_size, num_pages, scale, window, slopes,
-                         chunk, sinks, out_f32));
+                         chunk, sinks, softcap, static_cast<const Tp*>(gate), gate_stride, out_f32));
   return kvc_check_launch("kvc_paged_attention");
 }
 
@@ -218,7 +228,8 @@ extern "C" int kvc_paged_attention(void* out, const void* q, int64_t q_stride, c
 // multiplied by a gain shared by all heads; then its first rot_dim elements are rotated
 // (pairs (2j, 2j+1) when interleaved, (j, j + rot_dim/2) otherwise); all in float32, rounded
 // once on the way out.  q heads go back in place, k heads in place and to K[page, kv head,
-// offset, :]; the value heads of dv elements are copied to V[page, kv head, :, offset].
+// offset, :]; the value heads of dv elements, which stand at column v_begin of a row, are copied to
+// V[page, kv head, :, offset].  With keep_keys the k heads' columns stay as they are (they are the values).
 namespace {
 
 constexpr int kMaxValuePlanes = 4;
@@ -233,7 +244,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_kv_write_kernel(
     const float* __restrict__ q_gain, const float* __restrict__ k_gain, float eps,
     const float* __restrict__ cos_tab, const float* __restrict__ sin_tab, int rot_dim,
     int interleaved, const int32_t* __restrict__ kv_slot, int nh, int nkv, int d, int dv,
-    int page_size, int write_kv, int copy_values) {
+    int page_size, int write_kv, int copy_values, int v_begin, int keep_keys) {
   __shared__ float head_s[4][MAXD];
   const int t = blockIdx.x;
   const int slot = kv_slot[t];
@@ -296,7 +307,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_kv_write_kernel(
         y = (e == e0) ? rotate_first(x0, x1, cs[j], sn[j]) : rotate_second(x0, x1, cs[j], sn[j]);
       }
       const T r = from_float<T>(y);
-      hp[e] = r;
+      if (!keep_keys || head < nh) hp[e] = r;
       if (kc != nullptr) kc[e] = r;
     }
     __syncthreads();
@@ -304,7 +315,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_kv_write_kernel(
   if (!store_kv || !copy_values) return;
   // element i of a value head goes to plane i / v_chunk, V[page, kv head, i % v_chunk, offset];
   // the token's blocks share the copy
-  const T* vrow = row + static_cast<int64_t>(nh + nkv) * d;
+  const T* vrow = row + v_begin;
   const int64_t v_base = static_cast<int64_t>(page) * nkv * page_size * v_chunk + off;
   for (int w = blockIdx.y * blockDim.x + threadIdx.x; w < nkv * dv; w += blockDim.x * gridDim.y) {
     const int head = w / dv, i = w - head * dv;
@@ -323,7 +334,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_k_write_small_kernel(
     const float* __restrict__ q_gain, const float* __restrict__ k_gain, float eps,
     const float* __restrict__ cos_tab, const float* __restrict__ sin_tab, int rot_dim,
     int interleaved, const int32_t* __restrict__ kv_slot, int num_tokens, int nh, int nkv, int d,
-    int page_size, int write_kv) {
+    int page_size, int write_kv, int keep_keys) {
   const int lane = threadIdx.x & (kWave - 1);
   const int64_t item = static_cast<int64_t>(blockIdx.x) * 4 + threadIdx.x / kWave;
   const int heads = nh + nkv;
@@ -358,7 +369,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_k_write_small_kernel(
   }
   if (!in) return;
   const T r = from_float<T>(y);
-  hp[lane] = r;
+  if (!keep_keys || head < nh) hp[lane] = r;
   if (head >= nh && write_kv && slot >= 0) {
     const int page = slot / page_size, off = slot - page * page_size;
     k_cache[((static_cast<int64_t>(page) * nkv + (head - nh)) * page_size + off) * d + lane] = r;
@@ -373,7 +384,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_k_write_vec_kernel(
     bf16_t* __restrict__ qkv, int64_t row_stride, bf16_t* __restrict__ k_cache, const float* __restrict__ q_gain,
     const float* __restrict__ k_gain, float eps, const float* __restrict__ cos_tab, const float* __restrict__ sin_tab,
     int rot_dim, int interleaved, const int32_t* __restrict__ kv_slot, int num_tokens, int nh, int nkv, int page_size,
-    int write_kv) {
+    int write_kv, int keep_keys) {
   constexpr int L = D / 8;
   const int sub = threadIdx.x % L;
   const int heads = nh + nkv;
@@ -448,7 +459,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_k_write_vec_kernel(
     r.x = f32_to_bf16_bits(y[c][0]) | (static_cast<uint32_t>(f32_to_bf16_bits(y[c][1])) << 16);
     r.y = f32_to_bf16_bits(y[c][2]) | (static_cast<uint32_t>(f32_to_bf16_bits(y[c][3])) << 16);
     const int p = c ? p1 : p0;
-    *reinterpret_cast<uint2*>(hp + p) = r;
+    if (!keep_keys || head < nh) *reinterpret_cast<uint2*>(hp + p) = r;
     if (kc != nullptr) *reinterpret_cast<uint2*>(kc + p) = r;
   }
 }
@@ -504,14 +515,17 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
                                          const float* cos_tab, const float* sin_tab, int rot_dim,
                                          int interleaved, const int32_t* kv_slot, int T, int nh,
                                          int nkv, int d, int dv, int page_size, int write_kv,
-                                         int dtype, kvc_stream stream) {
+                                         int values_are_keys, int dtype, kvc_stream stream) {
   if (T < 0 || nh <= 0 || nkv < 0 || d <= 0 || dv <= 0 || page_size <= 0)
     return kvc_fail("kvc_qk_norm_rope_kv_write: bad sizes");
   if (nkv == 0 && write_kv) return kvc_fail("kvc_qk_norm_rope_kv_write: rows without keys have nothing to write");
   if (d > kMaxHeadDim) return kvc_fail("kvc_qk_norm_rope_kv_write: head size above 512");
   if (rot_dim < 0 || rot_dim > d || (rot_dim & 1))
     return kvc_fail("kvc_qk_norm_rope_kv_write: rot_dim must be even and at most the head size");
-  if (row_stride < static_cast<int64_t>(nh + nkv) * d + static_cast<int64_t>(nkv) * dv)
+  if (values_are_keys && (dv != d || nkv == 0))
+    return kvc_fail("kvc_qk_norm_rope_kv_write: values that are the keys have the keys' size");
+  const int v_begin = values_are_keys ? nh * d : (nh + nkv) * d;
+  if (row_stride < static_cast<int64_t>(v_begin) + static_cast<int64_t>(nkv) * dv)
     return kvc_fail("kvc_qk_norm_rope_kv_write: rows too short for the heads");
   if ((q_gain == nullptr) != (k_gain == nullptr))
     return kvc_fail("kvc_qk_norm_rope_kv_write: gains for both q and k, or for neither");
@@ -539,7 +553,7 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
 #define KVC_QK_VEC(D_)                                                                                              \
   hipLaunchKernelGGL(qk_norm_rope_k_write_vec_kernel<D_>, grid, dim3(256), 0, s, static_cast<bf16_t*>(qkv), row_stride, \
                      static_cast<bf16_t*>(k_cache), q_gain, k_gain, eps, cos_tab, sin_tab, rot_dim, interleaved,    \
-                     kv_slot, T, nh, nkv, page_size, write_kv)
+                     kv_slot, T, nh, nkv, page_size, write_kv, values_are_keys)
     if (d == 32) KVC_QK_VEC(32);
     else if (d == 64) KVC_QK_VEC(64);
     else if (d == 128) KVC_QK_VEC(128);
@@ -549,7 +563,7 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
       ValuePlanes<bf16_t> planes{};
       for (int c = 0; c < num_v_planes; ++c) planes.plane[c] = static_cast<bf16_t*>(host_v_planes[c]);
       hipLaunchKernelGGL(value_planes_write_tile_kernel<bf16_t>, dim3((T + 7) / 8), dim3(256), 0, s,
-                         static_cast<const bf16_t*>(qkv), row_stride, planes, v_chunk, kv_slot, T, (nh + nkv) * d, nkv,
+                         static_cast<const bf16_t*>(qkv), row_stride, planes, v_chunk, kv_slot, T, v_begin, nkv,
                          dv, page_size);
     }
     return kvc_check_launch("kvc_qk_norm_rope_kv_write");
@@ -563,11 +577,11 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
         hipLaunchKernelGGL(qk_norm_rope_k_write_small_kernel<Tp>, dim3(static_cast<unsigned>((waves + 3) / 4)),
                            dim3(256), 0, reinterpret_cast<hipStream_t>(stream), static_cast<Tp*>(qkv),
                            row_stride, static_cast<Tp*>(k_cache), q_gain, k_gain, eps, cos_tab, sin_tab,
-                           rot_dim, interleaved, kv_slot, T, nh, nkv, d, page_size, write_kv);
+                           rot_dim, interleaved, kv_slot, T, nh, nkv, d, page_size, write_kv, values_are_keys);
         if (tiled_values) hipLaunchKernelGGL(
             value_planes_write_tile_kernel<Tp>, dim3((T + 7) / 8), dim3(256), 0,
             reinterpret_cast<hipStream_t>(stream), static_cast<const Tp*>(qkv), row_stride,
-            planes, v_chunk, kv_slot, T, (nh + nkv) * d, nkv, dv, page_size));
+            planes, v_chunk, kv_slot, T, v_begin, nkv, dv, page_size));
     return kvc_check_launch("kvc_qk_norm_rope_kv_write");
   }
   if (d > kUsualHeadDim) {
@@ -578,11 +592,11 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
                            reinterpret_cast<hipStream_t>(stream), static_cast<Tp*>(qkv), row_stride,
                            static_cast<Tp*>(k_cache), planes, v_chunk, q_gain, k_gain, eps,
                            cos_tab, sin_tab, rot_dim, interleaved, kv_slot, nh, nkv, d, dv, page_size,
-                           write_kv, tiled_values ? 0 : 1);
+                           write_kv, tiled_values ? 0 : 1, v_begin, values_are_keys);
         if (tiled_values) hipLaunchKernelGGL(
             value_planes_write_tile_kernel<Tp>, dim3((T + 7) / 8), dim3(256), 0,
             reinterpret_cast<hipStream_t>(stream), static_cast<const Tp*>(qkv), row_stride, planes,
-            v_chunk, kv_slot, T, (nh + nkv) * d, nkv, dv, page_size));
+            v_chunk, kv_slot, T, v_begin, nkv, dv, page_size));
     return kvc_check_launch("kvc_qk_norm_rope_kv_write");
   }
   KVC_DISPATCH_DTYPE(
@@ -592,10 +606,10 @@ extern "C" int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_
                          reinterpret_cast<hipStream_t>(stream), static_cast<Tp*>(qkv), row_stride,
                          static_cast<Tp*>(k_cache), planes, v_chunk, q_gain, k_gain, eps,
                          cos_tab, sin_tab, rot_dim, interleaved, kv_slot, nh, nkv, d, dv, page_size,
-                         write_kv, tiled_values ? 0 : 1);
+                         write_kv, tiled_values ? 0 : 1, v_begin, values_are_keys);
       if (tiled_values) hipLaunchKernelGGL(
           value_planes_write_tile_kernel<Tp>, dim3((T + 7) / 8), dim3(256), 0,
           reinterpret_cast<hipStream_t>(stream), static_cast<const Tp*>(qkv), row_stride, planes,
-          v_chunk, kv_slot, T, (nh + nkv) * d, nkv, dv, page_size));
+          v_chunk, kv_slot, T, v_begin, nkv, dv, page_size));
   return kvc_check_launch("kvc_qk_norm_rope_kv_write");
 }

@@ -1,7 +1,7 @@
 // Paged attention for single tokens (decode), bfloat16, on the matrix cores, with the
 // rotation of the token's query and key and the write of its key and value into the cache
 // done by the same kernel, where the layer has one behind a norm of every query and key head.
-// Value heads are as wide as the keys or half as wide.
+// Value heads are as wide as the keys or half as wide, or the key heads themselves as projected.
 //
 // One block of W waves per (token, kv head, split of the key range); the waves take the
 // 16-key blocks of the range in turn.  The query heads that share the kv head are the
@@ -53,7 +53,7 @@ struct DecodeArgs {
   int out_f32;  // out receives float32 values (the sums as they are) instead of bfloat16
   float* part_o;
   float* part_ml;
-  const bf16_t* qkv;  // rows [nh q heads of d | nkv k heads of d | nkv v heads of dv]
+  const bf16_t* qkv;  // rows [nh q heads of d | nkv k heads of d], nkv v heads of dv from v_begin on
   int64_t qkv_stride;
   bf16_t* k_cache;
   bf16_t* v_cache;
@@ -73,10 +73,13 @@ struct DecodeArgs {
   int write_kv;  // store the token's key and value (and attend to them from LDS)
   int nh, nkv, page_size, num_pages;
   float scale_log2e;
+  float cap_rate, cap_log2e;  // cap_rate > 0: a score is cap_log2e * capped_unit(raw score, cap_rate)
   int window;
   const float* slopes;  // [nh] or null: slope * (position - key position) comes off the score
   int chunk;            // > 0: only the keys of the token's own chunk of so many positions
   const float* sinks;   // [nh] or null: exp(sink) joins the softmax's denominator and brings no value along
+  GateRows gate;        // sigmoid of these rows multiplies the result, element by element
+  int v_begin;          // column of the first value head in a row of qkv
   int nsplit;
   int lds_pages;  // page ids of a block's range that fit in LDS
 };
@@ -283,7 +286,7 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
       }
     }
     if (owner) {
-      const bf16_t* vsrc = trow + static_cast<int64_t>(nh + nkv) * D + static_cast<int64_t>(hk) * DV;
+      const bf16_t* vsrc = trow + a.v_begin + static_cast<int64_t>(hk) * DV;
       for (int e = tid; e < DV; e += nthreads) {
         const bf16_t v = vsrc[e];
         sv[e] = v;
@@ -342,7 +345,9 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
     for (int i = 0; i < 4; ++i) {
       const int key = key0 + i;
       ok[i] = key >= first && key <= pos;
-      sv4[i] = ok[i] ? __builtin_fmaf(s[i], a.scale_log2e, -slope_l2e * static_cast<float>(pos - key)) : -INFINITY;
+      const float score = a.cap_rate > 0.f ? a.cap_log2e * capped_unit(s[i], a.cap_rate)  // scalar
+                                           : __builtin_fmaf(s[i], a.scale_log2e, -slope_l2e * static_cast<float>(pos - key));
+      sv4[i] = ok[i] ? score : -INFINITY;
       mx = fmaxf(mx, sv4[i]);
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -428,7 +433,10 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
     }
     const int64_t th = static_cast<int64_t>(t) * nh + hk * g + h;
     if (nsplit == 1) {
-      store_result(a.out, th * DV + e, denom > 0.f ? acc / denom : 0.f, a.out_f32);
+      const float gain = a.gate.gate != nullptr  // scalar
+                             ? sigmoid_of(to_float(a.gate.gate[t * a.gate.stride + static_cast<int64_t>(hk * g) * DV + idx]))
+                             : 1.f;
+      store_result(a.out, th * DV + e, denom > 0.f ? acc / denom * gain : 0.f, a.out_f32);
     } else {
       a.part_o[(th * nsplit + split) * DV + e] = acc;
       if (e == 0) {
@@ -444,7 +452,8 @@ __global__ __launch_bounds__(max_waves<D>() * 64) void decode_attention_kernel(c
 // another wave; the partial outputs are asked for before the weights are known.
 constexpr int kMaxSplits = kMaxAttentionSplits;
 __global__ void decode_combine_kernel(bf16_t* __restrict__ out, const float* __restrict__ part_o,
-                                      const float* __restrict__ part_ml, int D, int nsplit, int out_f32) {
+                                      const float* __restrict__ part_ml, int D, int nsplit, int out_f32,
+                                      GateRows gate) {
   const int64_t th = blockIdx.x;  // token * nh + head
   const int lane = threadIdx.x & 63;
   const float* ml = part_ml + th * nsplit * 2;
@@ -458,6 +467,11 @@ __global__ void decode_combine_kernel(bf16_t* __restrict__ out, const float* __r
     const int e = e0 + threadIdx.x;
     const bool live = e < D;
     float acc = 0.f;
+    float raw_gate = 0.f;
+    if (gate.gate != nullptr && live) {  // asked for before the sums are known
+      const int64_t t = th / gate.nh;
+      raw_gate = to_float(gate.gate[t * gate.stride + (th - t * gate.nh) * D + e]);
+    }
     float mmax = wave_max(m_s);
     const float m_safe = (mmax == -INFINITY) ? 0.f : mmax;
     const float w_lane = __builtin_amdgcn_exp2f(m_s - m_safe);  // 0 for lanes beyond nsplit
@@ -473,7 +487,8 @@ __global__ void decode_combine_kernel(bf16_t* __restrict__ out, const float* __r
         if (s0 + i < nsplit && w > 0.f) acc += w * v[i];
       }
     }
-    if (live) store_result(out, th * D + e, denom > 0.f ? acc / denom : 0.f, out_f32);
+    const float gain = gate.gate != nullptr ? sigmoid_of(raw_gate) : 1.f;
+    if (live) store_result(out, th * D + e, denom > 0.f ? acc / denom * gain : 0.f, out_f32);
   }
 }
 
@@ -500,19 +515,19 @@ int launch_decode(DecodeArgs& args, int T, hipStream_t stream) {
                      lds_total(waves, g, D, args.lds_pages), stream, args);
   if (args.nsplit > 1)
     hipLaunchKernelGGL(decode_combine_kernel, dim3(T * args.nh), dim3((DV + 63) / 64 * 64), 0, stream,
-                       args.out, args.part_o, args.part_ml, DV, args.nsplit, args.out_f32);
+                       args.out, args.part_o, args.part_ml, DV, args.nsplit, args.out_f32, args.gate);
   return kvc_check_launch("kvc_decode_attention");
 }
 
 }  // namespace
 
 int kvc::launch_attention_combine(bf16_t* out, const float* part_o, const float* part_ml, int64_t rows,
-                                  int d, int nsplit, int out_f32, hipStream_t stream) {
+                                  int d, int nsplit, int out_f32, const GateRows& gate, hipStream_t stream) {
   if (rows <= 0) return 0;
   if (rows > 0x7fffffff || nsplit < 1 || nsplit > kMaxAttentionSplits)
     return kvc_fail("attention combine: bad sizes");
   hipLaunchKernelGGL(decode_combine_kernel, dim3(static_cast<unsigned>(rows)), dim3((d + 63) / 64 * 64), 0,
-                     stream, out, part_o, part_ml, d, nsplit, out_f32);
+                     stream, out, part_o, part_ml, d, nsplit, out_f32, gate);
   return kvc_check_launch("attention combine");
 }
 
@@ -545,14 +560,20 @@ extern "C" int kvc_decode_attention(void* out, void* part_o, void* part_ml, cons
                                     const float* cos_tab, const float* sin_tab, int rot_dim, int interleaved,
                                     const float* q_gain, const float* k_gain, float norm_eps, int write_kv, int T, int nh,
                                     int nkv, int d, int dv, int page_size, int num_pages, float scale,
-                                    int window, const float* slopes, int chunk, const float* sinks,
+                                    int window, const float* slopes, int chunk, const float* sinks, float softcap,
+                                    const void* gate, int64_t gate_stride, int values_are_keys,
                                     int nsplit, int out_f32, kvc_stream stream) {
   if (!kvc_decode_attention_supported(nh, nkv, d, dv, page_size, 1))
     return kvc_fail("kvc_decode_attention: unsupported shape (bfloat16, head size a multiple of 32 "
                     "up to 256, values as wide or half as wide, at most 16 query heads per kv head, page size a multiple of 16)");
   if (T < 0 || nsplit < 1 || nsplit > kMaxSplits || nkv > 65535 || table_stride <= 0 || num_pages <= 0)
     return kvc_fail("kvc_decode_attention: bad sizes (at most 64 splits)");
-  if (qkv_stride % 8 || qkv_stride < static_cast<int64_t>(nh) * d + (write_kv ? static_cast<int64_t>(nkv) * (d + dv) : 0))
+  if (values_are_keys && dv != d) return kvc_fail("kvc_decode_attention: values that are the keys have the keys' size");
+  if (softcap < 0.f || (softcap > 0.f && slopes != nullptr))
+    return kvc_fail("kvc_decode_attention: a soft cap is positive and does not go with distance slopes");
+  if (gate != nullptr && gate_stride < static_cast<int64_t>(nh) * dv)
+    return kvc_fail("kvc_decode_attention: gate rows too short");
+  if (qkv_stride % 8 || qkv_stride < static_cast<int64_t>(nh) * d + (write_kv ? static_cast<int64_t>(nkv) * (values_are_keys ? d : d + dv) : 0))
     return kvc_fail("kvc_decode_attention: token rows must be 16-byte aligned and hold q (and k, v)");
   if (rot_dim < 0 || rot_dim > d || rot_dim % 2)
     return kvc_fail("kvc_decode_attention: the rotated width must be even and at most the head size");
@@ -591,6 +612,10 @@ extern "C" int kvc_decode_attention(void* out, void* part_o, void* part_ml, cons
   args.page_size = page_size;
   args.num_pages = num_pages;
   args.scale_log2e = scale * kLog2e;
+  args.cap_rate = softcap > 0.f ? 2.f * kLog2e * scale / softcap : 0.f;
+  args.cap_log2e = softcap * kLog2e;
+  args.gate = GateRows{static_cast<const bf16_t*>(gate), gate_stride, nh};
+  args.v_begin = values_are_keys ? nh * d : (nh + nkv) * d;
   args.window = window;
   args.slopes = slopes;
   args.chunk = chunk;

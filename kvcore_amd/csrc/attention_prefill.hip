@@ -71,6 +71,8 @@ __device__ __forceinline__ float quad_sum(float v) {
   return __uint_as_float(b[0]) + __uint_as_float(b[1]);
 }
 
+constexpr float kBoundedLog2 = 64.f;  // scores capped to so many powers of two need no running maximum
+
 // KB: 16-key blocks per LDS tile
 template <int D, int DV, int KB>
 constexpr int tile_bytes() {
@@ -90,7 +92,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
     const float* __restrict__ slopes, int chunk, const float* __restrict__ sinks, float* __restrict__ part_o,
     float* __restrict__ part_ml, int single,
     const float* __restrict__ cos_tab, const float* __restrict__ sin_tab, int rot_dim, int interleaved,
-    int out_f32) {
+    float cap_rate, const GateRows gate, int out_f32) {
   constexpr int kKeyBlocks = KB;
   constexpr int NJ = DV / 16;
   constexpr int NC = D / 32;
@@ -103,6 +105,10 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
 
   const int g = nh / nkv;
   const int bq = (16 * W * CT) / g;  // tokens per block
+  // cap_rate > 0: raw scores become capped_unit(raw, cap_rate), numbers between -1 and 1, and scale_log2e is
+  // the cap in the exponent's units.  The exponents are then bounded, so with a cap of up to 44 no maximum
+  // is looked for: the sums stay relative to a score of zero (weights of at most 2^64).
+  const bool bounded = cap_rate > 0.f && scale_log2e <= kBoundedLog2;
   // Workgroups go to the chip's eight dies in turn (workgroup id modulo 8) and every die has
   // an L2 of its own, while all blocks of a kv head read the same keys and values.  So a kv
   // head's blocks get ids that land on one die (with fewer than eight kv heads, on 8 / nkv
@@ -265,7 +271,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
   float m[CT], l[CT];
 #pragma unroll
   for (int ct = 0; ct < CT; ++ct) {
-    m[ct] = -INFINITY;
+    m[ct] = bounded ? 0.f : -INFINITY;
     l[ct] = 0.f;
 #pragma unroll
     for (int j = 0; j < NJ; ++j) o_acc[ct][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -510,6 +516,14 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
             s[ct][kbi][i] = __builtin_fmaf(-my_slope[ct], d0 - static_cast<float>(16 * kbi + i), s[ct][kbi][i]);
       }
     }
+    if (cap_rate > 0.f) {  // scalar
+#pragma unroll
+      for (int ct = 0; ct < CT; ++ct)
+#pragma unroll
+        for (int kbi = 0; kbi < kKeyBlocks; ++kbi)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) s[ct][kbi][i] = capped_unit(s[ct][kbi][i], cap_rate);
+    }
 #pragma unroll
     for (int ct = 0; ct < CT; ++ct) {
       if (!whole) {
@@ -523,6 +537,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
           }
         }
       }
+      if (bounded) continue;  // scalar
       float v = -INFINITY;
 #pragma unroll
       for (int kbi = 0; kbi < kKeyBlocks; ++kbi)
@@ -532,7 +547,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
       mx[ct] = v;
       moved = moved || (v > m[ct] + unit);  // also true for the first visible key (m = -inf)
     }
-    if (__any(moved)) {
+    if (!bounded && __any(moved)) {
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct) {
         if (mx[ct] > m[ct] + unit) {
@@ -640,6 +655,17 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
     }
     const float inv = (l_row > 0.f) ? 1.f / l_row : 0.f;
     const int64_t at = (static_cast<int64_t>(my_tok[ct]) * nh + my_head[ct]) * DV + 4 * quad;
+    if (gate.gate != nullptr) {  // scalar: times the sigmoid of the gate's rows, four values of a head at a time
+      const bf16_t* gp = gate.gate + my_tok[ct] * gate.stride + static_cast<int64_t>(my_head[ct]) * DV + 4 * quad;
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) {
+        const uint2 w = *reinterpret_cast<const uint2*>(gp + 16 * j);
+        o_acc[ct][j][0] *= sigmoid_of(__uint_as_float(w.x << 16));
+        o_acc[ct][j][1] *= sigmoid_of(__uint_as_float(w.x & 0xffff0000u));
+        o_acc[ct][j][2] *= sigmoid_of(__uint_as_float(w.y << 16));
+        o_acc[ct][j][3] *= sigmoid_of(__uint_as_float(w.y & 0xffff0000u));
+      }
+    }
     if (out_f32) {  // the sums as they are, for a consumer that joins them before anything is rounded
       float* op = reinterpret_cast<float*>(out) + at;
 #pragma unroll
@@ -664,7 +690,8 @@ int launch_prefill_ct(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16
                       int R, int nh, int nkv, int page_size, int num_pages, float scale, int window,
                       const float* slopes, int chunk, const float* sinks, float* part_o, float* part_ml, int nsplit, int single,
                       const float* cos_tab,
-                      const float* sin_tab, int rot_dim, int interleaved, int out_f32, hipStream_t stream) {
+                      const float* sin_tab, int rot_dim, int interleaved, float softcap, const GateRows& gate,
+                      int out_f32, hipStream_t stream) {
   const int g = nh / nkv;
   const int bq = (16 * W * CT) / g;
   // every request may end in a ragged tile and have an odd number of tiles
@@ -692,10 +719,11 @@ int launch_prefill_ct(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16
   kvc_note_variant(kVariantPrefillAttention, variant);
   hipLaunchKernelGGL((prefill_attention_kernel<D, DV, CT, KB, W>), dim3(static_cast<unsigned>(wide), 1, nsplit), dim3(W * 64),
                      lds_bytes, stream, out, q, q_stride, k_cache, v_cache, table, table_stride, positions,
-                     q_start, slots, R, nh, nkv, page_size, num_pages, scale * kLog2e, window, slopes, chunk,
-                     sinks, part_o, part_ml, single, cos_tab, sin_tab, rot_dim, interleaved, out_f32);
+                     q_start, slots, R, nh, nkv, page_size, num_pages, (softcap > 0.f ? softcap : scale) * kLog2e, window,
+                     slopes, chunk, sinks, part_o, part_ml, single, cos_tab, sin_tab, rot_dim, interleaved,
+                     softcap > 0.f ? 2.f * kLog2e * scale / softcap : 0.f, gate, out_f32);
   if (nsplit > 1)
-    return launch_attention_combine(out, part_o, part_ml, static_cast<int64_t>(T) * nh, DV, nsplit, out_f32, stream);
+    return launch_attention_combine(out, part_o, part_ml, static_cast<int64_t>(T) * nh, DV, nsplit, out_f32, gate, stream);
   return kvc_check_launch("kvc_prefill_attention");
 }
 
@@ -706,7 +734,7 @@ int launch_prefill(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t*
                    int R, int nh, int nkv, int page_size, int num_pages, float scale, int window,
                    const float* slopes, int chunk, const float* sinks, float* part_o, float* part_ml, int nsplit,
                    const float* cos_tab, const float* sin_tab,
-                   int rot_dim, int interleaved, int out_f32, hipStream_t stream) {
+                   int rot_dim, int interleaved, float softcap, const GateRows& gate, int out_f32, hipStream_t stream) {
   const int g = nh / nkv;
   // Blocks of four waves lie two to a compute unit, blocks of eight waves one.  Tiles of 64
   // query rows, two a block one after the other (a late and an early one), are the fastest as
@@ -766,7 +794,7 @@ int launch_prefill(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t*
   return launch_prefill_ct<D, DV, CT_, W_>(out, q, q_stride, k_cache, v_cache, table, table_stride, positions, \
                                        q_start, slots, T, R, nh, nkv, page_size, num_pages, scale, window, \
                                        slopes, chunk, sinks, part_o, part_ml, nsplit, single, cos_tab, sin_tab, rot_dim,     \
-                                       interleaved, out_f32, stream)
+                                       interleaved, softcap, gate, out_f32, stream)
   if constexpr (DV >= 64) {
     if (waves == 8) {
       if (ct == 2) KVC_LAUNCH_PREFILL(2, 8);
@@ -795,8 +823,8 @@ extern "C" int kvc_prefill_attention(void* out, const void* q, int64_t q_stride,
                                      const int32_t* slots, int T, int R, int nh, int nkv, int d, int dv,
                                      int page_size, int num_pages, float scale, int window,
                                      const float* slopes, int chunk, const float* sinks, void* part_o, void* part_ml, int nsplit, const float* cos_tab,
-                                     const float* sin_tab, int rot_dim, int interleaved, int out_f32,
-                                     kvc_stream stream) {
+                                     const float* sin_tab, int rot_dim, int interleaved, float softcap,
+                                     const void* gate_rows, int64_t gate_stride, int out_f32, kvc_stream stream) {
   if (!kvc_prefill_attention_supported(nh, nkv, d, dv, page_size, 1))
     return kvc_fail("kvc_prefill_attention: unsupported shape (bfloat16, head size 64 or 128, values as "
                     "wide or half as wide, at most 64 query heads per kv head, page size a multiple of 16)");
@@ -814,7 +842,13 @@ extern "C" int kvc_prefill_attention(void* out, const void* q, int64_t q_stride,
       (rot_dim <= 0 || rot_dim > d || rot_dim % (interleaved ? 32 : 64)))
     return kvc_fail("kvc_prefill_attention: rotating the queries here needs rot_dim to be a multiple "
                     "of 64 (32 for neighbouring pairs) and at most the head size");
+  if (softcap < 0.f || (softcap > 0.f && slopes != nullptr))
+    return kvc_fail("kvc_prefill_attention: a soft cap is positive and does not go with distance slopes");
+  if (gate_rows != nullptr && (gate_stride < static_cast<int64_t>(nh) * dv || gate_stride % 4 ||
+                               (reinterpret_cast<uintptr_t>(gate_rows) & 7) != 0))
+    return kvc_fail("kvc_prefill_attention: gate rows too short or not 8-byte aligned");
   if (T == 0) return 0;
+  const GateRows gate{static_cast<const bf16_t*>(gate_rows), gate_stride, nh};
   float* po = static_cast<float*>(part_o);
   float* pml = static_cast<float*>(part_ml);
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
@@ -824,7 +858,7 @@ extern "C" int kvc_prefill_attention(void* out, const void* q, int64_t q_stride,
 #define KVC_PREFILL(D_, DV_)                                                                                      \
   return launch_prefill<D_, DV_>(static_cast<bf16_t*>(out), qq, q_stride, kc, vc, table, table_stride, positions, \
                                  q_start, slots, T, R, nh, nkv, page_size, num_pages, scale, window, slopes, chunk, \
-                                 sinks, po, pml, nsplit, cos_tab, sin_tab, rot_dim, interleaved, out_f32, s)
+                                 sinks, po, pml, nsplit, cos_tab, sin_tab, rot_dim, interleaved, softcap, gate, out_f32, s)
   if (d == 64) {
     if (dv == d) KVC_PREFILL(64, 64);
     KVC_PREFILL(64, 32);

@@ -48,6 +48,16 @@ __device__ __forceinline__ float rotate_second(float x0, float x1, float c, floa
   return __builtin_fmaf(x0, s, x1 * c);
 }
 
+__device__ __forceinline__ float sigmoid_of(float x) { return 1.f / (1.f + expf(-x)); }
+__device__ __forceinline__ float silu_of(float x) { return x / (1.f + expf(-x)); }
+
+// A soft cap on attention scores inside the matrix-core kernels: cap * tanh(scale * raw / cap) in units of
+// cap, from the raw score and rate = 2 * log2(e) * scale / cap.  tanh(y) = 1 - 2 / (1 + e^(2y)) with the
+// hardware's exponential and reciprocal: an absolute error of some 1e-7 of the cap.
+__device__ __forceinline__ float capped_unit(float raw, float rate) {
+  return __builtin_fmaf(-2.f, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(raw * rate)), 1.f);
+}
+
 // min(g, limit) * sigmoid(alpha * min(g, limit)) * (clamp(u, -limit, limit) + shift)
 __device__ __forceinline__ float clamped_glu(float g, float u, float limit, float alpha, float shift) {
   g = fminf(g, limit);

@@ -646,7 +646,7 @@ extern "C" int kvc_to_float(float* out, const void* in, int64_t n, int dtype, kv
 // -------------------------------------------------------------------- rotary tables
 __global__ void rope_table_kernel(float* __restrict__ cos_out, float* __restrict__ sin_out,
                                   const int32_t* __restrict__ positions,
-                                  const float* __restrict__ inv_freq, int half, int64_t n) {
+                                  const float* __restrict__ inv_freq, float scale, int half, int64_t n) {
   const int64_t idx = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   if (idx >= n) return;
   const int64_t t = idx / half;
@@ -654,18 +654,18 @@ __global__ void rope_table_kernel(float* __restrict__ cos_out, float* __restrict
   const float angle = static_cast<float>(positions[t]) * inv_freq[j];
   float s, c;
   sincosf(angle, &s, &c);
-  cos_out[idx] = c;
-  sin_out[idx] = s;
+  cos_out[idx] = c * scale;
+  sin_out[idx] = s * scale;
 }
 
 extern "C" int kvc_rope_table(float* cos_out, float* sin_out, const int32_t* positions,
-                              const float* inv_freq, int T, int half, kvc_stream stream) {
+                              const float* inv_freq, float scale, int T, int half, kvc_stream stream) {
   if (T < 0 || half <= 0) return kvc_fail("kvc_rope_table: bad sizes");
   const int64_t n = static_cast<int64_t>(T) * half;
   if (n == 0) return 0;
   const unsigned blocks = static_cast<unsigned>((n + 255) / 256);
   hipLaunchKernelGGL(rope_table_kernel, dim3(blocks), dim3(256), 0, S(stream), cos_out, sin_out,
-                     positions, inv_freq, half, n);
+                     positions, inv_freq, scale, half, n);
   return kvc_check_launch("kvc_rope_table");
 }
 

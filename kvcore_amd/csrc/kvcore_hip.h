@@ -99,9 +99,9 @@ int kvc_gather_rows(void* out, const void* in, const int32_t* rows, int S, int H
 // out = float(in) elementwise (n values).
 int kvc_to_float(float* out, const void* in, int64_t n, int dtype, kvc_stream stream);
 
-// cos/sin[t, j] of the angle float(positions[t]) * inv_freq[j], j < half.
+// cos/sin[t, j] of the angle float(positions[t]) * inv_freq[j], j < half, times scale.
 int kvc_rope_table(float* cos_out, float* sin_out, const int32_t* positions,
-                   const float* inv_freq, int T, int half, kvc_stream stream);
+                   const float* inv_freq, float scale, int T, int half, kvc_stream stream);
 
 // kv_slot[t] = page * page_size + position % page_size, where page = table[slots[
 // token_req[t]], position / page_size]; -1 when the table holds no page there, -2 for a
@@ -130,6 +130,9 @@ int kvc_rope_kv_write(void* qkv, void* k_cache, void* v_cache, const float* cos_
 // h.  chunk > 0: a token sees only the keys j with j / chunk == p / chunk.  sinks (float32 [nh],
 // or null): exp(sinks[h]) is added to the softmax's denominator of head h: a logit of its own,
 // taken as it is (scale does not apply), that brings no value into the weighted sum.
+// softcap > 0 (not with slopes): a scaled score s becomes softcap * tanh(s / softcap).  gate (rows of
+// nh * dv values of dtype, gate_stride apart, or null): the result is multiplied, element by element, by
+// the gate's sigmoid.
 // out_f32: out is float32 whatever dtype says of the operands (the weighted sums as they are, for a
 // consumer that joins results before anything is rounded); the two kernels below take it too.
 int kvc_paged_attention(void* out, const void* q, int64_t q_stride, const void* k_cache,
@@ -137,7 +140,8 @@ int kvc_paged_attention(void* out, const void* q, int64_t q_stride, const void* 
                         const int32_t* positions, const int32_t* token_req,
                         const int32_t* slots, int T, int nh, int nkv, int d, int dv, int page_size,
                         int num_pages, float scale, int window, const float* slopes, int chunk,
-                        const float* sinks, int out_f32, int dtype, kvc_stream stream);
+                        const float* sinks, float softcap, const void* gate, int64_t gate_stride, int out_f32,
+                        int dtype, kvc_stream stream);
 
 // residual[t, :] = float(table[ids[t], :]) + float(pairs[row, :]): row = buckets for the token at position
 // 0, else (prev * mul_prev + ids[t] * mul_cur) mod buckets with prev the token before it, ids[t - 1] or,
@@ -160,11 +164,13 @@ int kvc_embed_pairs(float* residual, const void* table, const void* pairs, const
 // array of their device pointers): element i of a value head then lies in plane i / (dv /
 // num_v_planes), so that kernels whose keys and values are of one size can serve a plane each.
 // nkv 0 (without write_kv): the rows hold queries alone, for a layer that reads another's cache.
+// values_are_keys (dv = d): the rows end with the k heads, whose columns are left as they are and written
+// as the values, before norm and rotation.
 int kvc_qk_norm_rope_kv_write(void* qkv, int64_t row_stride, void* k_cache,
                               void* const* host_v_planes, int num_v_planes, const float* q_gain, const float* k_gain, float eps,
                               const float* cos_tab, const float* sin_tab, int rot_dim,
                               int interleaved, const int32_t* kv_slot, int T, int nh, int nkv, int d,
-                              int dv, int page_size, int write_kv, int dtype, kvc_stream stream);
+                              int dv, int page_size, int write_kv, int values_are_keys, int dtype, kvc_stream stream);
 
 // residual += delta (skipped when delta is null); out = (residual - mean) / sqrt(var + eps) *
 // weight + bias (bias may be null), var the mean of the squared deviations; rounded to dt.
@@ -236,17 +242,19 @@ int kvc_gated_group_rmsnorm(void* out, int out_dtype, const float* y, const void
 // Per head h (its q and k come from head h / (nh / nqk) of nqk heads of d), token by token:
 //   delta_rule 0:  S = diag(decay[t, h, :]) S + k v^T            (decay rows of nh * d values)
 //   delta_rule 1:  S = decay[t, h] S;  u = beta[t, h] (v - S^T k);  S = S + k u^T
-//   delta_rule 2:  S = decay[t, h] S + beta[t, h] k v^T          (scalar gates per head)
+//   delta_rule 2:  S = decay[t, h] S + beta[t, h] k v^T          (scalar gates per head; beta may be null,
+//                  ones, and decay_stride 0, one row for every token)
 // and out[t, h] = S^T (q_scale q) after the token's write; out is [T, nh * dv] float32.  q, k, v, decay and
 // beta are float32 rows with strides.  d at most 256.  With ones_column the rows of v hold dv - 1
 // values a head and column dv - 1 of every head takes a one for each token: a normaliser that is
-// gated and read like the matrix, out[t, h, dv - 1] being its product with the query.
+// gated and read like the matrix, out[t, h, dv - 1] being its product with the query.  silu_in: q, k and v
+// pass through silu on their way in (q before its scale).
 int kvc_linear_state_scan(float* out, const float* q, int64_t q_stride, const float* k,
                           int64_t k_stride, const float* v, int64_t v_stride, const float* decay,
                           int64_t decay_stride, const float* beta, int64_t beta_stride, float* state,
                           const int32_t* positions, const int32_t* token_req, const int32_t* q_start,
                           const int32_t* slots, int R, int nh, int nqk, int d, int dv, int delta_rule,
-                          float q_scale, int ones_column, kvc_stream stream);
+                          float q_scale, int ones_column, int silu_in, kvc_stream stream);
 // The gates of a matrix memory with log gates and a running maximum m (mLSTM), per request in
 // token order: i = cap tanh((i_raw + i_bias) / cap), f = logsigmoid(cap tanh((f_raw + f_bias) / cap)),
 // m_t = max(f + m_(t-1), i), keep[t, h] = exp(f + m_(t-1) - m_t), take[t, h] = exp(i - m_t),
@@ -273,10 +281,11 @@ int kvc_decay_and_write_gates(float* g, float* beta, const float* a_raw, int64_t
 // first_heads heads take first_scale instead of scale.
 int kvc_unit_heads(float* x, int64_t stride, int T, int heads, int d, float eps, float scale,
                    int first_heads, float first_scale, kvc_stream stream);
-// out[t, h, c] = o[t, h, c] / sqrt(mean_c o[t, h, :]^2 + eps) * gain[c] * silu(gate[t, h, c]).
+// out[t, h, c] = o[t, h, c] / sqrt(mean_c o[t, h, :]^2 + eps) * gain[c] * silu(gate[t, h, c]), or, with
+// sigmoid_gate, * sigmoid(gate[t, h, c]).  A norm over all heads at once is one head of their whole width.
 int kvc_head_rmsnorm_gate(void* out, int out_dtype, const float* o, const void* gate,
                           int64_t gate_stride, int gate_dtype, const float* gain, float eps, int T,
-                          int heads, int dv, kvc_stream stream);
+                          int heads, int dv, int sigmoid_gate, kvc_stream stream);
 
 // ---- routed experts (moe.hip); see the head of that file.  choice and weight are [T, top];
 // sorted [pairs]; tiles [max_tiles, 3] (expert, first sorted row, rows); num_tiles [1].
@@ -284,14 +293,17 @@ int kvc_head_rmsnorm_gate(void* out, int out_dtype, const float* o, const void* 
 // `gated` [E, 2N, K] (gate rows, then up rows) and the activation applied; a sorted row i reads
 // x row sorted[i] / in_div (in_div 0: row i itself) and writes out row i (out_sorted) or
 // sorted[i].  dtype is that of x and w.  packed: w is the copy kvc_pack_weight makes of the whole
-// stacked matrix (bfloat16, N a multiple of 16, K of 64).
+// stacked matrix (bfloat16, N a multiple of 16, K of 64).  act, of a product that is not gated: -1 none, 0 the
+// square of relu.  row_scale [pairs] (or null): multiplies a pair's sums before any activation, which is
+// what multiplying its input does.
 // bias [E] (or null) joins the logits.  score_fn 0: softmax over the experts, 1: sigmoid of each logit,
 // 2: the logit itself, the weights then being the softmax over the chosen logits.  correction [E] (or
 // null) is added to the scores for the choice alone.  group_best 1 or 2: a group is worth its best choice score, or
-// the sum of its best two.  The weights are multiplied by weight_scale.
+// the sum of its best two.  The weights (the chosen experts' scores over their sum, or, renormalize 0, as they
+// are) are multiplied by weight_scale.
 int kvc_moe_route(int32_t* choice, float* weight, const float* logits, int T, int E, int top,
                   int groups, int keep, int score_fn, const float* bias, const float* correction,
-                  int group_best, float weight_scale, kvc_stream stream);
+                  int group_best, int renormalize, float weight_scale, kvc_stream stream);
 // Tiles hold up to tile_rows rows, 16 or 64 (kvc_moe_tile_rows says which a step's size asks
 // for; 64 is for bfloat16 with K a multiple of 32).
 int kvc_moe_tile_rows(int pairs, int E);
@@ -300,16 +312,17 @@ int kvc_moe_tile_rows(int pairs, int E);
 // and gate[t] = sigmoid(x[t] . its last row).
 int kvc_moe_router(int32_t* choice, float* weight, const void* x, int64_t x_stride, int x_dtype,
                    const float* router, float* gate, int T, int H, int E, int top, int groups, int keep,
-                   int score_fn, const float* bias, const float* correction, int group_best, float weight_scale,
-                   kvc_stream stream);
+                   int score_fn, const float* bias, const float* correction, int group_best, int renormalize,
+                   float weight_scale, kvc_stream stream);
 int kvc_moe_max_tiles(int pairs, int E, int tile_rows);
 int kvc_moe_align(int32_t* sorted, int32_t* tiles, int32_t* num_tiles, const int32_t* choice,
                   int pairs, int E, int max_tiles, int tile_rows, kvc_stream stream);
 int kvc_moe_gemm(void* out, int64_t out_stride, int out_dtype, const void* x, int64_t x_stride,
                  const void* w, int dtype, const int32_t* sorted, const int32_t* tiles,
                  const int32_t* num_tiles, int max_tiles, int tile_rows, int N, int K, int in_div, int out_sorted,
-                 int gated, float limit, float alpha, float up_shift, int packed, kvc_stream stream);
-// out[t] = sum_c weight[t, c] * y[t * top + c] + add0[t] + add1[t] (either may be null; add0 of
+                 int gated, float limit, float alpha, float up_shift, int act, const float* row_scale, int packed,
+                 kvc_stream stream);
+// out[t] = sum_c weight[t, c] * y[t * top + c] (weight null: ones) + add0[t] + add1[t] (either may be null; add0 of
 // dtype add0_dtype, add1 float32), float32.  add1_gate [T] (or null): add1[t] is multiplied by it.
 // accumulate: the sum is added into out instead of stored.
 int kvc_moe_combine(float* out, const float* y, const float* weight, int top, const void* add0,
@@ -335,8 +348,9 @@ int kvc_moe_combine(float* out, const float* y, const float* weight, int top, co
 // kvc_decode_attention_max_table: the widest block table (entries per request) whose page ids
 // for one split still fit in a block's LDS; a wider one is refused, so engines check it when
 // they are built.
-// slopes, sinks (float32 [nh] or null) and chunk as for kvc_paged_attention; the kernel for portions
-// (kvc_prefill_attention) takes them too.
+// slopes, sinks (float32 [nh] or null), chunk, softcap and gate (here bfloat16) as for kvc_paged_attention; the
+// kernel for portions (kvc_prefill_attention) takes them too (gate rows 8-byte aligned).  values_are_keys as
+// for kvc_qk_norm_rope_kv_write: rows of qkv end with the k heads, which are the values too.
 int kvc_decode_attention_supported(int nh, int nkv, int d, int dv, int page_size, int dtype);
 int kvc_decode_attention_waves(int nh, int nkv, int d);
 int kvc_decode_attention_max_table(int nh, int nkv, int d);
@@ -347,8 +361,9 @@ int kvc_decode_attention(void* out, void* part_o, void* part_ml, const void* qkv
                          const float* sin_tab, int rot_dim, int interleaved, const float* q_gain,
                          const float* k_gain, float norm_eps, int write_kv, int T,
                          int nh, int nkv, int d, int dv, int page_size, int num_pages, float scale,
-                         int window, const float* slopes, int chunk, const float* sinks, int nsplit,
-                         int out_f32, kvc_stream stream);
+                         int window, const float* slopes, int chunk, const float* sinks, float softcap,
+                         const void* gate, int64_t gate_stride, int values_are_keys, int nsplit, int out_f32,
+                         kvc_stream stream);
 
 // The same attention for bfloat16 portions of prompts on the matrix cores: a block per
 // (tile of a request's tokens, kv head), keys staged through LDS.  q_start [R+1] bounds
@@ -367,22 +382,23 @@ int kvc_prefill_attention(void* out, const void* q, int64_t q_stride, const void
                           float scale, int window, const float* slopes, int chunk, const float* sinks, void* part_o,
                           void* part_ml, int nsplit,
                           const float* cos_tab, const float* sin_tab, int rot_dim, int interleaved,
-                          int out_f32, kvc_stream stream);
+                          float softcap, const void* gate, int64_t gate_stride, int out_f32, kvc_stream stream);
 
 // ---- norms after a sublayer, norms over a whole projection, gates per head (norm_ops.hip)
 // residual[t, :] += post_gain * delta[t, :] / sqrt(mean(delta[t, :]^2) + eps), and then, if out is
-// not null, out[t, :] = next_gain * residual[t, :] / sqrt(mean(residual[t, :]^2) + next_eps): the norm
+// not null, out[t, :] = next_gain * residual[t, :] / sqrt(mean(residual[t, :]^2) + next_eps) (next_gain null:
+// residual[t, :] as it is): the norm
 // behind a sublayer, the sum into the float32 stream and the norm before the next sublayer in one
 // pass.  delta is float32 (delta_dtype 0) or bfloat16 (1); out likewise (out_dtype).  slices > 1:
 // delta holds [slices, T, H] float32 partial sums of a product cut along K (kvc_gemm_mid_bf16 mode
-// 2) and a row of the result is their sum in slice order.  weight [T, slices] (or null): delta instead
-// holds [T, slices, H] float32, the results of a token's experts, and a row of the result is their sum
-// in order, each times its weight, plus add[t] (float32 [T, H], or null) times add_gate[t] ([T], or null:
+// 2) and a row of the result is their sum in slice order.  by_token: delta instead holds [T, slices, H]
+// float32, the results of a token's experts, and a row of the result is their sum in order, each times its
+// weight [T, slices] (null: ones), plus add[t] (float32 [T, H], or null) times add_gate[t] ([T], or null:
 // once): what kvc_moe_combine stores, added up on the way.
 int kvc_norm_add_norm(void* out, int out_dtype, float* residual, const void* delta, int delta_dtype,
                       const float* post_gain, float eps, const float* next_gain, float next_eps,
-                      int T, int H, int slices, const float* weight, const float* add, const float* add_gate,
-                      kvc_stream stream);
+                      int T, int H, int slices, int by_token, const float* weight, const float* add,
+                      const float* add_gate, kvc_stream stream);
 // Rows of attn are [heads][2][dv]: out[t, h] = (a1 - lambda * a2) / sqrt(mean((a1 - lambda * a2)^2) + eps)
 // * post over the head's dv values, out [T, heads * dv] of dtype; attn of attn_dtype (dtype, or float32);
 // float32 arithmetic.

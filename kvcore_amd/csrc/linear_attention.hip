@@ -4,8 +4,10 @@
 // kvc_linear_state_scan walks each request's tokens in order.  Two update rules:
 //   key decay   S <- diag(a_t) S + k_t v_t^T                      (a_t one factor per key channel)
 //   delta rule  S <- g_t S;  u = beta_t (v_t - S^T k_t);  S <- S + k_t u^T   (g_t, beta_t scalars)
-//   scalar gates  S <- g_t S + beta_t k_t v_t^T                   (g_t, beta_t scalars per head)
-// and in all o_t = S^T (q_scale q_t), read after the token's write.  A block owns one (request, head, tile
+//   scalar gates  S <- g_t S + beta_t k_t v_t^T                   (g_t, beta_t scalars per head; beta may be
+//                 absent, and one row of g serve every token)
+// and in all o_t = S^T (q_scale q_t), read after the token's write; q, k and v may pass through silu on
+// their way in.  A block owns one (request, head, tile
 // of VT value channels); the NSL threads that share a column of the state are neighbouring lanes
 // (their partial sums meet through lane permutations, in one fixed order) and each keeps NPT rows in
 // registers; q, k, the factors and v of 16 tokens at a time go through LDS.  A request whose
@@ -62,11 +64,12 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
     int64_t decay_stride, const float* __restrict__ beta, int64_t beta_stride, float* __restrict__ state,
     const int32_t* __restrict__ positions, const int32_t* __restrict__ token_req,
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ slots, int nh, int nqk, int d,
-    int dv, float q_scale, int scalar_gates, int ones_column) {
+    int dv, float q_scale, int scalar_gates, int ones_column, int silu_in) {
   constexpr int VT = 256 / NSL;  // value channels a block
   // with ones_column the rows of v hold dv - 1 values a head and the last column of the state's dv
   // takes a one for every token (a normaliser kept beside the matrix)
   const int dvin = dv - ones_column;
+  auto take_in = [&](float x) -> float { return silu_in ? silu_of(x) : x; };
   // FULL: d == NPT * NSL, so no row needs a bound, and a thread's rows of q, k and the factors lie
   // side by side in LDS (row n of a token at (n % NSL) * NPT + n / NSL), read 16 bytes at a time
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -207,20 +210,20 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       for (int j = 0; j < QN; ++j) {
         const int idx = tid + 256 * j, tt = idx / d, n = idx - tt * d;
         const int64_t t = t0 + (tt < nt ? tt : 0);
-        qn[j] = q[t * q_stride + hk * d + n] * q_scale;
-        kn[j] = k[t * k_stride + hk * d + n];
+        qn[j] = take_in(q[t * q_stride + hk * d + n]) * q_scale;
+        kn[j] = take_in(k[t * k_stride + hk * d + n]);
         if (!DELTA) an[j] = decay[t * decay_stride + h * d + n];
       }
       if (DELTA) {
         const int64_t t = t0 + (tid < nt ? tid : 0);
         an[0] = decay[t * decay_stride + h];
-        an[1] = beta[t * beta_stride + h];
+        an[1] = beta != nullptr ? beta[t * beta_stride + h] : 1.f;
       }
 #pragma unroll
       for (int j = 0; j < VN; ++j) {
         const int idx = tid + 256 * j, tt = idx / VT, cc = c0 + idx - tt * VT;
         const int64_t t = t0 + (tt < nt ? tt : 0);
-        vn[j] = cc < dvin ? v[t * v_stride + h * dvin + cc] : (cc < dv ? 1.f : 0.f);
+        vn[j] = cc < dvin ? take_in(v[t * v_stride + h * dvin + cc]) : (cc < dv ? 1.f : 0.f);
       }
     };
     auto stash = [&](float* base) {
@@ -269,19 +272,19 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         const int tt = idx / d, n = idx - tt * d;
         const int64_t t = t0 + tt;
         const int at = FULL ? tt * d + (n % NSL) * NPT + n / NSL : idx;
-        q_s[at] = q[t * q_stride + hk * d + n] * q_scale;
-        k_s[at] = k[t * k_stride + hk * d + n];
+        q_s[at] = take_in(q[t * q_stride + hk * d + n]) * q_scale;
+        k_s[at] = take_in(k[t * k_stride + hk * d + n]);
         if (!DELTA) a_s[at] = decay[t * decay_stride + h * d + n];
       }
       if (DELTA) {
         for (int tt = tid; tt < nt; tt += nthreads) {
           a_s[2 * tt] = decay[static_cast<int64_t>(t0 + tt) * decay_stride + h];
-          a_s[2 * tt + 1] = beta[static_cast<int64_t>(t0 + tt) * beta_stride + h];
+          a_s[2 * tt + 1] = beta != nullptr ? beta[static_cast<int64_t>(t0 + tt) * beta_stride + h] : 1.f;
         }
       }
       for (int idx = tid; idx < nt * VT; idx += nthreads) {
         const int tt = idx / VT, cc = c0 + idx - tt * VT;
-        v_s[idx] = cc < dvin ? v[static_cast<int64_t>(t0 + tt) * v_stride + h * dvin + cc] : (cc < dv ? 1.f : 0.f);
+        v_s[idx] = cc < dvin ? take_in(v[static_cast<int64_t>(t0 + tt) * v_stride + h * dvin + cc]) : (cc < dv ? 1.f : 0.f);
       }
       __syncthreads();
       work_stage(q_s, k_s, a_s, v_s, t0, nt);
@@ -335,12 +338,12 @@ __global__ __launch_bounds__(256) void unit_heads_kernel(float* __restrict__ x, 
   for (int i = lane; i < d; i += kWave) p[i] *= inv;
 }
 
-// out[t, h, c] = o[t, h, c] / sqrt(mean_c o^2 + eps) * gain[c] * silu(gate[t, h, c]): the norm of
-// every head first, then the gate.  A wave a (token, head).
+// out[t, h, c] = o[t, h, c] / sqrt(mean_c o^2 + eps) * gain[c] * act(gate[t, h, c]), act silu or
+// (sigmoid_gate) the sigmoid: the norm of every head first, then the gate.  A wave a (token, head).
 template <typename TG, typename TO>
 __global__ __launch_bounds__(256) void head_rmsnorm_gate_kernel(
     TO* __restrict__ out, const float* __restrict__ o, const TG* __restrict__ gate, int64_t gate_stride,
-    const float* __restrict__ gain, float eps, int T, int heads, int dv) {
+    const float* __restrict__ gain, float eps, int T, int heads, int dv, int sigmoid_gate) {
   const int lane = threadIdx.x & (kWave - 1);
   const int64_t item = static_cast<int64_t>(blockIdx.x) * 4 + threadIdx.x / kWave;
   if (item >= static_cast<int64_t>(T) * heads) return;
@@ -353,7 +356,41 @@ __global__ __launch_bounds__(256) void head_rmsnorm_gate_kernel(
   const float inv = 1.f / sqrtf(ss / static_cast<float>(dv) + eps);
   TO* op = out + (static_cast<int64_t>(t) * heads + h) * dv;
   for (int i = lane; i < dv; i += kWave)
-    op[i] = from_float<TO>(p[i] * inv * gain[i] * silu_ff(to_float(gp[i])));
+    op[i] = from_float<TO>(p[i] * inv * gain[i] * (sigmoid_gate ? sigmoid_f(to_float(gp[i])) : silu_ff(to_float(gp[i]))));
+}
+
+// The same for wide heads (a norm over all heads at once is one wide head): a block a (token, head), four
+// values a thread at a time.
+template <typename TG, typename TO>
+__global__ __launch_bounds__(256) void wide_rmsnorm_gate_kernel(
+    TO* __restrict__ out, const float* __restrict__ o, const TG* __restrict__ gate, int64_t gate_stride,
+    const float* __restrict__ gain, float eps, int heads, int dv, int sigmoid_gate) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, h = blockIdx.y;
+  const float* p = o + (static_cast<int64_t>(t) * heads + h) * dv;
+  const TG* gp = gate + t * gate_stride + static_cast<int64_t>(h) * dv;
+  TO* op = out + (static_cast<int64_t>(t) * heads + h) * dv;
+  float ss = 0.f;
+  for (int i = 4 * threadIdx.x; i < dv; i += 4 * blockDim.x) {
+    const float4 v = *reinterpret_cast<const float4*>(p + i);
+    ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+  }
+  const float inv = 1.f / sqrtf(block_sum(ss, scratch) / static_cast<float>(dv) + eps);
+  for (int i = 4 * threadIdx.x; i < dv; i += 4 * blockDim.x) {
+    const float4 v = *reinterpret_cast<const float4*>(p + i), w = *reinterpret_cast<const float4*>(gain + i);
+    const float x[4] = {v.x, v.y, v.z, v.w}, gn[4] = {w.x, w.y, w.z, w.w};
+    alignas(16) TG g[4];
+    if constexpr (sizeof(TG) == 4) *reinterpret_cast<float4*>(g) = *reinterpret_cast<const float4*>(gp + i);
+    else *reinterpret_cast<uint2*>(g) = *reinterpret_cast<const uint2*>(gp + i);
+    alignas(16) TO y[4];
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      const float z = to_float(g[c]);
+      y[c] = from_float<TO>(x[c] * inv * gn[c] * (sigmoid_gate ? sigmoid_f(z) : silu_ff(z)));
+    }
+    if constexpr (sizeof(TO) == 4) *reinterpret_cast<float4*>(op + i) = *reinterpret_cast<const float4*>(y);
+    else *reinterpret_cast<uint2*>(op + i) = *reinterpret_cast<const uint2*>(y);
+  }
 }
 
 
@@ -536,7 +573,7 @@ extern "C" int kvc_linear_state_scan(float* out, const float* q, int64_t q_strid
                                      int64_t beta_stride, float* state, const int32_t* positions,
                                      const int32_t* token_req, const int32_t* q_start,
                                      const int32_t* slots, int R, int nh, int nqk, int d, int dv,
-                                     int rule, float q_scale, int ones_column,
+                                     int rule, float q_scale, int ones_column, int silu_in,
                                      kvc_stream stream) {
   ones_column = ones_column ? 1 : 0;
   if (rule < 0 || rule > 2) return kvc_fail("kvc_linear_state_scan: the rule is 0 (key decay), 1 (delta) or 2 (scalar gates)");
@@ -545,10 +582,11 @@ extern "C" int kvc_linear_state_scan(float* out, const float* q, int64_t q_strid
   if (R < 0 || nh <= 0 || nqk <= 0 || nh % nqk || d <= 0 || dv <= 0)
     return kvc_fail("kvc_linear_state_scan: bad sizes");
   if (d > 256) return kvc_fail("kvc_linear_state_scan: at most 256 key channels a head");
-  if (delta_rule && beta == nullptr) return kvc_fail("kvc_linear_state_scan: this rule needs beta");
-  if (delta_rule && beta_stride < nh) return kvc_fail("kvc_linear_state_scan: rows of beta too short for the heads");
+  if (rule == 1 && beta == nullptr) return kvc_fail("kvc_linear_state_scan: this rule needs beta");
+  if (delta_rule && beta != nullptr && beta_stride < nh) return kvc_fail("kvc_linear_state_scan: rows of beta too short for the heads");
   if (q_stride < static_cast<int64_t>(nqk) * d || k_stride < static_cast<int64_t>(nqk) * d ||
-      v_stride < static_cast<int64_t>(nh) * (dv - ones_column) || dv - ones_column <= 0 || decay_stride < (delta_rule ? nh : static_cast<int64_t>(nh) * d))
+      v_stride < static_cast<int64_t>(nh) * (dv - ones_column) || dv - ones_column <= 0 ||
+      (decay_stride < (delta_rule ? nh : static_cast<int64_t>(nh) * d) && !(scalar_gates && decay_stride == 0)))
     return kvc_fail("kvc_linear_state_scan: rows too short for the heads");
   if (R == 0) return 0;
   // tiles of 64 value channels with 4 threads a column, or, where that leaves compute units
@@ -565,7 +603,7 @@ extern "C" int kvc_linear_state_scan(float* out, const float* q, int64_t q_strid
   hipLaunchKernelGGL((linear_state_scan_kernel<NPT, DELTA, NSL_, FULL_, PF_>), grid, dim3(256),               \
                      lds*(PF_ ? 2 : 1), S(stream), out, q, q_stride, k, k_stride, v, v_stride, decay,         \
                      decay_stride, beta, beta_stride, state, positions, token_req, q_start, slots, nh, nqk, d, \
-                     dv, q_scale, scalar_gates, ones_column)
+                     dv, q_scale, scalar_gates, ones_column, silu_in)
   // two sets of LDS buffers (the next stage fetched while one is worked on) where a stage's values
   // deal out evenly to the threads and both sets fit the 64 KB a block may take
 #define KVC_LSCAN(NPT, DELTA, NSL_)                                                  \
@@ -642,15 +680,26 @@ extern "C" int kvc_unit_heads(float* x, int64_t stride, int T, int heads, int d,
 
 extern "C" int kvc_head_rmsnorm_gate(void* out, int out_dtype, const float* o, const void* gate,
                                      int64_t gate_stride, int gate_dtype, const float* gain, float eps,
-                                     int T, int heads, int dv, kvc_stream stream) {
+                                     int T, int heads, int dv, int sigmoid_gate, kvc_stream stream) {
   if (T < 0 || heads <= 0 || dv <= 0 || gate_stride < static_cast<int64_t>(heads) * dv)
     return kvc_fail("kvc_head_rmsnorm_gate: bad sizes");
   if (T == 0) return 0;
   const int64_t waves = static_cast<int64_t>(T) * heads;
   const dim3 grid(static_cast<unsigned>((waves + 3) / 4));
-#define KVC_HRG(TG, TO)                                                                                  \
-  hipLaunchKernelGGL((head_rmsnorm_gate_kernel<TG, TO>), grid, dim3(256), 0, S(stream), static_cast<TO*>(out), o, \
-                     static_cast<const TG*>(gate), gate_stride, gain, eps, T, heads, dv)
+  // wide heads whose rows 16-byte loads divide take a block each
+  const bool wide = dv > 256 && dv % 4 == 0 && gate_stride % 4 == 0 && heads <= 65535 &&
+                    ((reinterpret_cast<uintptr_t>(out) | reinterpret_cast<uintptr_t>(o) |
+                      reinterpret_cast<uintptr_t>(gate) | reinterpret_cast<uintptr_t>(gain)) & 15) == 0;
+#define KVC_HRG(TG, TO)                                                                                           \
+  do {                                                                                                            \
+    if (wide)                                                                                                     \
+      hipLaunchKernelGGL((wide_rmsnorm_gate_kernel<TG, TO>), dim3(T, heads), dim3(256), 0, S(stream),             \
+                         static_cast<TO*>(out), o, static_cast<const TG*>(gate), gate_stride, gain, eps, heads,   \
+                         dv, sigmoid_gate);                                                                       \
+    else                                                                                                          \
+      hipLaunchKernelGGL((head_rmsnorm_gate_kernel<TG, TO>), grid, dim3(256), 0, S(stream), static_cast<TO*>(out), o, \
+                         static_cast<const TG*>(gate), gate_stride, gain, eps, T, heads, dv, sigmoid_gate);       \
+  } while (0)
   if (gate_dtype == 0 && out_dtype == 0) {
     KVC_HRG(float, float);
   } else if (gate_dtype == 0 && out_dtype == 1) {

@@ -10,8 +10,9 @@
 //                    an optional correction per expert: the `keep` groups that are worth most (a
 //                    group's best choice score, or the sum of its best two); the `top` best experts of
 //                    those groups (the lower index on a tie); weights = the chosen experts' plain
-//                    scores / (their sum + 1e-20) * weight_scale, or, where the scores are the logits,
-//                    the softmax over the chosen logits * weight_scale.  A wave a token.
+//                    scores / (their sum + 1e-20) * weight_scale, or (renormalize 0) the scores as they
+//                    are * weight_scale, or, where the scores are the logits, the softmax over the chosen
+//                    logits * weight_scale.  A wave a token.
 //   kvc_moe_router   the router's product (float32 sums in one fixed order over rows of either dtype)
 //                    and the choice in one kernel; a further row of the router's matrix may give one
 //                    number a token, a sigmoid gate for an expert that every token runs.
@@ -20,11 +21,13 @@
 //   kvc_moe_gemm     for every tile, rows x that expert's matrix.  Gated: gate and up rows of the
 //                    expert side by side in one pass, and the activation
 //                    min(g, limit) * sigmoid(alpha * g) * (clamp(u, -limit, limit) + up_shift) on the way
-//                    out (an infinite limit, alpha 1 and up_shift 0: silu(g) * u).
+//                    out (an infinite limit, alpha 1 and up_shift 0: silu(g) * u).  Not gated: the rows as
+//                    they are, or their square of relu.  row_scale: a number a pair that multiplies the
+//                    pair's input (the sums, before any activation).
 //                    bfloat16 operands go through the matrix cores (16 x 16 x 32, the expert's rows as
 //                    the A operand, the tokens as B) with float32 sums; float32 operands, and rows
 //                    that 16-byte loads do not divide, are summed in float32 in index order.  A row's sums do not depend on which tile it is in.
-//   kvc_moe_combine  out[t] = sum_c weight[t, c] * y[t * top + c] (+ up to two more row sets, the second
+//   kvc_moe_combine  out[t] = sum_c weight[t, c] * y[t * top + c] (without weights: the plain sum) (+ up to two more row sets, the second
 //                    times a number a token where one is given), float32, in the order of the
 //                    choices; or added into out (the residual stream).
 
@@ -43,6 +46,15 @@ namespace {
 constexpr int kTileRows = 16;
 constexpr int kBigTileRows = 64;
 
+// What happens to the sums of an ungated product on their way out (the codes of kvc_activation; -1: nothing).
+__device__ __forceinline__ float plain_act(float v, int act) {
+  if (act == 0) {
+    v = fmaxf(v, 0.f);
+    return v * v;
+  }
+  return v;
+}
+
 // the lane that holds the largest value (the lowest index among equals) tells everyone
 __device__ __forceinline__ void wave_argmax(float& val, int& idx) {
 #pragma unroll
@@ -59,12 +71,13 @@ __device__ __forceinline__ void wave_argmax(float& val, int& idx) {
 // How a token's experts are chosen from its logits (+ bias[e], which may be null).  score_fn 0: softmax
 // over the experts, 1: a sigmoid of each logit, 2: the logit itself.  The choice is made on score +
 // correction[e] (correction may be null) and may so be negative; the weights are the plain scores of
-// the chosen, over their sum (+ 1e-20), or (2) the softmax over the chosen logits, times weight_scale.
+// the chosen, over their sum (+ 1e-20) where `renormalize` is set, or (2) the softmax over the chosen
+// logits, times weight_scale.
 // With keep < groups only the experts of the best `keep` of `groups` equal
 // groups of neighbours may be chosen; a group is worth the sum of its `group_best` (1 or 2) largest
 // choice scores.  The lower index wins a tie.
 struct RouteRule {
-  int top, groups, keep, score_fn, group_best;
+  int top, groups, keep, score_fn, group_best, renormalize;
   const float* bias;
   const float* correction;
   float weight_scale;
@@ -159,7 +172,7 @@ __device__ __forceinline__ void route_one(int32_t* __restrict__ choice, float* _
     if (lane == 0) pk[idx] = -INFINITY;
     __builtin_amdgcn_wave_barrier();
   }
-  float norm = rule.weight_scale / (total + 1e-20f);
+  float norm = rule.renormalize ? rule.weight_scale / (total + 1e-20f) : rule.weight_scale;
   if (rule.score_fn == 2) {  // the softmax over the chosen logits alone
     const float mx = wave_max(mine_ok ? mine : -INFINITY);
     mine = mine_ok ? expf(mine - mx) : 0.f;
@@ -359,7 +372,8 @@ template <int GATED, typename TO, int PACKED>
 __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
     TO* __restrict__ out, int64_t out_stride, const bf16_t* __restrict__ x, int64_t x_stride,
     const bf16_t* __restrict__ w, const int32_t* __restrict__ sorted, const int32_t* __restrict__ tiles,
-    const int32_t* __restrict__ num_tiles, int N, int K, int in_div, int out_sorted, float limit, float alpha, float shift) {
+    const int32_t* __restrict__ num_tiles, int N, int K, int in_div, int out_sorted, float limit, float alpha, float shift,
+    int act, const float* __restrict__ row_scale) {
   const int tile = blockIdx.x;
   if (tile >= *num_tiles) return;
   const int e = tiles[3 * tile], r0 = tiles[3 * tile + 1], nr = tiles[3 * tile + 2];
@@ -447,10 +461,10 @@ __global__ __launch_bounds__(256) void moe_gemm_bf16_kernel(
   }
   // lane holds column (token) li, rows (features) n0 + 4 * lk + i
   if (!row_ok) return;
-  if (GATED) {
+  const float scale = row_scale != nullptr ? row_scale[pair] : 1.f;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] = clamped_glu(acc[i], acc2[i], limit, alpha, shift);
-  }
+  for (int i = 0; i < 4; ++i)
+    acc[i] = GATED ? clamped_glu(acc[i] * scale, acc2[i] * scale, limit, alpha, shift) : plain_act(acc[i] * scale, act);
   const int64_t out_row = out_sorted ? r0 + li : pair;
   const int nf = n0 + 4 * lk;
   if (nf < N) store4<TO>(out + out_row * out_stride + nf, acc, N - nf);
@@ -465,7 +479,8 @@ template <int GATED, typename TO, int PACKED>
 __global__ __launch_bounds__(256) void moe_gemm_tiled_kernel(
     TO* __restrict__ out, int64_t out_stride, const bf16_t* __restrict__ x, int64_t x_stride,
     const bf16_t* __restrict__ w, const int32_t* __restrict__ sorted, const int32_t* __restrict__ tiles,
-    const int32_t* __restrict__ num_tiles, int N, int K, int in_div, int out_sorted, float limit, float alpha, float shift) {
+    const int32_t* __restrict__ num_tiles, int N, int K, int in_div, int out_sorted, float limit, float alpha, float shift,
+    int act, const float* __restrict__ row_scale) {
   constexpr int NF = GATED ? 2 : 4;   // column blocks of 16 a wave
   constexpr int NR = kBigTileRows / 16;
   constexpr int KC = 64;              // values of K a pass (two matrix instructions deep)
@@ -565,14 +580,16 @@ __global__ __launch_bounds__(256) void moe_gemm_tiled_kernel(
   for (int r = 0; r < NR; ++r) {
     const int row = 16 * r + li;
     if (row >= nr) continue;
-    const int64_t out_row = out_sorted ? r0 + row : sorted[r0 + row];
+    const int pair = sorted[r0 + row];
+    const int64_t out_row = out_sorted ? r0 + row : pair;
+    const float scale = row_scale != nullptr ? row_scale[pair] : 1.f;
 #pragma unroll
     for (int f = 0; f < NF; ++f) {
       f32x4_t v = acc[f][r];
-      if (GATED) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = clamped_glu(v[i], acc2[f][r][i], limit, alpha, shift);
-      }
+      for (int i = 0; i < 4; ++i)
+        v[i] = GATED ? clamped_glu(v[i] * scale, acc2[GATED ? f : 0][r][i] * scale, limit, alpha, shift)
+                     : plain_act(v[i] * scale, act);
       const int nf = n0 + 16 * f + 4 * lk;
       if (nf < N) store4<TO>(out + out_row * out_stride + nf, v, N - nf);
     }
@@ -585,7 +602,8 @@ template <int GATED, typename TI, typename TO>
 __global__ __launch_bounds__(256) void moe_gemm_plain_kernel(
     TO* __restrict__ out, int64_t out_stride, const TI* __restrict__ x, int64_t x_stride,
     const TI* __restrict__ w, const int32_t* __restrict__ sorted, const int32_t* __restrict__ tiles,
-    const int32_t* __restrict__ num_tiles, int N, int K, int in_div, int out_sorted, float limit, float alpha, float shift) {
+    const int32_t* __restrict__ num_tiles, int N, int K, int in_div, int out_sorted, float limit, float alpha, float shift,
+    int act, const float* __restrict__ row_scale) {
   const int tile = blockIdx.x;
   if (tile >= *num_tiles) return;
   const int e = tiles[3 * tile], r0 = tiles[3 * tile + 1], nr = tiles[3 * tile + 2];
@@ -604,7 +622,9 @@ __global__ __launch_bounds__(256) void moe_gemm_plain_kernel(
       acc = fmaf(xv, to_float(wr[k]), acc);
       if (GATED) acc2 = fmaf(xv, to_float(wr[static_cast<int64_t>(N) * K + k]), acc2);
     }
-    out[out_row * out_stride + n] = from_float<TO>(GATED ? clamped_glu(acc, acc2, limit, alpha, shift) : acc);
+    const float scale = row_scale != nullptr ? row_scale[pair] : 1.f;
+    out[out_row * out_stride + n] = from_float<TO>(
+        GATED ? clamped_glu(acc * scale, acc2 * scale, limit, alpha, shift) : plain_act(acc * scale, act));
   }
 }
 
@@ -619,7 +639,8 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ ou
   const int t = static_cast<int>(idx / H), c = static_cast<int>(idx - static_cast<int64_t>(t) * H);
   float acc = 0.f;
   for (int j = 0; j < top; ++j)
-    acc = fmaf(weight[static_cast<int64_t>(t) * top + j], y[(static_cast<int64_t>(t) * top + j) * H + c], acc);
+    acc = fmaf(weight != nullptr ? weight[static_cast<int64_t>(t) * top + j] : 1.f,
+               y[(static_cast<int64_t>(t) * top + j) * H + c], acc);
   if (add0 != nullptr) acc += to_float(add0[idx]);
   if (add1 != nullptr) acc = add1_gate != nullptr ? fmaf(add1_gate[t], add1[idx], acc) : acc + add1[idx];
   out[idx] = accumulate ? out[idx] + acc : acc;
@@ -629,13 +650,13 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ ou
 
 extern "C" int kvc_moe_route(int32_t* choice, float* weight, const float* logits, int T, int E, int top,
                              int groups, int keep, int score_fn, const float* bias, const float* correction,
-                             int group_best, float weight_scale, kvc_stream stream) {
+                             int group_best, int renormalize, float weight_scale, kvc_stream stream) {
   if (T < 0 || E <= 0 || top <= 0 || top > E || top > kWave || groups <= 0 || E % groups || keep <= 0 ||
       keep > groups)
     return kvc_fail("kvc_moe_route: bad sizes (at most 64 choices; the experts in equal groups)");
   if (score_fn < 0 || score_fn > 2 || (group_best != 1 && group_best != 2))
     return kvc_fail("kvc_moe_route: scores by softmax (0), sigmoid (1) or logit (2); a group is worth its best 1 or 2");
-  const RouteRule rule{top, groups, keep, score_fn, group_best, bias, correction, weight_scale};
+  const RouteRule rule{top, groups, keep, score_fn, group_best, renormalize, bias, correction, weight_scale};
   const size_t lds = sizeof(float) * 4 * (2 * E + groups);
   if (lds > 60000) return kvc_fail("kvc_moe_route: too many experts for a wave's scores in LDS");
   if (T == 0) return 0;
@@ -647,13 +668,13 @@ extern "C" int kvc_moe_route(int32_t* choice, float* weight, const float* logits
 extern "C" int kvc_moe_router(int32_t* choice, float* weight, const void* x, int64_t x_stride, int x_dtype,
                               const float* router, float* gate, int T, int H, int E, int top, int groups, int keep,
                               int score_fn, const float* bias, const float* correction, int group_best,
-                              float weight_scale, kvc_stream stream) {
+                              int renormalize, float weight_scale, kvc_stream stream) {
   if (T < 0 || H <= 0 || E <= 0 || top <= 0 || top > E || top > kWave || groups <= 0 || E % groups || keep <= 0 ||
       keep > groups || x_stride < H)
     return kvc_fail("kvc_moe_router: bad sizes (at most 64 choices; the experts in equal groups)");
   if (score_fn < 0 || score_fn > 2 || (group_best != 1 && group_best != 2))
     return kvc_fail("kvc_moe_router: scores by softmax (0), sigmoid (1) or logit (2); a group is worth its best 1 or 2");
-  const RouteRule rule{top, groups, keep, score_fn, group_best, bias, correction, weight_scale};
+  const RouteRule rule{top, groups, keep, score_fn, group_best, renormalize, bias, correction, weight_scale};
   if (T == 0) return 0;
   const size_t lds = sizeof(float) * (static_cast<size_t>(kRouterWaves) * (kRouterRows * kRouterPad + kRouterTokens) +
                                       static_cast<size_t>(kRouterTokens) * (2 * E + groups));
@@ -704,15 +725,17 @@ extern "C" int kvc_moe_align(int32_t* sorted, int32_t* tiles, int32_t* num_tiles
 extern "C" int kvc_moe_gemm(void* out, int64_t out_stride, int out_dtype, const void* x, int64_t x_stride,
                             const void* w, int dtype, const int32_t* sorted, const int32_t* tiles,
                             const int32_t* num_tiles, int max_tiles, int tile_rows, int N, int K, int in_div,
-                            int out_sorted, int gated, float limit, float alpha, float up_shift, int packed,
-                            kvc_stream stream) {
+                            int out_sorted, int gated, float limit, float alpha, float up_shift, int act,
+                            const float* row_scale, int packed, kvc_stream stream) {
   if (max_tiles < 0 || N <= 0 || K <= 0 || x_stride < K || out_stride < N)
     return kvc_fail("kvc_moe_gemm: bad sizes");
   if (tile_rows != kTileRows && tile_rows != kBigTileRows) return kvc_fail("kvc_moe_gemm: tiles of 16 or 64 rows");
+  if (act < -1 || act > 0 || (gated && act != -1))
+    return kvc_fail("kvc_moe_gemm: an ungated product has no activation (-1) or the square of relu (0)");
   if (max_tiles == 0) return 0;
   dim3 grid(max_tiles, (N + 63) / 64);
   if (grid.y > 65535u) return kvc_fail("kvc_moe_gemm: too many columns");
-#define KVC_MOE_ARGS sorted, tiles, num_tiles, N, K, in_div, out_sorted, limit, alpha, up_shift
+#define KVC_MOE_ARGS sorted, tiles, num_tiles, N, K, in_div, out_sorted, limit, alpha, up_shift, act, row_scale
 #define KVC_MOE_LAUNCH(KERNEL, TI, TO)                                                                          \
   hipLaunchKernelGGL(KERNEL, grid, dim3(256), 0, S(stream), static_cast<TO*>(out), out_stride,                   \
                      static_cast<const TI*>(x), x_stride, static_cast<const TI*>(w), KVC_MOE_ARGS)

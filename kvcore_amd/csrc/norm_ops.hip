@@ -2,7 +2,8 @@
 //
 // kvc_norm_add_norm: a layer that norms a sublayer's result before it joins the stream
 // (x <- x + norm_b(f(norm_a(x)))) needs, between two sublayers, the norm of the result, the sum
-// into the float32 stream and the norm of the new stream: one block a row does all three with
+// into the float32 stream and the norm of the new stream (or, where sublayers read the stream as it is,
+// the new stream itself, rounded to the model's dtype): one block a row does all three with
 // the row in registers (rows of a multiple of 8 values up to 16,384), or from memory otherwise.
 // kvc_wide_qk_norm: the query and key norms of an attention whose norm spans all heads at once.
 // kvc_latent_rows: the two latent norms of a latent attention and its one key/value row a token.
@@ -49,13 +50,13 @@ __device__ __forceinline__ void st8(bf16_t* p, const float* v) {
 }
 
 // Where a row of a sublayer's result comes from.  Plain: the row itself, or, where the product before
-// left partial sums of slices along K ([slices, T, H] float32), their sum in slice order.  Weighted
-// (`weight` is not null): the results of a token's experts ([T, slices, H] float32), each times its
-// weight, and a further row times a number a token.
+// left partial sums of slices along K ([slices, T, H] float32), their sum in slice order.  By token
+// (`by_token`): the results of a token's experts ([T, slices, H] float32), each times its weight (once
+// where there is none), and a further row times a number a token.
 struct SumRule {
-  int slices;
+  int slices, by_token;
   int64_t row_stride, slice_stride;
-  const float* weight;    // [T, slices]
+  const float* weight;    // [T, slices] or null (ones)
   const float* add;       // [T, H] or null
   const float* add_gate;  // [T] or null (one)
 };
@@ -64,7 +65,7 @@ struct SumRule {
 template <typename TD>
 __device__ __forceinline__ void ld8_sum(const TD* delta, const SumRule& rule, int64_t t, int H, int e, float* v) {
   const TD* p = delta + t * rule.row_stride + e;
-  if (rule.weight == nullptr) {
+  if (!rule.by_token) {
     ld8(p, v);
     for (int s = 1; s < rule.slices; ++s) {
       float u[8];
@@ -77,7 +78,7 @@ __device__ __forceinline__ void ld8_sum(const TD* delta, const SumRule& rule, in
 #pragma unroll
   for (int i = 0; i < 8; ++i) v[i] = 0.f;
   for (int s = 0; s < rule.slices; ++s) {
-    const float w = rule.weight[t * rule.slices + s];
+    const float w = rule.weight != nullptr ? rule.weight[t * rule.slices + s] : 1.f;
     float u[8];
     ld8(p + s * rule.slice_stride, u);
 #pragma unroll
@@ -94,13 +95,14 @@ __device__ __forceinline__ void ld8_sum(const TD* delta, const SumRule& rule, in
 template <typename TD>
 __device__ __forceinline__ float ld_sum(const TD* delta, const SumRule& rule, int64_t t, int H, int e) {
   const TD* p = delta + t * rule.row_stride + e;
-  if (rule.weight == nullptr) {
+  if (!rule.by_token) {
     float v = to_float(p[0]);
     for (int s = 1; s < rule.slices; ++s) v += to_float(p[s * rule.slice_stride]);
     return v;
   }
   float v = 0.f;
-  for (int s = 0; s < rule.slices; ++s) v = fmaf(rule.weight[t * rule.slices + s], to_float(p[s * rule.slice_stride]), v);
+  for (int s = 0; s < rule.slices; ++s)
+    v = fmaf(rule.weight != nullptr ? rule.weight[t * rule.slices + s] : 1.f, to_float(p[s * rule.slice_stride]), v);
   if (rule.add != nullptr) v = fmaf(rule.add_gate != nullptr ? rule.add_gate[t] : 1.f, rule.add[t * H + e], v);
   return v;
 }
@@ -127,8 +129,12 @@ __global__ __launch_bounds__(256) void norm_add_norm_kernel(
     ss += v * v;
   }
   if (out == nullptr) return;  // the same for the whole grid
-  const float inv = rsqrtf(block_sum(ss, scratch) / static_cast<float>(H) + next_eps);
   TO* o = out + base;
+  if (next_gain == nullptr) {  // the stream as it is
+    for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = from_float<TO>(r[i]);
+    return;
+  }
+  const float inv = rsqrtf(block_sum(ss, scratch) / static_cast<float>(H) + next_eps);
   for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = from_float<TO>(next_gain[i] * (r[i] * inv));
 }
 
@@ -167,9 +173,10 @@ __global__ __launch_bounds__(256) void norm_add_norm_vec_kernel(
         ss += v[c][i] * v[c][i];
       }
       st8(residual + base + e, v[c]);
+      if (out != nullptr && next_gain == nullptr) st8(out + base + e, v[c]);  // the stream as it is
     }
   }
-  if (out == nullptr) return;  // the same for the whole grid
+  if (out == nullptr || next_gain == nullptr) return;  // the same for the whole grid
   const float inv = rsqrtf(block_sum(ss, scratch) / static_cast<float>(H) + next_eps);
 #pragma unroll
   for (int c = 0; c < NCH; ++c) {
@@ -317,19 +324,17 @@ __global__ __launch_bounds__(256) void diff_heads_norm_kernel(T* __restrict__ ou
 
 extern "C" int kvc_norm_add_norm(void* out, int out_dtype, float* residual, const void* delta, int delta_dtype,
                                  const float* post_gain, float eps, const float* next_gain, float next_eps,
-                                 int T, int H, int slices, const float* weight, const float* add,
+                                 int T, int H, int slices, int by_token, const float* weight, const float* add,
                                  const float* add_gate, kvc_stream stream) {
   if (T < 0 || H <= 0 || slices < 1) return kvc_fail("kvc_norm_add_norm: bad sizes");
-  if ((slices > 1 || weight != nullptr) && delta_dtype != 0)
-    return kvc_fail("kvc_norm_add_norm: partial sums and weighted rows are float32");
-  if (weight == nullptr && (add != nullptr || add_gate != nullptr))
-    return kvc_fail("kvc_norm_add_norm: a further row joins weighted rows only");
+  if ((slices > 1 || by_token) && delta_dtype != 0)
+    return kvc_fail("kvc_norm_add_norm: partial sums and the rows of a token's experts are float32");
+  if (!by_token && (weight != nullptr || add != nullptr || add_gate != nullptr))
+    return kvc_fail("kvc_norm_add_norm: weights and a further row belong to the rows of a token's experts");
   if (residual == nullptr || delta == nullptr || post_gain == nullptr) return kvc_fail("kvc_norm_add_norm: null operand");
-  if (out != nullptr && next_gain == nullptr) return kvc_fail("kvc_norm_add_norm: the second norm needs its gain");
   if (T == 0) return 0;
-  if (out == nullptr) next_gain = post_gain;  // never read
-  SumRule rule{slices, H, static_cast<int64_t>(T) * H, weight, add, add_gate};
-  if (weight != nullptr) {  // a token's rows lie one after the other
+  SumRule rule{slices, by_token, H, static_cast<int64_t>(T) * H, weight, add, add_gate};
+  if (by_token) {  // a token's rows lie one after the other
     rule.row_stride = static_cast<int64_t>(slices) * H;
     rule.slice_stride = H;
   }

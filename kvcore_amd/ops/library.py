@@ -49,7 +49,7 @@ def _declare(lib: ctypes.CDLL) -> None:
         "kvc_hyper_step": [P, I, P, P, I, I, P, I, P, P, F, P, P, F, I, I, I, P],
         "kvc_spread_streams": [P, P, I, I, I, P],
         "kvc_diff_heads_norm": [P, P, L, I, F, F, F, I, I, I, I, P],
-        "kvc_norm_add_norm": [P, I, P, P, I, P, F, P, F, I, I, I, P, P, P, P],
+        "kvc_norm_add_norm": [P, I, P, P, I, P, F, P, F, I, I, I, I, P, P, P, P],
         "kvc_wide_qk_norm": [P, L, P, P, F, I, I, I, I, I, P],
         "kvc_head_gate": [P, P, L, P, L, I, I, I, I, I, I, P],
         "kvc_latent_rows": [P, L, P, P, L, P, L, P, P, F, I, I, I, I, I, P],
@@ -57,23 +57,23 @@ def _declare(lib: ctypes.CDLL) -> None:
         "kvc_max_gated_finish": [P, I, P, P, P, L, I, P, F, F, I, I, I, P],
         "kvc_gather_rows": [P, P, P, I, I, I, I, P],
         "kvc_to_float": [P, P, L, I, P],
-        "kvc_rope_table": [P, P, P, P, I, I, P],
+        "kvc_rope_table": [P, P, P, P, F, I, I, P],
         "kvc_kv_slots": [P, P, P, P, P, I, I, I, I, P],
         "kvc_rope_kv_write": [P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, I, P],
-        "kvc_paged_attention": [P, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, P, I, P, I, I, P],
-        "kvc_linear_state_scan": [P, P, L, P, L, P, L, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, F, I, P],
+        "kvc_paged_attention": [P, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, P, I, P, F, P, L, I, I, P],
+        "kvc_linear_state_scan": [P, P, L, P, L, P, L, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P],
         "kvc_sigmoid_power": [P, P, L, P, F, I, I, P],
         "kvc_decay_and_write_gates": [P, P, P, L, P, L, P, P, I, I, P],
         "kvc_unit_heads": [P, L, I, I, I, F, F, I, F, P],
-        "kvc_head_rmsnorm_gate": [P, I, P, P, L, I, P, F, I, I, I, P],
-        "kvc_moe_route": [P, P, P, I, I, I, I, I, I, P, P, I, F, P],
-        "kvc_moe_router": [P, P, P, L, I, P, P, I, I, I, I, I, I, I, P, P, I, F, P],
+        "kvc_head_rmsnorm_gate": [P, I, P, P, L, I, P, F, I, I, I, I, P],
+        "kvc_moe_route": [P, P, P, I, I, I, I, I, I, P, P, I, I, F, P],
+        "kvc_moe_router": [P, P, P, L, I, P, P, I, I, I, I, I, I, I, P, P, I, I, F, P],
         "kvc_moe_max_tiles": [I, I, I],
         "kvc_moe_tile_rows": [I, I],
         "kvc_moe_align": [P, P, P, P, I, I, I, I, P],
-        "kvc_moe_gemm": [P, L, I, P, L, P, I, P, P, P, I, I, I, I, I, I, I, F, F, F, I, P],
+        "kvc_moe_gemm": [P, L, I, P, L, P, I, P, P, P, I, I, I, I, I, I, I, F, F, F, I, P, I, P],
         "kvc_moe_combine": [P, P, P, I, P, I, P, P, I, I, I, P],
-        "kvc_qk_norm_rope_kv_write": [P, L, P, P, I, P, P, F, P, P, I, I, P, I, I, I, I, I, I, I, I, P],
+        "kvc_qk_norm_rope_kv_write": [P, L, P, P, I, P, P, F, P, P, I, I, P, I, I, I, I, I, I, I, I, I, P],
         "kvc_add_layernorm": [P, P, P, P, P, F, I, I, I, P],
         "kvc_rms_branches_mean": [P, P, P, I, F, I, I, I, P],
         "kvc_concat2": [P, P, P, I, I, I, P],
@@ -84,12 +84,12 @@ def _declare(lib: ctypes.CDLL) -> None:
         "kvc_ssm_scan": [P, P, L, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
         "kvc_gated_group_rmsnorm": [P, I, P, P, L, I, P, F, I, I, I, P],
         "kvc_decode_attention": [P, P, P, P, L, P, P, P, I, P, P, P, P, P, P, I, I, P, P, F, I, I, I, I, I, I,
-                                 I, I, F, I, P, I, P, I, I, P],
+                                 I, I, F, I, P, I, P, F, P, L, I, I, I, P],
         "kvc_decode_attention_waves": [I, I, I],
         "kvc_decode_attention_max_table": [I, I, I],
         "kvc_decode_attention_supported": [I, I, I, I, I, I],
         "kvc_prefill_attention": [P, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, I, I, F, I, P, I, P, P, P, I,
-                                  P, P, I, I, I, P],
+                                  P, P, I, I, F, P, L, I, P],
         "kvc_prefill_attention_supported": [I, I, I, I, I, I],
         "kvc_gemm_mid_slices": [I, I],
         "kvc_gemm_mid_bf16": [P, P, P, P, P, I, I, I, L, L, I, I, F, F, F, I, P],
@@ -464,13 +464,14 @@ def to_float(out: torch.Tensor, src: torch.Tensor) -> None:
 
 
 def rope_table(cos: torch.Tensor, sin: torch.Tensor, positions: torch.Tensor,
-               inv_freq: torch.Tensor) -> None:
+               inv_freq: torch.Tensor, scale: float = 1.0) -> None:
+    """``cos``/``sin [T, half]`` of the float32 angles ``positions[t] * inv_freq[j]``, times ``scale``."""
     T, half = cos.shape
     if sin.shape != (T, half) or positions.numel() < T or inv_freq.numel() != half:
         raise KernelError("rope_table: shapes do not match")
     _check(load().kvc_rope_table(_dev(cos, "cos", torch.float32), _dev(sin, "sin", torch.float32),
                                  _dev(positions, "positions", torch.int32),
-                                 _dev(inv_freq, "inv_freq", torch.float32), T, half, _stream()),
+                                 _dev(inv_freq, "inv_freq", torch.float32), float(scale), T, half, _stream()),
            "kvc_rope_table")
 
 
@@ -516,12 +517,15 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
                     *, table: torch.Tensor, positions: torch.Tensor, token_req: torch.Tensor,
                     slots: torch.Tensor, nh: int, nkv: int, d: int, scale: float,
                     window: int = 0, dv: int | None = None, slopes: torch.Tensor | None = None,
-                    chunk: int = 0, sinks: torch.Tensor | None = None) -> None:
+                    chunk: int = 0, sinks: torch.Tensor | None = None, softcap: float = 0.0,
+                    gate: torch.Tensor | None = None) -> None:
     """``q`` is a ``[T, >= nh*d]`` view whose rows hold the query heads first.  ``dv``: the size
     of a value head where it differs from a key head's ``d`` (``out`` is ``[T, nh*dv]``).
     ``slopes`` (float32 ``[nh]``): ``slopes[h] * distance`` is taken off every score of head h;
     ``chunk``: a token sees only the keys of its own chunk of that many positions.  ``sinks``
-    (float32 ``[nh]``): ``exp(sinks[h])`` joins the softmax's denominator of head h.  ``out`` has
+    (float32 ``[nh]``): ``exp(sinks[h])`` joins the softmax's denominator of head h.  ``softcap`` > 0: a
+    scaled score ``s`` becomes ``softcap * tanh(s / softcap)``.  ``gate [T, >= nh*dv]`` (the queries' dtype, a
+    column view is fine): its sigmoid multiplies the result element by element.  ``out`` has
     the queries' dtype, or is float32 beside bfloat16 queries: the weighted sums unrounded (the two
     matrix-core kernels take such an ``out`` too)."""
     if slopes is not None and (slopes.shape != (nh,) or slopes.dtype != torch.float32):
@@ -543,7 +547,7 @@ def paged_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v
         _dev(positions, "positions", torch.int32), _dev(token_req, "token_req", torch.int32),
         _dev(slots, "slots", torch.int32), T, nh, nkv, d, dv, page_size, num_pages, float(scale),
         int(window), None if slopes is None else _dev(slopes, "slopes"), int(chunk), _sinks(sinks, nh),
-        int(out.dtype == torch.float32 and q.dtype != torch.float32), _code(q, "q"), _stream()), "kvc_paged_attention")
+        float(softcap), *_gate(gate, T, nh * dv, q.dtype), int(out.dtype == torch.float32 and q.dtype != torch.float32), _code(q, "q"), _stream()), "kvc_paged_attention")
 
 
 def qk_norm_rope_kv_write(qkv: torch.Tensor, k_cache: torch.Tensor,
@@ -551,19 +555,24 @@ def qk_norm_rope_kv_write(qkv: torch.Tensor, k_cache: torch.Tensor,
                           cos: torch.Tensor, sin: torch.Tensor, *, rot_dim: int, interleaved: bool,
                           kv_slot: torch.Tensor, nh: int, nkv: int, d: int, dv: int,
                           q_gain: torch.Tensor | None = None, k_gain: torch.Tensor | None = None,
-                          eps: float = 0.0, write_kv: bool = True, queries_only: bool = False) -> None:
+                          eps: float = 0.0, write_kv: bool = True, queries_only: bool = False,
+                          values_are_keys: bool = False) -> None:
     """Rows of ``qkv`` are ``[nh heads of d | nkv heads of d | nkv heads of dv]``.  With gains
     (float32 ``[d]``, shared by all heads) every q and k head is first divided by its root mean
     square (``eps`` inside the root) and multiplied by the gain; then the first ``rot_dim``
     elements are rotated; q and k are rewritten in place, k and v stored at ``kv_slot``
     (``k_cache [pages, nkv, page_size, d]``, ``v_cache [pages, nkv, dv, page_size]``, or a list of
     up to four planes ``[pages, nkv, dv / n, page_size]`` that each hold a slice of every value
-    head).  ``queries_only``: the rows hold the query heads alone and nothing is stored."""
+    head).  ``queries_only``: the rows hold the query heads alone and nothing is stored.
+    ``values_are_keys``: the rows hold no values; the k heads as they are become the values, and their
+    columns are left unchanged."""
     T = qkv.shape[0]
     row_kv = 0 if queries_only else nkv
+    if values_are_keys and (queries_only or dv != d):
+        raise KernelError("qk_norm_rope_kv_write: values that are the keys have the keys' size")
     if queries_only and write_kv:
         raise KernelError("qk_norm_rope_kv_write: rows of queries alone have nothing to store")
-    if qkv.dim() != 2 or qkv.stride(1) != 1 or qkv.shape[1] < (nh + row_kv) * d + row_kv * dv:
+    if qkv.dim() != 2 or qkv.stride(1) != 1 or qkv.shape[1] < (nh + row_kv) * d + (0 if values_are_keys else row_kv * dv):
         raise KernelError(f"qk_norm_rope_kv_write: qkv shape {tuple(qkv.shape)} does not fit the heads")
     planes = list(v_cache) if isinstance(v_cache, (list, tuple)) else [v_cache]
     if not 1 <= len(planes) <= 4 or dv % len(planes):
@@ -588,7 +597,7 @@ def qk_norm_rope_kv_write(qkv: torch.Tensor, k_cache: torch.Tensor,
         None if q_gain is None else _dev(q_gain, "q_gain"), None if k_gain is None else _dev(k_gain, "k_gain"),
         float(eps), _dev(cos, "cos", torch.float32), _dev(sin, "sin", torch.float32), int(rot_dim),
         int(bool(interleaved)), _dev(kv_slot, "kv_slot", torch.int32), T, nh, row_kv, d, dv, page_size,
-        int(write_kv), _code(qkv, "qkv"), _stream()), "kvc_qk_norm_rope_kv_write")
+        int(write_kv), int(bool(values_are_keys)), _code(qkv, "qkv"), _stream()), "kvc_qk_norm_rope_kv_write")
 
 
 def _slopes(slopes: torch.Tensor | None, nh: int) -> int | None:
@@ -607,6 +616,21 @@ def _sinks(sinks: torch.Tensor | None, nh: int) -> int | None:
     if sinks.shape != (nh,):
         raise KernelError("attention: a sink per query head")
     return _dev(sinks, "sinks", torch.float32)
+
+
+def _gate(gate: torch.Tensor | None, T: int, width: int, dtype: torch.dtype) -> tuple[int | None, int]:
+    """(pointer, row stride) of the rows whose sigmoid gates an attention's result, or (None, 0)."""
+    if gate is None:
+        return None, 0
+    if gate.dim() != 2 or gate.shape[0] < T or gate.shape[1] < width or gate.stride(1) != 1 or gate.dtype != dtype \
+            or not gate.is_cuda:
+        raise KernelError(f"attention: the gate's rows must be {dtype} GPU rows of {width} values")
+    return gate.data_ptr(), gate.stride(0)
+
+
+def attention_gate_ok(gate: torch.Tensor) -> bool:
+    """Whether every attention kernel can take these gate rows (the one for portions reads 8 bytes at a time)."""
+    return gate.stride(0) % 4 == 0 and gate.data_ptr() % 8 == 0
 
 
 def decode_attention_supported(nh: int, nkv: int, d: int, page_size: int, dtype: torch.dtype,
@@ -698,7 +722,8 @@ def decode_attention(out: torch.Tensor, qkv: torch.Tensor, k_cache: torch.Tensor
                      slopes: torch.Tensor | None = None, chunk: int = 0,
                      sinks: torch.Tensor | None = None, dv: int | None = None,
                      q_gain: torch.Tensor | None = None, k_gain: torch.Tensor | None = None,
-                     eps: float = 0.0) -> None:
+                     eps: float = 0.0, softcap: float = 0.0, gate: torch.Tensor | None = None,
+                     values_are_keys: bool = False) -> None:
     """bfloat16 attention of single tokens on the matrix cores (see the C header), with the
     rotation of each token's query and key and the write of its key and value into the cache
     (``write_kv``) in the same kernel; ``qkv`` is not changed.  With ``rot_dim = 0`` and
@@ -708,12 +733,15 @@ def decode_attention(out: torch.Tensor, qkv: torch.Tensor, k_cache: torch.Tensor
     elements when ``nsplit > 1``.  ``dv``: the size of a value head, ``d`` (the default) or half of
     it.  ``q_gain`` and ``k_gain`` (float32 ``[d]``): every query head, and the key head that is
     written, is divided by its root mean square (``eps`` inside the root) and multiplied by the
-    gain before the rotation."""
+    gain before the rotation.  ``softcap`` and ``gate`` as for :func:`paged_attention`.
+    ``values_are_keys``: the rows of ``qkv`` hold no values; the keys as they are become the values."""
     T = out.shape[0]
     dv = d if dv is None else dv
     if out.shape != (T, nh * dv) or not out.is_contiguous() or out.dtype not in (torch.bfloat16, torch.float32):
         raise KernelError("decode_attention: out must be contiguous bfloat16 (or float32) [T, nh*dv]")
-    need = (nh + nkv) * d + nkv * dv if write_kv else nh * d
+    if values_are_keys and dv != d:
+        raise KernelError("decode_attention: values that are the keys have the keys' size")
+    need = (nh + nkv) * d + (0 if values_are_keys else nkv * dv) if write_kv else nh * d
     for gain in (q_gain, k_gain):
         if gain is not None and gain.shape != (d,):
             raise KernelError("decode_attention: a gain must be float32 [d]")
@@ -746,7 +774,8 @@ def decode_attention(out: torch.Tensor, qkv: torch.Tensor, k_cache: torch.Tensor
         None if q_gain is None else _dev(q_gain, "q_gain", torch.float32),
         None if k_gain is None else _dev(k_gain, "k_gain", torch.float32), float(eps),
         int(bool(write_kv)), T, nh, nkv, d, dv, page_size, num_pages, float(scale),
-        int(window), _slopes(slopes, nh), int(chunk), _sinks(sinks, nh), int(nsplit),
+        int(window), _slopes(slopes, nh), int(chunk), _sinks(sinks, nh), float(softcap),
+        *_gate(gate, T, nh * dv, torch.bfloat16), int(bool(values_are_keys)), int(nsplit),
         int(out.dtype == torch.float32), _stream()),
         "kvc_decode_attention")
 
@@ -764,11 +793,13 @@ def prefill_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
                       part_ml: torch.Tensor | None = None, cos: torch.Tensor | None = None,
                       sin: torch.Tensor | None = None, rot_dim: int = 0, interleaved: bool = False,
                       slopes: torch.Tensor | None = None, chunk: int = 0,
-                      sinks: torch.Tensor | None = None, dv: int | None = None) -> None:
+                      sinks: torch.Tensor | None = None, dv: int | None = None, softcap: float = 0.0,
+                      gate: torch.Tensor | None = None) -> None:
     """bfloat16 attention of portions of prompts on the matrix cores (see the C header).
     ``nsplit > 1`` deals every tile's keys to that many blocks; ``part_o`` (float32,
     ``T*nh*nsplit*dv`` values) and ``part_ml`` (``T*nh*nsplit*2``) are then the workspace.
-    ``dv``: the size of a value head, ``d`` (the default) or half of it.
+    ``dv``: the size of a value head, ``d`` (the default) or half of it.  ``softcap`` and ``gate`` as for
+    :func:`paged_attention` (the gate's rows 8-byte aligned).
     With ``cos`` and ``sin`` (``[T, rot_dim / 2]`` float32) the queries come unrotated and
     the kernel rotates them (``prefill_attention_rotates`` says for which shapes)."""
     T = out.shape[0]
@@ -800,7 +831,7 @@ def prefill_attention(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor,
         _dev(q_start, "q_start", torch.int32), _dev(slots, "slots", torch.int32), T, num_reqs,
         nh, nkv, d, dv, page_size, num_pages, float(scale), int(window), _slopes(slopes, nh), int(chunk),
         _sinks(sinks, nh), po, pml, int(nsplit), cs, sn, int(rot_dim) if cs is not None else 0, int(interleaved),
-        int(out.dtype == torch.float32), _stream()),
+        float(softcap), *_gate(gate, T, nh * dv, torch.bfloat16), int(out.dtype == torch.float32), _stream()),
         "kvc_prefill_attention")
 
 
@@ -971,18 +1002,19 @@ class SlicedRows:
 @dataclass
 class WeightedRows:
     """The results of a token's experts, not yet added up: ``data [>= T * n, H]`` float32 (token t's ``n``
-    rows one after the other), ``weight [T, n]``; row t is ``sum_c weight[t, c] * data[t * n + c]``, plus
-    ``add[t]`` (float32, or None) times ``add_gate[t]`` (``[T, 1]``, or None: once).  ``norm_add_norm`` takes
-    it in place of the summed rows (``moe_combine`` makes those)."""
+    rows one after the other), ``weight [T, n]``, or None (all ones) with ``count`` n; row t is ``sum_c
+    weight[t, c] * data[t * n + c]``, plus ``add[t]`` (float32, or None) times ``add_gate[t]`` (``[T, 1]``, or
+    None: once).  ``norm_add_norm`` takes it in place of the summed rows (``moe_combine`` makes those)."""
 
     data: torch.Tensor
-    weight: torch.Tensor
+    weight: torch.Tensor | None
     add: torch.Tensor | None = None
     add_gate: torch.Tensor | None = None
+    count: int = 0
 
     def check(self, T: int, H: int) -> int:
-        n = self.weight.shape[1]
-        if self.weight.shape[0] != T or n < 1 or self.data.shape[1] != H or self.data.shape[0] < T * n \
+        n = self.weight.shape[1] if self.weight is not None else self.count
+        if (self.weight is not None and self.weight.shape[0] != T) or n < 1 or self.data.shape[1] != H or self.data.shape[0] < T * n \
                 or (self.add is not None and self.add.shape != (T, H)) \
                 or (self.add_gate is not None and (self.add is None or self.add_gate.numel() != T)):
             raise KernelError("weighted rows do not fit")
@@ -1558,11 +1590,12 @@ def linear_state_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: to
                       positions: torch.Tensor, token_req: torch.Tensor, q_start: torch.Tensor,
                       slots: torch.Tensor, num_reqs: int, heads: int, qk_heads: int, dim: int,
                       vdim: int, delta_rule: bool = False, q_scale: float = 1.0,
-                      scalar_gates: bool = False, ones_column: bool = False) -> None:
+                      scalar_gates: bool = False, ones_column: bool = False, silu_in: bool = False) -> None:
     """The recurrence of a matrix state per head (see the C header): ``q, k [T, qk_heads * dim]``,
     ``v [T, heads * vdim]``, all float32 rows (column views are fine); ``decay [T, heads * dim]``
     (a factor per key channel) or, with ``delta_rule``, ``decay`` and ``beta [T, heads]``; with
-    ``scalar_gates`` the rule is ``S <- decay S + beta k v^T`` with the same two ``[T, heads]``;
+    ``scalar_gates`` the rule is ``S <- decay S + beta k v^T`` with the same two ``[T, heads]`` (``beta`` None:
+    ones; ``decay [1, heads]``: the same for every token); ``silu_in``: q, k and v pass through silu first;
     with ``ones_column`` ``v`` is ``[T, heads * (vdim - 1)]`` and the last of a head's ``vdim``
     columns takes a one for every token (a normaliser beside the matrix);
     ``state [slots, heads, linear_state_rows(dim), vdim]`` float32, in an order of the kernel's own;
@@ -1574,7 +1607,8 @@ def linear_state_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: to
     if tuple(state.shape[1:]) != (heads, linear_state_rows(dim), vdim) or state.dtype != torch.float32 \
             or not state.is_contiguous():
         raise KernelError("linear_state_scan: state must be float32 [slots, heads, linear_state_rows(dim), vdim]")
-    if min(q.shape[0], k.shape[0], v.shape[0], decay.shape[0]) < T or positions.numel() < T \
+    fixed = scalar_gates and decay.shape[0] == 1
+    if min(q.shape[0], k.shape[0], v.shape[0], T if fixed else decay.shape[0]) < T or positions.numel() < T \
             or token_req.numel() < T or q_start.numel() < num_reqs + 1:
         raise KernelError("linear_state_scan: rows or index arrays too short")
     qp, qs = _f32_rows(q, "q", qk_heads * dim)
@@ -1584,8 +1618,10 @@ def linear_state_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: to
         raise KernelError("linear_state_scan: one rule at a time")
     per_head = delta_rule or scalar_gates
     dp, ds = _f32_rows(decay, "decay", heads if per_head else heads * dim)
+    if fixed:
+        ds = 0
     bp, bs = (0, 0)
-    if per_head:
+    if per_head and not (scalar_gates and beta is None):
         if beta is None or beta.shape[0] < T:
             raise KernelError("linear_state_scan: this rule needs beta")
         bp, bs = _f32_rows(beta, "beta", heads)
@@ -1594,7 +1630,7 @@ def linear_state_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: to
         _dev(positions, "positions", torch.int32), _dev(token_req, "token_req", torch.int32),
         _dev(q_start, "q_start", torch.int32), _dev(slots, "slots", torch.int32), num_reqs, heads,
         qk_heads, dim, vdim, 2 if scalar_gates else int(bool(delta_rule)), float(q_scale), int(bool(ones_column)),
-        _stream()),
+        int(bool(silu_in)), _stream()),
         "kvc_linear_state_scan")
 
 
@@ -1633,8 +1669,8 @@ def unit_heads(x: torch.Tensor, heads: int, dim: int, eps: float, scale: float =
 
 
 def head_rmsnorm_gate(out: torch.Tensor, o: torch.Tensor, gate: torch.Tensor, gain: torch.Tensor, eps: float,
-                      heads: int, vdim: int) -> None:
-    """``out = o / rms_head(o) * gain * silu(gate)``: every head of ``vdim`` values of the float32
+                      heads: int, vdim: int, act: str = "silu") -> None:
+    """``out = o / rms_head(o) * gain * act(gate)`` (``act``: ``silu`` or ``sigmoid``): every head of ``vdim`` values of the float32
     ``o [T, heads * vdim]`` over its root mean square, times ``gain [vdim]`` (shared by the heads),
     times the gate (rows of any dtype, a column view is fine)."""
     T = o.shape[0]
@@ -1643,7 +1679,8 @@ def head_rmsnorm_gate(out: torch.Tensor, o: torch.Tensor, gate: torch.Tensor, ga
         raise KernelError("head_rmsnorm_gate: shapes do not match")
     gp, gs, gc = _rows(gate, "gate", heads * vdim)
     _check(load().kvc_head_rmsnorm_gate(_dev(out, "out"), _code(out, "out"), _dev(o, "o", torch.float32), gp, gs, gc,
-                                        _dev(gain, "gain", torch.float32), float(eps), T, heads, vdim, _stream()),
+                                        _dev(gain, "gain", torch.float32), float(eps), T, heads, vdim,
+                                        {"silu": 0, "sigmoid": 1}[act], _stream()),
            "kvc_head_rmsnorm_gate")
 
 
@@ -1694,14 +1731,16 @@ def norm_add_norm(out: torch.Tensor | None, residual: torch.Tensor, delta: "torc
                   post_gain: torch.Tensor, eps: float, next_gain: torch.Tensor | None = None,
                   next_eps: float | None = None) -> None:
     """``residual += post_gain * delta / rms(delta)``, then, given ``out``, ``out = next_gain *
-    residual / rms(residual)``: the norm behind a sublayer, the sum into the float32 stream and the
-    norm before the next sublayer in one pass (both roots hold their eps).  ``delta`` is float32
+    residual / rms(residual)``, or, without ``next_gain``, ``out = residual`` rounded: the norm behind a
+    sublayer, the sum into the float32 stream and what the next sublayer reads of it in one pass (both roots
+    hold their eps).  ``delta`` is float32
     or bfloat16, or the :class:`SlicedRows` that a product left (their sum is the result), or the
     :class:`WeightedRows` of a feed-forward of routed experts."""
     T, H = residual.shape
     slices = 1
+    by_token = isinstance(delta, WeightedRows)
     weight = add = add_gate = None
-    if isinstance(delta, WeightedRows):
+    if by_token:
         slices = delta.check(T, H)
         weight, add, add_gate, delta = delta.weight, delta.add, delta.add_gate, delta.data
     elif isinstance(delta, SlicedRows):
@@ -1715,15 +1754,15 @@ def norm_add_norm(out: torch.Tensor | None, residual: torch.Tensor, delta: "torc
         raise KernelError("norm_add_norm: shapes do not match")
     if not residual.is_contiguous() or post_gain.shape != (H,):
         raise KernelError("norm_add_norm: shapes do not match")
-    if out is not None and (out.shape != (T, H) or not out.is_contiguous() or next_gain is None
-                            or next_gain.shape != (H,)):
+    if out is not None and (out.shape != (T, H) or not out.is_contiguous()
+                            or (next_gain is not None and next_gain.shape != (H,))):
         raise KernelError("norm_add_norm: the second norm's rows or gain do not fit")
     _check(load().kvc_norm_add_norm(
         None if out is None else _dev(out, "out"), 0 if out is None else _code(out, "out"),
         _dev(residual, "residual", torch.float32), _dev(delta, "delta"), _code(delta, "delta"),
         _dev(post_gain, "post_gain", torch.float32), float(eps),
-        None if out is None else _dev(next_gain, "next_gain", torch.float32),
-        float(eps if next_eps is None else next_eps), T, H, slices,
+        None if out is None or next_gain is None else _dev(next_gain, "next_gain", torch.float32),
+        float(eps if next_eps is None else next_eps), T, H, slices, int(by_token),
         *(None if t is None else _dev(t, "a weight", torch.float32) for t in (weight, add, add_gate)), _stream()),
         "kvc_norm_add_norm")
 
@@ -1788,7 +1827,7 @@ ROUTE_SCORES = {"softmax": 0, "sigmoid": 1, "logit": 2}
 
 
 def _route_rule(E: int, score: str, bias: torch.Tensor | None, correction: torch.Tensor | None, group_best: int,
-                weight_scale: float) -> tuple[int, int | None, int | None, int, float]:
+                weight_scale: float, renormalize: bool) -> tuple[int, int | None, int | None, int, int, float]:
     if score not in ROUTE_SCORES:
         raise KernelError(f"unknown router score {score!r} (known: {sorted(ROUTE_SCORES)})")
     for t, what in ((bias, "bias"), (correction, "correction")):
@@ -1797,31 +1836,32 @@ def _route_rule(E: int, score: str, bias: torch.Tensor | None, correction: torch
     if group_best not in (1, 2):
         raise KernelError("moe routing: a group is worth its best choice score or the sum of its best two")
     return (ROUTE_SCORES[score], None if bias is None else _dev(bias, "bias"),
-            None if correction is None else _dev(correction, "correction"), int(group_best), float(weight_scale))
+            None if correction is None else _dev(correction, "correction"), int(group_best), int(bool(renormalize)),
+            float(weight_scale))
 
 
 def moe_route(choice: torch.Tensor, weight: torch.Tensor, logits: torch.Tensor, *, top: int, groups: int = 1,
               keep: int = 1, score: str = "softmax", correction: torch.Tensor | None = None, group_best: int = 1,
-              weight_scale: float = 1.0, bias: torch.Tensor | None = None) -> None:
+              weight_scale: float = 1.0, bias: torch.Tensor | None = None, renormalize: bool = True) -> None:
     """The router's choice from float32 ``logits [T, E]``: ``choice`` (int32) and ``weight``
     (float32), both ``[T, top]``.  ``bias`` (float32 ``[E]``) joins the logits.  ``score``: ``softmax`` over the
     experts, a ``sigmoid`` of each logit, or the ``logit`` itself (the weights are then the softmax over the
     chosen logits); ``correction`` (float32 ``[E]``) joins the scores for the choice alone; a group is worth
     its ``group_best`` (1 or 2) best choice scores; the weights (the chosen experts' plain scores
-    over their sum) are multiplied by ``weight_scale``."""
+    over their sum, or, without ``renormalize``, as they are) are multiplied by ``weight_scale``."""
     T, E = logits.shape
     if choice.shape != (T, top) or weight.shape != (T, top):
         raise KernelError("moe_route: shapes do not match")
     _check(load().kvc_moe_route(_dev(choice, "choice", torch.int32), _dev(weight, "weight", torch.float32),
                                 _dev(logits, "logits", torch.float32), T, E, top, groups, keep,
-                                *_route_rule(E, score, bias, correction, group_best, weight_scale), _stream()),
+                                *_route_rule(E, score, bias, correction, group_best, weight_scale, renormalize), _stream()),
            "kvc_moe_route")
 
 
 def moe_router(choice: torch.Tensor, weight: torch.Tensor, x: torch.Tensor, router: torch.Tensor, *, top: int,
                groups: int = 1, keep: int = 1, score: str = "softmax", correction: torch.Tensor | None = None,
                group_best: int = 1, weight_scale: float = 1.0, bias: torch.Tensor | None = None,
-               gate: torch.Tensor | None = None) -> None:
+               gate: torch.Tensor | None = None, renormalize: bool = True) -> None:
     """``moe_route`` of the logits ``x @ router.T`` (float32 sums in one fixed order; ``x [T, H]`` of
     either dtype, ``router [E, H]`` float32) without storing the logits.  With ``gate`` (float32, a
     value a token) the router has one row more, and ``gate[t] = sigmoid(x[t] . that row)``."""
@@ -1834,7 +1874,7 @@ def moe_router(choice: torch.Tensor, weight: torch.Tensor, x: torch.Tensor, rout
     _check(load().kvc_moe_router(_dev(choice, "choice", torch.int32), _dev(weight, "weight", torch.float32),
                                  x.data_ptr(), x.stride(0), _code(x, "x"), _dev(router, "router", torch.float32),
                                  None if gate is None else _dev(gate, "gate", torch.float32), T, H, E, top, groups, keep,
-                                 *_route_rule(E, score, bias, correction, group_best, weight_scale), _stream()),
+                                 *_route_rule(E, score, bias, correction, group_best, weight_scale, renormalize), _stream()),
            "kvc_moe_router")
 
 
@@ -1865,15 +1905,22 @@ def moe_align(sorted_pairs: torch.Tensor, tiles: torch.Tensor, num_tiles: torch.
 
 def moe_gemm(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, sorted_pairs: torch.Tensor, tiles: torch.Tensor,
              num_tiles: torch.Tensor, *, pairs: int, experts: int, in_div: int, out_sorted: bool, gated: bool,
-             limit: float = 0.0, alpha: float = 0.0, up_shift: float = 1.0, tile_rows: int = 16) -> None:
+             limit: float = 0.0, alpha: float = 0.0, up_shift: float = 1.0, tile_rows: int = 16,
+             act: str | None = None, row_scale: torch.Tensor | None = None) -> None:
     """Every expert's product over its own rows.  ``w`` is ``[experts * N, K]`` (``experts * 2N``
     rows when ``gated``: each expert's gate rows, then its up rows); ``out [pairs, N]``.  The gated
-    form stores ``min(g, limit) * sigmoid(alpha * g) * (clamp(u, -limit, limit) + up_shift)``."""
+    form stores ``min(g, limit) * sigmoid(alpha * g) * (clamp(u, -limit, limit) + up_shift)``; without a gate
+    ``act`` may name one of :data:`ACTIVATIONS`.  ``row_scale`` (float32, a value a pair) multiplies a pair's
+    input: its sums, before any activation."""
     N = out.shape[1]
     K = x.shape[1]
     rows = experts * N * (2 if gated else 1)
     if w.shape != (rows, K) or out.shape[0] < pairs or x.dtype != w.dtype or out.stride(1) != 1 or x.stride(1) != 1:
         raise KernelError("moe_gemm: shapes do not match")
+    if act is not None and (gated or act not in ACTIVATIONS):
+        raise KernelError(f"moe_gemm: activation {act!r} of a product without a gate (known: {sorted(ACTIVATIONS)})")
+    if row_scale is not None and row_scale.numel() < pairs:
+        raise KernelError("moe_gemm: a scale a pair")
     max_tiles = min(tiles.shape[0], moe_max_tiles(pairs, experts, tile_rows))
     # the bfloat16 kernels read the packed twin of the experts' matrix where the model keeps one
     w_ptr, packed = (_streamed(w, N) if N % 16 == 0 and K % 64 == 0 else (_dev(w, "w"), 0))
@@ -1881,16 +1928,19 @@ def moe_gemm(out: torch.Tensor, x: torch.Tensor, w: torch.Tensor, sorted_pairs: 
                                w_ptr, _code(x, "x"), _dev(sorted_pairs, "sorted", torch.int32),
                                _dev(tiles, "tiles", torch.int32), _dev(num_tiles, "num_tiles", torch.int32),
                                max_tiles, tile_rows, N, K, int(in_div), int(bool(out_sorted)), int(bool(gated)),
-                               float(limit), float(alpha), float(up_shift), packed, _stream()), "kvc_moe_gemm")
+                               float(limit), float(alpha), float(up_shift), -1 if act is None else ACTIVATIONS[act],
+                               None if row_scale is None else _dev(row_scale, "row_scale", torch.float32), packed,
+                               _stream()), "kvc_moe_gemm")
 
 
-def moe_combine(out: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, add0: torch.Tensor | None = None,
+def moe_combine(out: torch.Tensor, y: torch.Tensor, weight: torch.Tensor | None, add0: torch.Tensor | None = None,
                 add1: torch.Tensor | None = None, accumulate: bool = False,
-                add1_gate: torch.Tensor | None = None) -> None:
+                add1_gate: torch.Tensor | None = None, count: int = 0) -> None:
     """``out[t] = sum_c weight[t, c] * y[t * top + c] (+ add0[t]) (+ add1[t])``, float32; ``add0``
-    of either dtype, ``add1`` float32, times ``add1_gate`` (a value a token) if given.  ``accumulate``: the sum is added into ``out``."""
+    of either dtype, ``add1`` float32, times ``add1_gate`` (a value a token) if given.  ``accumulate``: the sum is
+    added into ``out``.  ``weight`` None: ``count`` rows a token, each once."""
     T, H = out.shape
-    top = weight.shape[1] if weight.dim() == 2 else 0
+    top = count if weight is None else weight.shape[1] if weight.dim() == 2 else 0
     if out.dtype != torch.float32 or (top and (y.shape[0] < T * top or y.shape[1] != H)):
         raise KernelError("moe_combine: shapes do not match")
     for a in (add0, add1):
@@ -1898,8 +1948,8 @@ def moe_combine(out: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, add0: 
             raise KernelError("moe_combine: an added row set does not fit")
     if add1_gate is not None and (add1 is None or add1_gate.numel() != T):
         raise KernelError("moe_combine: a gate value a token, for the second added row set")
-    _check(load().kvc_moe_combine(_dev(out, "out"), _dev(y, "y", torch.float32), _dev(weight, "weight", torch.float32),
-                                  top, None if add0 is None else _dev(add0, "add0"),
+    _check(load().kvc_moe_combine(_dev(out, "out"), _dev(y, "y", torch.float32),
+                                  None if weight is None else _dev(weight, "weight", torch.float32), top, None if add0 is None else _dev(add0, "add0"),
                                   0 if add0 is None else _code(add0, "add0"),
                                   None if add1 is None else _dev(add1, "add1", torch.float32),
                                   None if add1_gate is None else _dev(add1_gate, "add1_gate", torch.float32), T, H,

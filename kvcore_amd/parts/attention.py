@@ -118,7 +118,8 @@ class PagedAttention(Mixer):
                  qk_norm_gain: bool = True, distance_slopes: tuple[float, ...] | None = None,
                  chunk: int = 0, qk_norm_span: str = "head", values_are_keys: bool = False,
                  sinks: bool | float = False, sized_buffers: bool = False, o_bias: bool | None = None,
-                 own_kv: bool = True, position: PositionEncoding | None = None) -> None:
+                 own_kv: bool = True, softcap: float = 0.0, output_gate: bool = False,
+                 position: PositionEncoding | None = None) -> None:
         """``v_head_dim``: the size of a value head where it differs from ``head_dim``, the
         size of a query and key head.  ``qk_norm_eps`` (None: no such norm): every query and
         key head is divided by its root mean square, eps inside the root, and multiplied by a
@@ -138,7 +139,10 @@ class PagedAttention(Mixer):
         instead is that score for every head, and there is no tensor.  ``o_bias`` None: the output
         product has a bias iff the others do (``bias``).  ``own_kv`` False: the layer has no
         projections of keys and values and reads the cache that another layer with the same head
-        counts and sizes has written (its schedule entry says ``cache_from``).
+        counts and sizes has written (its schedule entry says ``cache_from``).  ``softcap`` > 0: a scaled
+        score ``s`` becomes ``softcap * tanh(s / softcap)`` before the softmax.  ``output_gate``: the heads'
+        results, side by side, are multiplied element by element by ``sigmoid(W_g h)`` before the output
+        product (tensor ``g``, no bias; its rows are part of the one input product).
         ``sized_buffers``: name the step buffers by their width, for a model whose attention layers
         differ in size."""
         if qk_norm_span not in ("head", "projection"):
@@ -149,14 +153,16 @@ class PagedAttention(Mixer):
             raise ValueError("values that are the keys have the keys' size")
         if not own_kv and (values_are_keys or qk_norm_span == "projection"):
             raise ValueError("a layer that reads another's cache projects queries alone, normed head by head")
+        if softcap < 0 or (softcap and distance_slopes is not None):
+            raise ValueError("a soft cap is positive and does not go with distance slopes")
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} kv heads")
         v_head_dim = head_dim if v_head_dim is None else v_head_dim
         self.head_norm = qk_norm_eps is not None and qk_norm_span == "head"
         self.wide_norm = qk_norm_eps is not None and qk_norm_span == "projection"
         plain = v_head_dim == head_dim and not self.head_norm
-        if not own_kv:
-            plain = False  # rows of queries alone
+        if not own_kv or output_gate:
+            plain = False  # rows of queries alone, or rows with a gate behind the heads
         elif plain and (head_dim % 16 or head_dim > 256):
             if qk_norm_eps is None and not values_are_keys and not self.any_head_size:
                 raise ValueError(f"head size {head_dim} is not supported (multiples of 16 up to 256)")
@@ -174,6 +180,10 @@ class PagedAttention(Mixer):
         self.has_sinks = sinks is True  # a learned score a head
         self.fixed_sink = float(sinks) if not isinstance(sinks, bool) else None  # the same for every head
         self.own_kv = bool(own_kv)
+        self.softcap, self.output_gate = float(softcap), bool(output_gate)
+        # values that are the keys before a norm of every head are read from the keys' own columns: the
+        # rows hold no values then (elsewhere the keys are copied behind themselves)
+        self.keys_serve_as_values = self.values_are_keys and self.head_norm
         if distance_slopes is not None and len(distance_slopes) != num_heads:
             raise ValueError(f"{len(distance_slopes)} distance slopes for {num_heads} heads")
         if chunk < 0:
@@ -191,8 +201,9 @@ class PagedAttention(Mixer):
         self.kv_size = num_kv_heads * head_dim
         self.v_size = num_kv_heads * v_head_dim
         self.o_size = num_heads * v_head_dim
-        # the width of a projected row
-        self.row_size = self.q_size + (self.kv_size + self.v_size if own_kv else 0)
+        # the width of a projected row, and where the gate stands in it
+        self.gate_at = self.q_size + (self.kv_size + (0 if self.keys_serve_as_values else self.v_size) if own_kv else 0)
+        self.row_size = self.gate_at + (self.o_size if self.output_gate else 0)
         self.plain = plain
         # layers that are all alike share one step buffer a role; others name theirs by width
         self.shared_buffers = plain and not sized_buffers and not self.any_head_size
@@ -204,14 +215,18 @@ class PagedAttention(Mixer):
         self.names = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight",
                       "o": "o_proj.weight", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight",
                       "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias",
-                      "o_bias": "o_proj.bias", "sink": "sinks", **(tensor_names or {})}
+                      "o_bias": "o_proj.bias", "sink": "sinks", "g": "g_proj.weight", **(tensor_names or {})}
+
+    @property
+    def heads_rows(self) -> int:
+        """Rows of the input product that project heads (what follows are the gate's)."""
+        if not self.own_kv:
+            return self.q_size
+        return self.q_size + self.kv_size + (0 if self.values_are_keys else self.v_size)
 
     def param_specs(self) -> list[ParamSpec]:
-        total = self.row_size
         n = self.names
-
-        if self.values_are_keys:  # no value projection: q and k alone
-            total = self.q_size + self.kv_size
+        total = self.heads_rows + (self.o_size if self.output_gate else 0)
 
         def stacked(q: str, k: str, v: str) -> tuple[ParamSource, ...]:
             if not self.own_kv:
@@ -221,8 +236,9 @@ class PagedAttention(Mixer):
                 return qk
             return (*qk, ParamSource(n[v], self.q_size + self.kv_size, self.v_size))
 
+        gate = (ParamSource(n["g"], self.heads_rows, self.o_size),) if self.output_gate else ()
         specs = [
-            ParamSpec("qkv_proj.weight", (total, self.hidden_size), sources=stacked("q", "k", "v")),
+            ParamSpec("qkv_proj.weight", (total, self.hidden_size), sources=(*stacked("q", "k", "v"), *gate)),
             ParamSpec("o_proj.weight", (self.hidden_size, self.o_size),
                       sources=(ParamSource(n["o"], 0, self.hidden_size),)),
         ]
@@ -251,6 +267,11 @@ class PagedAttention(Mixer):
             self._slopes = torch.tensor(self.distance_slopes, dtype=torch.float32, device=runtime.device)
         if self.head_norm and not self.qk_norm_gain:
             self._unit_gain = torch.ones(self.head_dim, dtype=torch.float32, device=runtime.device)
+
+    def weights_loaded(self) -> None:
+        super().weights_loaded()
+        if self.output_gate and self.bias:  # the gate has no bias
+            self.params["qkv_proj.bias"][self.heads_rows:].zero_()
 
     def cache_need(self) -> CacheNeed:
         values = ((self.num_kv_heads, self.v_plane_dim),) * self.v_planes
@@ -299,10 +320,14 @@ class PagedAttention(Mixer):
         p = self.params
         # step buffers are named by their width: layers of one model may differ in size
         qkv = ctx.buf(_sized("attn_qkv", self.row_size, self.shared_buffers), self.row_size)
-        if self.values_are_keys:
-            ops.linear(qkv[:, : self.q_size + self.kv_size], x, p["qkv_proj.weight"], p.get("qkv_proj.bias"))
+        if self.values_are_keys and not self.keys_serve_as_values:
+            n, bias = self.heads_rows, p.get("qkv_proj.bias")
+            ops.linear(qkv[:, :n], x, p["qkv_proj.weight"][:n] if self.output_gate else p["qkv_proj.weight"],
+                       bias if bias is None else bias[:n])
+            if self.output_gate:
+                ops.linear(qkv[:, self.gate_at:], x, p["qkv_proj.weight"][n:])
             if not self.wide_norm:  # the values are the keys as projected
-                qkv[:, self.q_size + self.kv_size:].copy_(qkv[:, self.q_size: self.q_size + self.kv_size])
+                qkv[:, self.q_size + self.kv_size: self.gate_at].copy_(qkv[:, self.q_size: self.q_size + self.kv_size])
         else:
             ops.linear(qkv, x, p["qkv_proj.weight"], p.get("qkv_proj.bias"))
         if self.wide_norm:
@@ -346,12 +371,15 @@ class PagedAttention(Mixer):
                                       nkv=self.num_kv_heads, d=self.head_dim, dv=self.v_head_dim,
                                       q_gain=q_gain, k_gain=k_gain if self.own_kv else q_gain,
                                       eps=self.qk_norm_eps or 0.0, write_kv=call.write_cache and self.own_kv,
-                                      queries_only=not self.own_kv)
+                                      queries_only=not self.own_kv, values_are_keys=self.keys_serve_as_values)
             rot_dim, interleaved = 0, False
             cos = sin = ctx.buffers.get("rope_none", ctx.num_tokens, 0, torch.float32)
+        # the attention kernels gate their results on the way out where they see whole heads
+        gate = qkv[:, self.gate_at: self.gate_at + self.o_size] if self.output_gate else None
+        gate_inside = gate is not None and self.v_planes == 1 and ops.attention_gate_ok(gate)
         if self.v_planes == 1:
             self._attend(attn, qkv, k_cache, v_planes[0], ctx, call, group, cos, sin, rot_dim, interleaved, prepared,
-                         q_gain, k_gain)
+                         q_gain, k_gain, gate if gate_inside else None)
         else:
             # the same scores against each plane of the values; the planes' results, each [T, heads
             # * plane size], are then laid side by side within every head
@@ -363,6 +391,8 @@ class PagedAttention(Mixer):
                              rot_dim, interleaved, prepared, q_gain, k_gain)
             attn.view(T, self.num_heads, m, self.v_plane_dim).copy_(
                 parts.view(m, T, self.num_heads, self.v_plane_dim).permute(1, 2, 0, 3))
+        if gate is not None and not gate_inside:
+            ops.head_gate(attn, attn, gate, heads=self.o_size, head_stride=1, skip=0, n=1)
         return attn
 
     def _output(self, attn, ctx, sink=None):
@@ -377,7 +407,7 @@ class PagedAttention(Mixer):
         return out
 
     def _attend(self, attn, qkv, k_cache, v_cache, ctx, call, group, cos, sin, rot_dim, interleaved, prepared,
-                q_gain=None, k_gain=None):
+                q_gain=None, k_gain=None, gate=None):
         """The attention itself into ``attn [T, heads * plane size]`` over one plane of values,
         by the kernel that serves the step's shape.  ``prepared``: q is ready and the cache is
         written; otherwise the kernels chosen here rotate and write on their way."""
@@ -387,7 +417,7 @@ class PagedAttention(Mixer):
         x_dtype = qkv.dtype
         # a distance bias and a chunked view are options of every attention kernel
         sinks = self.params.get("sinks", self._sinks)
-        common.update(slopes=self._slopes, chunk=self.chunk, sinks=sinks)
+        common.update(slopes=self._slopes, chunk=self.chunk, sinks=sinks, softcap=self.softcap, gate=gate)
         # a token never sees more keys than its window or its chunk holds: what the launch plans count
         reach = min((n for n in (self.window, self.chunk) if n > 0), default=0)
         if ctx.max_query_len == 1 and self._decode_kernel(group.page_size, x_dtype):
@@ -410,7 +440,7 @@ class PagedAttention(Mixer):
             ops.decode_attention(attn, qkv, k_cache, v_cache, nsplit=nsplit, part_o=part_o,
                                  part_ml=part_ml, cos=cos, sin=sin, rot_dim=rot_dim,
                                  interleaved=interleaved, write_kv=call.write_cache and self.own_kv and not prepared,
-                                 token_rows=ctx.token_rows, **({} if prepared or not self.head_norm else dict(
+                                 token_rows=ctx.token_rows, values_are_keys=self.keys_serve_as_values, **({} if prepared or not self.head_norm else dict(
                                      q_gain=q_gain, k_gain=k_gain, eps=self.qk_norm_eps)), **common)
         else:
             on_matrix_cores = ctx.max_query_len > 1 and self._prefill_kernel(group.page_size, x_dtype)
@@ -441,7 +471,7 @@ class PagedAttention(Mixer):
                                       positions=ctx.positions, q_start=ctx.q_start, slots=ctx.slots,
                                       num_reqs=ctx.num_reqs, nh=self.num_heads, nkv=self.num_kv_heads,
                                       d=self.head_dim, dv=self.v_plane_dim, scale=self.scale, window=self.window,
-                                      slopes=self._slopes, chunk=self.chunk, sinks=sinks,
+                                      slopes=self._slopes, chunk=self.chunk, sinks=sinks, softcap=self.softcap, gate=gate,
                                       nsplit=nsplit, part_o=part_o, part_ml=part_ml,
                                       **(dict(cos=cos, sin=sin, rot_dim=rot_dim, interleaved=interleaved)
                                          if rotates else {}))

@@ -344,6 +344,10 @@ class Block(Part):
         slices = ctx.buffers.get("block_slices", ops.mid_slices_bound(H) * ops.MID_ROWS, H, torch.float32)
         return ops.ResidualSink(residual, gain[0], gain[1], rows, None, slices)
 
+    # the block's first sublayer reads the stream as it is: a block before it whose last kernel has the new
+    # stream in its registers may hand over those rows, in the model's dtype, as ``ops.NormedRows``
+    takes_stream = False
+
     # how many copies of every token's row the residual stream holds for this arrangement (the
     # model allocates ``[T, stream_copies * hidden]``; all blocks of a model agree)
     stream_copies = 1

@@ -139,28 +139,37 @@ class ParallelResidualBlock(Block):
         return None
 
 
+STREAM = (None, 0.0)  # in the place of a norm's (gain, eps): the rows of the stream as they are
+
+
 class SandwichNormBlock(Block):
     """A norm before and a norm behind each sublayer: ``r += post_mixer(mixer(pre_mixer(r)));
     r += post_ffn(ffn(pre_ffn(r)))``, all four RMS norms with a gain.  Between two sublayers the
     norm of the result, the sum into the float32 stream and the next sublayer's first norm are one
     kernel (``ops.norm_add_norm``); so the block hands the next block its first norm's rows where
     that block says it takes them (``input_gain``), and takes its own from the block before.  With
-    a feed-forward of kind ``none`` the layer is its first half."""
+    a feed-forward of kind ``none`` the layer is its first half.  ``pre_mixer`` and ``pre_ffn`` None: no
+    norm before the sublayers, which read the stream itself (rounded to the model's dtype): ``r +=
+    post_mixer(mixer(r)); r += post_ffn(ffn(r))``; the kernel between two sublayers then hands on the new
+    stream instead of its norm (``takes_stream``)."""
 
     def __init__(self, *, mixer: Mixer, ffn: FeedForward, norms: dict[str, Norm],
-                 mixer_name: str = "mixer", ffn_name: str = "mlp", pre_mixer: str = "norm1",
-                 post_mixer: str = "norm1b", pre_ffn: str = "norm2", post_ffn: str = "norm2b") -> None:
+                 mixer_name: str = "mixer", ffn_name: str = "mlp", pre_mixer: str | None = "norm1",
+                 post_mixer: str = "norm1b", pre_ffn: str | None = "norm2", post_ffn: str = "norm2b") -> None:
         super().__init__(mixer=mixer, ffn=ffn, norms=norms)
+        if (pre_mixer is None) != (pre_ffn is None):
+            raise ValueError("either both sublayers have a norm before them or neither has")
         self.mixer_only = bool(getattr(ffn, "absent", False))
         self.mixer_name, self.ffn_name = mixer_name, ffn_name
+        self.takes_stream = pre_mixer is None
         self.norm_names = (pre_mixer, post_mixer) if self.mixer_only else (pre_mixer, post_mixer, pre_ffn, post_ffn)
-        missing = [n for n in self.norm_names if n not in norms]
-        if missing or len(set(self.norm_names)) != len(self.norm_names):
-            raise ValueError(f"a block with norms on both sides of its sublayers needs {self.norm_names}; "
-                             f"given {list(norms)}")
+        named = [n for n in self.norm_names if n is not None]
+        missing = [n for n in named if n not in norms]
+        if missing or len(set(named)) != len(named):
+            raise ValueError(f"a block with norms behind its sublayers needs {named}; given {list(norms)}")
 
     def children(self) -> dict[str, Part]:
-        out: dict[str, Part] = {n: self.norms[n] for n in self.norm_names}
+        out: dict[str, Part] = {n: self.norms[n] for n in self.norm_names if n is not None}
         out[self.mixer_name] = self.mixer
         if not self.mixer_only:
             out[self.ffn_name] = self.ffn
@@ -169,7 +178,7 @@ class SandwichNormBlock(Block):
     def input_gain(self, scaled: bool = True):
         # finished rows are welcome; rows whose norm the mixer's first product would have to
         # finish are not (the mixers of such layers read their input more than once)
-        return None if scaled else self.norms[self.norm_names[0]].as_gain()
+        return None if scaled or self.takes_stream else self.norms[self.norm_names[0]].as_gain()
 
     def _gain(self, i: int):
         gain = self.norms[self.norm_names[i]].as_gain()
@@ -178,8 +187,8 @@ class SandwichNormBlock(Block):
         return gain
 
     def _join(self, result, residual, ctx, post, following, name: str):
-        """``residual += post(result)``, and the rows of the norm ``following`` (a (gain, eps) or
-        None) into the step buffer ``name``.  ``result`` is a tensor or the partial sums that a
+        """``residual += post(result)``, and the rows of the norm ``following`` (a (gain, eps), ``STREAM``
+        for the stream as it is, or None) into the step buffer ``name``.  ``result`` is a tensor or the partial sums that a
         part's last product left (``ops.SlicedRows``), or the results of a feed-forward's experts
         (``ops.WeightedRows``)."""
         post_gain, post_eps = post
@@ -207,14 +216,21 @@ class SandwichNormBlock(Block):
             x = delta.data  # the block before made this block's first norm
         else:
             x = ctx.buf("block_x", residual.shape[1])
-            self.norms[self.norm_names[0]].forward_fused(x, residual, delta)
-        following = next_block.input_gain(scaled=False) if next_block is not None else None
+            if self.takes_stream:
+                self.settle(delta, residual, ctx)
+                x.copy_(residual)
+            else:
+                self.norms[self.norm_names[0]].forward_fused(x, residual, delta)
+        following = None
+        if next_block is not None:
+            following = STREAM if next_block.takes_stream else next_block.input_gain(scaled=False)
+        inner = STREAM if self.takes_stream or self.mixer_only else self._gain(2)
         sink = self._slice_sink(self.mixer, residual, ctx)
         a = self.mixer.forward(x, ctx, call) if sink is None else self.mixer.forward(x, ctx, call, sink=sink)
         if self.mixer_only:
             rows = self._join(a, residual, ctx, self._gain(1), following, "block_x")
             return None if rows is None else ops.NormedRows(rows)
-        x2 = self._join(a, residual, ctx, self._gain(1), self._gain(2), "block_x2")
+        x2 = self._join(a, residual, ctx, self._gain(1), inner, "block_x2")
         sink = self._slice_sink(self.ffn, residual, ctx)
         if self.ffn.gives_weighted_rows:  # the norm behind the experts adds their results up
             f = self.ffn.forward_weighted(x2, ctx, call)

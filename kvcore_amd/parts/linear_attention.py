@@ -13,7 +13,13 @@ softplus(W_a h + dt_bias))``;
 
     S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q.
 
-Both finish alike: every head's ``o`` over its root mean square, times a gain of ``vdim`` values
+``LightningAttention``: ``q = silu(W_q h)``, ``k = silu(W_k h)``, ``v = silu(W_v h)``, one fixed decay per head;
+
+    S_t = decay S_(t-1) + k_t v_t^T,    o_t = S_t^T q_t;
+
+its heads are normed all together and gated by ``sigmoid(W_g h)``.
+
+The first two finish alike: every head's ``o`` over its root mean square, times a gain of ``vdim`` values
 shared by the heads, times ``silu(W_g h)``, then the output product.  The state (and the
 convolution's last ``taps - 1`` inputs) live in float32 slot arrays; a request starts from zeros
 at position 0.  Decays, gates, unit norms and the recurrence are float32; the products run in the
@@ -44,10 +50,15 @@ def _stacked(pairs: list[tuple[str, int]]) -> tuple[ParamSource, ...]:
 class _MatrixStateMixer(Mixer):
     """What the two mixers share: the sizes, the state, the head norm with its gate, the output."""
 
-    def _finish(self, o: torch.Tensor, gate: torch.Tensor, ctx) -> torch.Tensor:
+    def _finish(self, o: torch.Tensor, gate: torch.Tensor, ctx, sink=None, *, norm_heads: int | None = None,
+                act: str = "silu") -> torch.Tensor:
+        """The norm of every head (``norm_heads`` 1: of all heads at once), the gate, the output product."""
         p = self.params
         normed = ctx.buf(f"ms_normed:{self.inner}", self.inner)
-        ops.head_rmsnorm_gate(normed, o, gate, p["norm"], self.eps, self.heads, self.vdim)
+        heads = self.heads if norm_heads is None else norm_heads
+        ops.head_rmsnorm_gate(normed, o, gate, p["norm"], self.eps, heads, self.inner // heads, act=act)
+        if sink is not None:
+            return ops.linear(sink, normed, p["o.weight"])
         if self.float32_result:
             out = ctx.buf("mixer_out_f32", self.hidden_size, torch.float32)
         else:
@@ -275,6 +286,57 @@ class MaxGatedMatrixMemory(_MatrixStateMixer):
         return out
 
 
+class LightningAttention(_MatrixStateMixer):
+    """``heads`` heads with keys of ``dim`` and values of ``vdim``; ``decay`` a constant per head.
+    ``tensor_names`` renames checkpoint tensors (keys: q, k, v, g, o, norm)."""
+
+    def __init__(self, *, hidden_size: int, heads: int, dim: int, vdim: int, decay: tuple[float, ...], eps: float,
+                 tensor_names: dict[str, str] | None = None, float32_result: bool = False, position=None) -> None:
+        if min(heads, dim, vdim) <= 0 or len(decay) != heads:
+            raise ValueError(f"lightning attention needs positive sizes and a decay per head ({len(decay)} for {heads})")
+        self.hidden_size, self.heads, self.dim, self.vdim = hidden_size, heads, dim, vdim
+        self.decay, self.eps, self.float32_result = tuple(float(v) for v in decay), eps, float32_result
+        self.qk, self.inner = heads * dim, heads * vdim
+        self.names = {"q": "q.weight", "k": "k.weight", "v": "v.weight", "g": "g.weight", "o": "o.weight",
+                      "norm": "norm.weight", **(tensor_names or {})}
+
+    def param_specs(self) -> list[ParamSpec]:
+        n, H = self.names, self.hidden_size
+        return [
+            ParamSpec("in_proj.weight", (2 * self.qk + 2 * self.inner, H), sources=_stacked(
+                [(n["q"], self.qk), (n["k"], self.qk), (n["v"], self.inner), (n["g"], self.inner)])),
+            ParamSpec("norm", (self.inner,), kind="vector", init="gain", sources=_src(n["norm"], self.inner)),
+            ParamSpec("o.weight", (H, self.inner), sources=_src(n["o"], H)),
+        ]
+
+    def setup(self, runtime) -> None:
+        super().setup(runtime)
+        self._decay = torch.tensor([self.decay], dtype=torch.float32, device=runtime.device)
+
+    def product_weights(self) -> tuple[str, ...]:
+        return ("in_proj.weight", "o.weight")
+
+    @property
+    def takes_slice_sink(self) -> bool:
+        return self.inner % 8 == 0
+
+    def state_needs(self) -> tuple[StateNeed, ...]:
+        return (StateNeed((self.heads, ops.linear_state_rows(self.dim), self.vdim)),)
+
+    def forward(self, x, ctx, call, sink=None):
+        p, qk, inner = self.params, self.qk, self.inner
+        state = ctx.states[call.state_indices[0]]
+        width = 2 * qk + 2 * inner
+        proj = ctx.buf(f"la_proj:{width}", width, torch.float32)
+        ops.linear(proj, x, p["in_proj.weight"])
+        o = ctx.buf(f"ms_o:{inner}", inner, torch.float32)
+        ops.linear_state_scan(o, proj[:, :qk], proj[:, qk:2 * qk], proj[:, 2 * qk:2 * qk + inner], self._decay, None,
+                              state, heads=self.heads, qk_heads=self.heads, dim=self.dim, vdim=self.vdim,
+                              scalar_gates=True, silu_in=True, **self._batch(ctx))
+        return self._finish(o, proj[:, 2 * qk + inner:], ctx, sink, norm_heads=1, act="sigmoid")
+
+
+register_mixer("lightning_attention", LightningAttention)
 register_mixer("gated_linear_attention", GatedLinearAttention)
 register_mixer("max_gated_matrix_memory", MaxGatedMatrixMemory)
 register_mixer("gated_delta_rule", GatedDeltaRule)

@@ -87,5 +87,10 @@ def _register_builtin() -> None:
 
     register_architecture("Sopulorn", SopulornConfig.from_dict, sopulorn_spec)
 
+    from kvcore_amd.config.zikupel_config import ZikupelConfig
+    from kvcore_amd.models.zikupel import zikupel_spec
+
+    register_architecture("Zikupel", ZikupelConfig.from_dict, zikupel_spec)
+
 
 _register_builtin()
