@@ -255,6 +255,15 @@ int kvc_linear_state_scan(float* out, const float* q, int64_t q_stride, const fl
                           const int32_t* positions, const int32_t* token_req, const int32_t* q_start,
                           const int32_t* slots, int R, int nh, int nqk, int d, int dv, int delta_rule,
                           float q_scale, int ones_column, int silu_in, kvc_stream stream);
+// delta_rule 2 with a fixed decay per head (decay [nh], no beta) over portions of prompts, in chunks of
+// kvc_fixed_decay_chunk_tokens() tokens side by side (chunked_state.hip): the same results as the scan's, up to
+// the order of sums.  work: work_chunks >= min(T, T / chunk + R) chunks of nh * dpad * dv floats each.
+int kvc_fixed_decay_chunk_tokens(void);
+int kvc_fixed_decay_chunks(float* out, const float* q, int64_t q_stride, const float* k, int64_t k_stride,
+                           const float* v, int64_t v_stride, const float* decay, float* state, float* work,
+                           int64_t work_chunks, const int32_t* positions, const int32_t* token_req,
+                           const int32_t* q_start, const int32_t* slots, int T, int R, int nh, int nqk, int d,
+                           int dv, float q_scale, int silu_in, kvc_stream stream);
 // The gates of a matrix memory with log gates and a running maximum m (mLSTM), per request in
 // token order: i = cap tanh((i_raw + i_bias) / cap), f = logsigmoid(cap tanh((f_raw + f_bias) / cap)),
 // m_t = max(f + m_(t-1), i), keep[t, h] = exp(f + m_(t-1) - m_t), take[t, h] = exp(i - m_t),

@@ -62,6 +62,7 @@ def _declare(lib: ctypes.CDLL) -> None:
         "kvc_rope_kv_write": [P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, I, P],
         "kvc_paged_attention": [P, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, I, F, I, P, I, P, F, P, L, I, I, P],
         "kvc_linear_state_scan": [P, P, L, P, L, P, L, P, L, P, L, P, P, P, P, P, I, I, I, I, I, I, F, I, I, P],
+        "kvc_fixed_decay_chunks": [P, P, L, P, L, P, L, P, P, P, L, P, P, P, P, I, I, I, I, I, I, F, I, P],
         "kvc_sigmoid_power": [P, P, L, P, F, I, I, P],
         "kvc_decay_and_write_gates": [P, P, P, L, P, L, P, P, I, I, P],
         "kvc_unit_heads": [P, L, I, I, I, F, F, I, F, P],
@@ -123,6 +124,8 @@ def _declare(lib: ctypes.CDLL) -> None:
     lib.kvc_argmax_static_capacity.argtypes = []
     lib.kvc_ssm_scan_max_state.restype = c_int
     lib.kvc_ssm_scan_max_state.argtypes = []
+    lib.kvc_fixed_decay_chunk_tokens.restype = c_int
+    lib.kvc_fixed_decay_chunk_tokens.argtypes = []
     lib.kvc_rglru_scan_segment.restype = c_int
     lib.kvc_rglru_scan_segment.argtypes = []
 
@@ -1632,6 +1635,42 @@ def linear_state_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: to
         qk_heads, dim, vdim, 2 if scalar_gates else int(bool(delta_rule)), float(q_scale), int(bool(ones_column)),
         int(bool(silu_in)), _stream()),
         "kvc_linear_state_scan")
+
+
+def fixed_decay_chunk_count(tokens: int, num_reqs: int) -> int:
+    """The most chunks that ``fixed_decay_chunks`` cuts a step of ``tokens`` tokens into."""
+    return max(1, min(tokens, tokens // int(load().kvc_fixed_decay_chunk_tokens()) + num_reqs))
+
+
+def fixed_decay_chunks(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor,
+                       state: torch.Tensor, work: torch.Tensor, *, positions: torch.Tensor,
+                       token_req: torch.Tensor, q_start: torch.Tensor, slots: torch.Tensor, num_reqs: int,
+                       heads: int, qk_heads: int, dim: int, vdim: int, q_scale: float = 1.0,
+                       silu_in: bool = False) -> None:
+    """``linear_state_scan`` with ``scalar_gates``, no ``beta`` and one ``decay [1, heads]`` for every token, over
+    portions of prompts: chunks of tokens side by side (see the C header).  ``work``: float32, a row of
+    ``heads * linear_state_rows(dim) * vdim`` values for each of ``fixed_decay_chunk_count`` chunks."""
+    T = out.shape[0]
+    size = heads * linear_state_rows(dim) * vdim
+    if out.shape != (T, heads * vdim) or not out.is_contiguous() or out.dtype != torch.float32:
+        raise KernelError("fixed_decay_chunks: out must be contiguous float32 [T, heads * vdim]")
+    if tuple(state.shape[1:]) != (heads, linear_state_rows(dim), vdim) or state.dtype != torch.float32 \
+            or not state.is_contiguous():
+        raise KernelError("fixed_decay_chunks: state must be float32 [slots, heads, linear_state_rows(dim), vdim]")
+    if decay.numel() != heads or work.dim() != 2 or work.shape[1] != size or not work.is_contiguous():
+        raise KernelError("fixed_decay_chunks: a decay per head, and a workspace row per chunk")
+    if min(q.shape[0], k.shape[0], v.shape[0]) < T or positions.numel() < T or token_req.numel() < T \
+            or q_start.numel() < num_reqs + 1:
+        raise KernelError("fixed_decay_chunks: rows or index arrays too short")
+    qp, qs = _f32_rows(q, "q", qk_heads * dim)
+    kp, ks = _f32_rows(k, "k", qk_heads * dim)
+    vp, vs = _f32_rows(v, "v", heads * vdim)
+    f, i32 = torch.float32, torch.int32
+    _check(load().kvc_fixed_decay_chunks(
+        out.data_ptr(), qp, qs, kp, ks, vp, vs, _dev(decay, "decay", f), _dev(state, "state"), _dev(work, "work", f),
+        work.shape[0], _dev(positions, "positions", i32), _dev(token_req, "token_req", i32),
+        _dev(q_start, "q_start", i32), _dev(slots, "slots", i32), T, num_reqs, heads, qk_heads, dim, vdim,
+        float(q_scale), int(bool(silu_in)), _stream()), "kvc_fixed_decay_chunks")
 
 
 def sigmoid_power(out: torch.Tensor, z: torch.Tensor, bias: torch.Tensor | None, inv_tau: float) -> None:

@@ -35,6 +35,10 @@ from kvcore_amd.ops import library as ops
 from .base import Mixer, ParamSource, ParamSpec, StateNeed, register_mixer
 
 
+# from so many tokens of one request in a step on, lightning attention works in chunks
+CHUNKED_FROM = 48
+
+
 def _src(name: str, rows: int) -> tuple[ParamSource, ...]:
     return (ParamSource(name, 0, rows),)
 
@@ -330,9 +334,16 @@ class LightningAttention(_MatrixStateMixer):
         proj = ctx.buf(f"la_proj:{width}", width, torch.float32)
         ops.linear(proj, x, p["in_proj.weight"])
         o = ctx.buf(f"ms_o:{inner}", inner, torch.float32)
-        ops.linear_state_scan(o, proj[:, :qk], proj[:, qk:2 * qk], proj[:, 2 * qk:2 * qk + inner], self._decay, None,
-                              state, heads=self.heads, qk_heads=self.heads, dim=self.dim, vdim=self.vdim,
-                              scalar_gates=True, silu_in=True, **self._batch(ctx))
+        rows = (proj[:, :qk], proj[:, qk:2 * qk], proj[:, 2 * qk:2 * qk + inner])
+        sizes = dict(heads=self.heads, qk_heads=self.heads, dim=self.dim, vdim=self.vdim, silu_in=True)
+        if ctx.max_query_len >= CHUNKED_FROM:  # a portion of a prompt: chunks of tokens side by side
+            each = self.heads * ops.linear_state_rows(self.dim) * self.vdim
+            room = ctx.buffers
+            work = room.get(f"la_chunks:{each}", ops.fixed_decay_chunk_count(ctx.num_tokens, ctx.num_reqs), each,
+                            torch.float32, reserve=ops.fixed_decay_chunk_count(room.token_capacity, room.seq_capacity))
+            ops.fixed_decay_chunks(o, *rows, self._decay, state, work, **sizes, **self._batch(ctx))
+        else:
+            ops.linear_state_scan(o, *rows, self._decay, None, state, scalar_gates=True, **sizes, **self._batch(ctx))
         return self._finish(o, proj[:, 2 * qk + inner:], ctx, sink, norm_heads=1, act="sigmoid")
 
 
