@@ -20,7 +20,8 @@ Other workloads print a line of their own: ``--only-prefill``, ``--mixed`` (64 r
 with prompts of 16 to 2,048 tokens in portions of 512), ``--long-prompt N`` (time to the
 first token of one N-token prompt in portions of 2,048), ``--sweep`` (decode at further
 batch sizes and context lengths, a line each with its share of the memory bandwidth);
-``--model 1b|70b`` and ``--batch`` change the shape.  ``--sopulorn s|m`` times the Sopulorn decoder
+``--model 1b|70b`` and ``--batch`` change the shape.  ``--zikupel s|m`` times the Zikupel decoder
+beside the Sopulorn, the Vovalix and the Llama of equal width and depth.  ``--sopulorn s|m`` times the Sopulorn decoder
 beside the Vovalix and the Llama of equal width and depth.  ``--darovik s|m`` times the Darovik decoder
 beside the Tazunex, the Vovalix and the Llama of equal width and depth.  ``--tazunex s|m`` times the Tazunex
 decoder beside the Vovalix and the Llama of equal width and depth.  ``--vovalix s|m`` times the Vovalix
@@ -196,6 +197,44 @@ SOPULORN_SHAPES = {
 }
 
 
+def _zikupel_layers(n, width, heads, kv, ff, experts, top):
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": experts, "top": top}, "shared": {"ff": ff // 4}}
+    attention = {"type": "attention",
+                 "mixer": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 0.09, "softcap": 40.0,
+                           "rot": {"dims": 64, "base": 500000.0,
+                                   "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    lightning = {"type": "lightning",
+                 "mixer": {"heads": heads, "dim": 64, "vdim": 128,
+                           "decay": [1.0 - 2.0 ** (-1.0 - 8.0 * h / heads) for h in range(heads)]}}
+    return [dict(lightning if i % 4 == 3 else attention, mlp=moe if i else dense) for i in range(n)]
+
+
+# Zikupel at the layer sizes of a real model: of every four layers three attention (keys of 128 that are
+# the values too, capped scores, an output gate) and one lightning attention (keys of 64, values of 128, as
+# many heads as the Vovalix of the same width has in its linear attention); the first layer with the dense
+# feed-forward of the Llama of the same width, the rest with routed experts and a shared one in the numbers
+# and widths that the Sopulorn and the Vovalix of the same width have (without their gates' matrices)
+ZIKUPEL_SHAPES = {
+    "s": {"architecture": "Zikupel", "vocab": 32000, "width": 1024, "norm": {"eps": 1e-5},
+          "layers": _zikupel_layers(8, 1024, 8, 2, 4096, 16, 4)},
+    "m": {"architecture": "Zikupel", "vocab": 32000, "width": 2048, "norm": {"eps": 1e-5},
+          "layers": _zikupel_layers(16, 2048, 16, 4, 8192, 32, 4)},
+}
+
+
+def bench_zikupel(args) -> int:
+    """The workloads of ``bench_dirulorn`` for a Zikupel shape beside the Sopulorn of the same width and
+    depth (the closest model the engine has: attention with normed heads and routed experts, norms behind
+    sublayers), the Vovalix (a matrix state per head beside attention and routed experts) and the Llama."""
+    shapes = (ZIKUPEL_SHAPES[args.zikupel], SOPULORN_SHAPES[args.zikupel], VOVALIX_SHAPES[args.zikupel],
+              DIRULORN_SHAPES[args.zikupel][1])
+    names = (f"zikupel-{args.zikupel}", f"sopulorn-of-zikupel-{args.zikupel}", f"vovalix-of-zikupel-{args.zikupel}",
+             f"llama-of-zikupel-{args.zikupel}")
+    which = {"all": (0, 1, 2, 3), "zikupel": (0,), "sopulorn": (1,), "vovalix": (2,), "llama": (3,)}[args.zikupel_only]
+    return _bench_design(args, shapes, names, which, args.zikupel_workload)
+
+
 def bench_sopulorn(args) -> int:
     """The workloads of ``bench_dirulorn`` for a Sopulorn shape beside the Vovalix of the same width
     and depth (the closest model the engine has: routed experts and a shared one in every layer) and
@@ -361,6 +400,13 @@ def parse_args():
                    help="with --dirulorn: run one of the two models only (for profiling)")
     p.add_argument("--dirulorn-workload", default="all", choices=["all", "prefill", "decode8", "decode64"],
                    help="with --dirulorn: run one of the workloads only (for profiling)")
+    p.add_argument("--zikupel", default=None, choices=sorted(ZIKUPEL_SHAPES),
+                   help="instead of the default run: prefill and decode of the Zikupel decoder at this size, and "
+                        "of the Sopulorn, the Vovalix and the Llama of the same width and depth")
+    p.add_argument("--zikupel-only", default="all", choices=["all", "zikupel", "sopulorn", "vovalix", "llama"],
+                   help="with --zikupel: run one of the models only (for profiling)")
+    p.add_argument("--zikupel-workload", default="all", choices=["all", "prefill", "decode8", "decode64"],
+                   help="with --zikupel: run one of the workloads only (for profiling)")
     p.add_argument("--sopulorn", default=None, choices=sorted(SOPULORN_SHAPES),
                    help="instead of the default run: prefill and decode of the Sopulorn decoder at this size, and "
                         "of the Vovalix and the Llama of the same width and depth; a line each")
@@ -540,6 +586,8 @@ def main() -> int:
     if args.gpus != 1:
         print(f"bench.py: this engine runs on one GPU; --gpus {args.gpus} is not supported")
         return 2
+    if args.zikupel:
+        return bench_zikupel(args)
     if args.sopulorn:
         return bench_sopulorn(args)
     if args.darovik:
