@@ -82,7 +82,9 @@ constexpr int tile_bytes() {
 // W: waves of a block (4 or 8).  Eight waves stage each key tile for twice the rows, which
 // halves the block's loads and LDS writes per row; a compute unit then holds one block.
 // D: the size of a query and key head; DV: the size of a value head.
-template <int D, int DV, int CT, int KB, int W>
+// CAP_GATE: the scores may be softly capped and the results gated (instances of their own: the others keep
+// their registers).
+template <int D, int DV, int CT, int KB, int W, int CAP_GATE>
 __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ q, int64_t q_stride,
     const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
@@ -108,7 +110,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
   // cap_rate > 0: raw scores become capped_unit(raw, cap_rate), numbers between -1 and 1, and scale_log2e is
   // the cap in the exponent's units.  The exponents are then bounded, so with a cap of up to 44 no maximum
   // is looked for: the sums stay relative to a score of zero (weights of at most 2^64).
-  const bool bounded = cap_rate > 0.f && scale_log2e <= kBoundedLog2;
+  const bool bounded = CAP_GATE && cap_rate > 0.f && scale_log2e <= kBoundedLog2;
   // Workgroups go to the chip's eight dies in turn (workgroup id modulo 8) and every die has
   // an L2 of its own, while all blocks of a kv head read the same keys and values.  So a kv
   // head's blocks get ids that land on one die (with fewer than eight kv heads, on 8 / nkv
@@ -516,7 +518,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
             s[ct][kbi][i] = __builtin_fmaf(-my_slope[ct], d0 - static_cast<float>(16 * kbi + i), s[ct][kbi][i]);
       }
     }
-    if (cap_rate > 0.f) {  // scalar
+    if (CAP_GATE && cap_rate > 0.f) {  // scalar
 #pragma unroll
       for (int ct = 0; ct < CT; ++ct)
 #pragma unroll
@@ -655,7 +657,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
     }
     const float inv = (l_row > 0.f) ? 1.f / l_row : 0.f;
     const int64_t at = (static_cast<int64_t>(my_tok[ct]) * nh + my_head[ct]) * DV + 4 * quad;
-    if (gate.gate != nullptr) {  // scalar: times the sigmoid of the gate's rows, four values of a head at a time
+    if (CAP_GATE && gate.gate != nullptr) {  // scalar: times the sigmoid of the gate's rows, four values of a head at a time
       const bf16_t* gp = gate.gate + my_tok[ct] * gate.stride + static_cast<int64_t>(my_head[ct]) * DV + 4 * quad;
 #pragma unroll
       for (int j = 0; j < NJ; ++j) {
@@ -683,7 +685,7 @@ __global__ __launch_bounds__(W * 64, (W == 4) ? 2 : 1) void prefill_attention_ke
   }  // turn
 }
 
-template <int D, int DV, int CT, int W>
+template <int D, int DV, int CT, int W, int CAP_GATE>
 int launch_prefill_ct(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t* k_cache,
                       const bf16_t* v_cache, const int32_t* table, int table_stride,
                       const int32_t* positions, const int32_t* q_start, const int32_t* slots, int T,
@@ -706,7 +708,7 @@ int launch_prefill_ct(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16
   constexpr int KB = (W == 8 || DV < 64) ? 8 : 4;
   constexpr int lds_bytes = 2 * tile_bytes<D, DV, KB>();
   static const hipError_t attr = hipFuncSetAttribute(
-      reinterpret_cast<const void*>(&prefill_attention_kernel<D, DV, CT, KB, W>),
+      reinterpret_cast<const void*>(&prefill_attention_kernel<D, DV, CT, KB, W, CAP_GATE>),
       hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);
   if (attr != hipSuccess) return kvc_fail("kvc_prefill_attention: the kernel's LDS size was refused");
   // see the kernel on how block ids map to (kv head, pair)
@@ -717,7 +719,7 @@ int launch_prefill_ct(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16
   snprintf(variant, sizeof(variant), "prefill_attention_kernel<%d,%d,%d,%d>%s x%d", D, CT, KB, W,
            single ? " one tile a block" : "", nsplit);
   kvc_note_variant(kVariantPrefillAttention, variant);
-  hipLaunchKernelGGL((prefill_attention_kernel<D, DV, CT, KB, W>), dim3(static_cast<unsigned>(wide), 1, nsplit), dim3(W * 64),
+  hipLaunchKernelGGL((prefill_attention_kernel<D, DV, CT, KB, W, CAP_GATE>), dim3(static_cast<unsigned>(wide), 1, nsplit), dim3(W * 64),
                      lds_bytes, stream, out, q, q_stride, k_cache, v_cache, table, table_stride, positions,
                      q_start, slots, R, nh, nkv, page_size, num_pages, (softcap > 0.f ? softcap : scale) * kLog2e, window,
                      slopes, chunk, sinks, part_o, part_ml, single, cos_tab, sin_tab, rot_dim, interleaved,
@@ -791,7 +793,9 @@ int launch_prefill(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t*
   if (DV < 64) waves = 4;  // eight waves would stage the values of more key blocks than a tile has
   if (g > 16 * waves * ct) return kvc_fail("kvc_prefill_attention: too many query heads per kv head");
 #define KVC_LAUNCH_PREFILL(CT_, W_)                                                                      \
-  return launch_prefill_ct<D, DV, CT_, W_>(out, q, q_stride, k_cache, v_cache, table, table_stride, positions, \
+  return softcap > 0.f || gate.gate != nullptr ? LAUNCH_WITH(CT_, W_, 1) : LAUNCH_WITH(CT_, W_, 0)
+#define LAUNCH_WITH(CT_, W_, CAP_GATE_)                                                                  \
+  launch_prefill_ct<D, DV, CT_, W_, CAP_GATE_>(out, q, q_stride, k_cache, v_cache, table, table_stride, positions, \
                                        q_start, slots, T, R, nh, nkv, page_size, num_pages, scale, window, \
                                        slopes, chunk, sinks, part_o, part_ml, nsplit, single, cos_tab, sin_tab, rot_dim,     \
                                        interleaved, softcap, gate, out_f32, stream)
@@ -804,6 +808,7 @@ int launch_prefill(bf16_t* out, const bf16_t* q, int64_t q_stride, const bf16_t*
   if (ct == 2) KVC_LAUNCH_PREFILL(2, 4);
   KVC_LAUNCH_PREFILL(1, 4);
 #undef KVC_LAUNCH_PREFILL
+#undef LAUNCH_WITH
 }
 
 }  // namespace

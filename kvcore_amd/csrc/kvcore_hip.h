@@ -248,7 +248,7 @@ int kvc_gated_group_rmsnorm(void* out, int out_dtype, const float* y, const void
 // beta are float32 rows with strides.  d at most 256.  With ones_column the rows of v hold dv - 1
 // values a head and column dv - 1 of every head takes a one for each token: a normaliser that is
 // gated and read like the matrix, out[t, h, dv - 1] being its product with the query.  silu_in: q, k and v
-// pass through silu on their way in (q before its scale).
+// pass through silu on their way in (q before its scale; delta_rule 2 without beta only).
 int kvc_linear_state_scan(float* out, const float* q, int64_t q_stride, const float* k,
                           int64_t k_stride, const float* v, int64_t v_stride, const float* decay,
                           int64_t decay_stride, const float* beta, int64_t beta_stride, float* state,

@@ -57,6 +57,8 @@ __device__ __forceinline__ float group_sum(float v) {
   return v;
 }
 
+// DELTA: 0 key decay, 1 the delta rule or scalar gates, 2 scalar gates without beta, with silu on the way in
+// where asked (an instance of its own: the others keep their registers).
 template <int NPT, int DELTA, int NSL, int FULL, int PF>
 __global__ __launch_bounds__(256) void linear_state_scan_kernel(
     float* __restrict__ out, const float* __restrict__ q, int64_t q_stride, const float* __restrict__ k,
@@ -69,7 +71,8 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
   // with ones_column the rows of v hold dv - 1 values a head and the last column of the state's dv
   // takes a one for every token (a normaliser kept beside the matrix)
   const int dvin = dv - ones_column;
-  auto take_in = [&](float x) -> float { return silu_in ? silu_of(x) : x; };
+  // (tokens that a stage does not have are left alone: whole waves skip the work)
+  auto take_in = [&](float x, bool there) -> float { return DELTA == 2 && silu_in && there ? silu_of(x) : x; };
   // FULL: d == NPT * NSL, so no row needs a bound, and a thread's rows of q, k and the factors lie
   // side by side in LDS (row n of a token at (n % NSL) * NPT + n / NSL), read 16 bytes at a time
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -121,7 +124,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       constexpr int ST = FULL ? 1 : NSL;  // from one of the thread's rows to its next, in LDS
       const float vv = v_s[tt * VT + pl];
       float acc = 0.f;
-      if (DELTA && scalar_gates) {  // the same for the whole grid: S <- g S + (beta k) v^T
+      if (DELTA == 2 || (DELTA && scalar_gates)) {  // the same for the whole grid: S <- g S + (beta k) v^T
         const float g = a_s[2 * tt], bv = a_s[2 * tt + 1] * vv;
         float acc1 = 0.f;
 #pragma unroll
@@ -210,20 +213,20 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       for (int j = 0; j < QN; ++j) {
         const int idx = tid + 256 * j, tt = idx / d, n = idx - tt * d;
         const int64_t t = t0 + (tt < nt ? tt : 0);
-        qn[j] = take_in(q[t * q_stride + hk * d + n]) * q_scale;
-        kn[j] = take_in(k[t * k_stride + hk * d + n]);
+        qn[j] = take_in(q[t * q_stride + hk * d + n], tt < nt) * q_scale;
+        kn[j] = take_in(k[t * k_stride + hk * d + n], tt < nt);
         if (!DELTA) an[j] = decay[t * decay_stride + h * d + n];
       }
       if (DELTA) {
         const int64_t t = t0 + (tid < nt ? tid : 0);
         an[0] = decay[t * decay_stride + h];
-        an[1] = beta != nullptr ? beta[t * beta_stride + h] : 1.f;
+        an[1] = DELTA == 2 ? 1.f : beta[t * beta_stride + h];
       }
 #pragma unroll
       for (int j = 0; j < VN; ++j) {
         const int idx = tid + 256 * j, tt = idx / VT, cc = c0 + idx - tt * VT;
         const int64_t t = t0 + (tt < nt ? tt : 0);
-        vn[j] = cc < dvin ? take_in(v[t * v_stride + h * dvin + cc]) : (cc < dv ? 1.f : 0.f);
+        vn[j] = cc < dvin ? take_in(v[t * v_stride + h * dvin + cc], tt < nt) : (cc < dv ? 1.f : 0.f);
       }
     };
     auto stash = [&](float* base) {
@@ -272,19 +275,19 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         const int tt = idx / d, n = idx - tt * d;
         const int64_t t = t0 + tt;
         const int at = FULL ? tt * d + (n % NSL) * NPT + n / NSL : idx;
-        q_s[at] = take_in(q[t * q_stride + hk * d + n]) * q_scale;
-        k_s[at] = take_in(k[t * k_stride + hk * d + n]);
+        q_s[at] = take_in(q[t * q_stride + hk * d + n], true) * q_scale;
+        k_s[at] = take_in(k[t * k_stride + hk * d + n], true);
         if (!DELTA) a_s[at] = decay[t * decay_stride + h * d + n];
       }
       if (DELTA) {
         for (int tt = tid; tt < nt; tt += nthreads) {
           a_s[2 * tt] = decay[static_cast<int64_t>(t0 + tt) * decay_stride + h];
-          a_s[2 * tt + 1] = beta != nullptr ? beta[static_cast<int64_t>(t0 + tt) * beta_stride + h] : 1.f;
+          a_s[2 * tt + 1] = DELTA == 2 ? 1.f : beta[static_cast<int64_t>(t0 + tt) * beta_stride + h];
         }
       }
       for (int idx = tid; idx < nt * VT; idx += nthreads) {
         const int tt = idx / VT, cc = c0 + idx - tt * VT;
-        v_s[idx] = cc < dvin ? take_in(v[static_cast<int64_t>(t0 + tt) * v_stride + h * dvin + cc]) : (cc < dv ? 1.f : 0.f);
+        v_s[idx] = cc < dvin ? take_in(v[static_cast<int64_t>(t0 + tt) * v_stride + h * dvin + cc], true) : (cc < dv ? 1.f : 0.f);
       }
       __syncthreads();
       work_stage(q_s, k_s, a_s, v_s, t0, nt);
@@ -579,6 +582,8 @@ extern "C" int kvc_linear_state_scan(float* out, const float* q, int64_t q_strid
   if (rule < 0 || rule > 2) return kvc_fail("kvc_linear_state_scan: the rule is 0 (key decay), 1 (delta) or 2 (scalar gates)");
   const int delta_rule = rule != 0;  // a gate and a factor per head and token instead of a decay per key channel
   const int scalar_gates = rule == 2;
+  const bool fixed_gates = scalar_gates && beta == nullptr;
+  if (silu_in && !fixed_gates) return kvc_fail("kvc_linear_state_scan: silu on the way in goes with scalar gates without beta");
   if (R < 0 || nh <= 0 || nqk <= 0 || nh % nqk || d <= 0 || dv <= 0)
     return kvc_fail("kvc_linear_state_scan: bad sizes");
   if (d > 256) return kvc_fail("kvc_linear_state_scan: at most 256 key channels a head");
@@ -618,7 +623,11 @@ extern "C" int kvc_linear_state_scan(float* out, const float* q, int64_t q_strid
   } while (0)
 #define KVC_LSCAN_N(NPT)                 \
   do {                                   \
-    if (delta_rule && narrow) {          \
+    if (fixed_gates && narrow) {         \
+      KVC_LSCAN(NPT, 2, 16);             \
+    } else if (fixed_gates) {            \
+      KVC_LSCAN(NPT, 2, 4);              \
+    } else if (delta_rule && narrow) {   \
       KVC_LSCAN(NPT, 1, 16);             \
     } else if (delta_rule) {             \
       KVC_LSCAN(NPT, 1, 4);              \

@@ -1598,7 +1598,7 @@ def linear_state_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: to
     ``v [T, heads * vdim]``, all float32 rows (column views are fine); ``decay [T, heads * dim]``
     (a factor per key channel) or, with ``delta_rule``, ``decay`` and ``beta [T, heads]``; with
     ``scalar_gates`` the rule is ``S <- decay S + beta k v^T`` with the same two ``[T, heads]`` (``beta`` None:
-    ones; ``decay [1, heads]``: the same for every token); ``silu_in``: q, k and v pass through silu first;
+    ones; ``decay [1, heads]``: the same for every token); ``silu_in`` (without ``beta``): q, k and v pass through silu first;
     with ``ones_column`` ``v`` is ``[T, heads * (vdim - 1)]`` and the last of a head's ``vdim``
     columns takes a one for every token (a normaliser beside the matrix);
     ``state [slots, heads, linear_state_rows(dim), vdim]`` float32, in an order of the kernel's own;

@@ -60,6 +60,9 @@ def rotary_inv_freq(rot_dim: int, theta: float, scaling: dict | None = None) -> 
         inv_freq = torch.where(wavelen < orig / high, inv_freq,
                                torch.where(wavelen > orig / low, inv_freq / factor, blended))
     elif rope_type == "yarn":
+        missing = [k for k in ("factor", "original", "fast", "slow") if k not in scaling]
+        if missing:
+            raise ValueError(f"rope_type 'yarn' needs {missing}")
         ramp = yarn_ramp(rot_dim, float(theta), *(float(scaling[k]) for k in ("original", "fast", "slow")))
         inv_freq = inv_freq / float(scaling["factor"]) * ramp + inv_freq * (1.0 - ramp)
     elif rope_type != "default":
