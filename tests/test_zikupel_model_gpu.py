@@ -197,6 +197,10 @@ def test_unequal_requests_side_by_side_with_slots_used_again(models, name, dtype
         [("b", 15), ("d", 1)], [("d", 14), ("e", 2)], [("f", 1)],
     ]
     compare(replay(s, seqs, plan), want, dtype, excused=3)
+    # portions long enough for chunks beside single tokens and short portions
+    three = {k: seqs[k] for k in "abd"}
+    plan = [[("b", 20)], [("a", 50), ("b", 1), ("d", 2)], [("b", 11), ("a", 11), ("d", 1)], [("d", 44), ("b", 1)]]
+    compare(replay(s, three, plan), want, dtype, excused=3)
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=IDS)
